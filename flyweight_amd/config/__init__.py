@@ -5,6 +5,7 @@ from .koketar import KoketarConfig
 from .vavelorn import VavelornConfig
 from .dalerax import DaleraxConfig
 from .telapel import TelapelConfig
+from .zaluvik import ZaluvikConfig
 from .registry import (architecture_name, config_from_dict, load_config,
                        register_architecture, registered_architectures)
 
@@ -14,9 +15,10 @@ register_architecture("Koketar", KoketarConfig)
 register_architecture("Vavelorn", VavelornConfig)
 register_architecture("Dalerax", DaleraxConfig)
 register_architecture("Telapel", TelapelConfig)
+register_architecture("Zaluvik", ZaluvikConfig)
 
 __all__ = [
     "ConfigError", "LayerSpec", "ModelSpec", "PartSpec", "ScheduleEntry", "default_schedule",
-    "Lfm2Config", "KoketarConfig", "VavelornConfig", "DaleraxConfig", "TelapelConfig", "architecture_name", "config_from_dict", "load_config",
+    "Lfm2Config", "KoketarConfig", "VavelornConfig", "DaleraxConfig", "TelapelConfig", "ZaluvikConfig", "architecture_name", "config_from_dict", "load_config",
     "register_architecture", "registered_architectures",
 ]

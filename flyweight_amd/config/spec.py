@@ -63,11 +63,12 @@ class ScheduleEntry:
     mixer uses during this execution; two entries with the same ``cache`` share
     keys/values or state, and only the one with ``writes_cache`` appends to it.
     A layer may be named by several entries (it then runs several times with the
-    same weights)."""
+    same weights). ``joins_input``: the model's ``input_join`` runs right ahead of this execution."""
 
     layer: int
     cache: Optional[int] = None
     writes_cache: bool = True
+    joins_input: bool = False
 
 
 @dataclass(frozen=True)
@@ -90,6 +91,9 @@ class ModelSpec:
     logit_softcap: float = 0.0
     # a table [max_positions, hidden] of learned vectors, one per position, added to the embedding rows (None: none)
     position_table_name: Optional[str] = None
+    # a map of the residual stream and the embedding output that replaces the stream ahead of the schedule entries that
+    # say so (None: there is none; see parts/input_join.py)
+    input_join: Optional[PartSpec] = None
 
     def validate(self) -> None:
         if self.hidden_size <= 0 or self.vocab_size <= 0:
@@ -98,6 +102,8 @@ class ModelSpec:
             raise ConfigError("logit_softcap must not be negative (0 switches it off)")
         if not self.layers or not self.schedule:
             raise ConfigError("a model needs at least one layer and one schedule entry")
+        if any(entry.joins_input for entry in self.schedule) and self.input_join is None:
+            raise ConfigError("a schedule entry joins the model's input, but the model has no map for it")
         writers = {}
         for index, entry in enumerate(self.schedule):
             if not 0 <= entry.layer < len(self.layers):

@@ -169,7 +169,7 @@ __global__ __launch_bounds__(64) void qk_norm_rope_kv_write_rows_kernel(
     }
 }
 
-extern "C" int fw_qk_norm_rope_kv_write(const void* qkv, int in_dtype, void* q_out, int dtype, const float* q_norm_weight,
+extern "C" int fw_qk_norm_rope_kv_write(const void* qkv, int in_dtype, int row_stride, void* q_out, int dtype, const float* q_norm_weight,
                                         const float* k_norm_weight, float eps, const float* cos_table,
                                         const float* sin_table, int rotary_dim, void* k_pages, void* v_pages,
                                         const int32_t* block_table, int table_stride, const int32_t* row_seg,
@@ -188,7 +188,9 @@ extern "C" int fw_qk_norm_rope_kv_write(const void* qkv, int in_dtype, void* q_o
     if (rows == 0) return 0;
     FW_REQUIRE(!(q_only && write_kv), "qk_norm_rope: rows that hold queries only bring no keys or values to store");
     const int vectors = write_kv ? num_heads + 2 * num_kv_heads : num_heads;
-    const int width = q_only ? num_heads * head_dim : (num_heads + num_kv_heads) * head_dim + num_kv_heads * v_dim;
+    const int needed = q_only ? num_heads * head_dim : (num_heads + num_kv_heads) * head_dim + num_kv_heads * v_dim;
+    const int width = row_stride > 0 ? row_stride : needed;      // rows may hold more behind the values
+    FW_REQUIRE(width >= needed, "qk_norm_rope: rows %d wide do not hold %d", width, needed);
     FW_REQUIRE(vectors <= 65535, "qk_norm_rope: too many heads (%d)", vectors);
     dim3 grid(rows, vectors);
     hipStream_t s = (hipStream_t)stream;

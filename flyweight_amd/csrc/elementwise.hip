@@ -16,7 +16,7 @@ void fw_set_error(const char* format, ...) {
     va_end(args);
 }
 extern "C" const char* fw_last_error(void) { return fw_error_text; }
-extern "C" int fw_abi_version(void) { return 16; }
+extern "C" int fw_abi_version(void) { return 17; }
 
 // ---- embedding -------------------------------------------------------------------------
 // The reference gathers one row per token and widens it to float32
@@ -409,12 +409,12 @@ extern "C" int fw_fill_zero(void* ptr, long long bytes, void* stream) {
     return 0;
 }
 
-// ---- layer norm with a weight and no bias -----------------------------------------------------------
-// out[r] = (x[src] - mean) / sqrt(mean((x[src] - mean)^2) + eps) * w, src = row_index ? row_index[r] : r.
+// ---- layer norm with a weight and an optional bias ---------------------------------------------------
+// out[r] = (x[src] - mean) / sqrt(mean((x[src] - mean)^2) + eps) * w (+ bias), src = row_index ? row_index[r] : r.
 // The mean first, then the mean of the squared deviations from it (not E[x^2] - mean^2, which loses
 // digits where the mean is large beside the spread). A row of up to 4,096 values stays in registers.
 template <typename T>
-__global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __restrict__ x, const float* __restrict__ weight,
+__global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __restrict__ x, const float* __restrict__ weight, const float* __restrict__ bias,
                                                              T* __restrict__ out, const int32_t* __restrict__ row_index,
                                                              int hidden, float eps) {
     __shared__ float scratch[16];
@@ -453,23 +453,28 @@ __global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __rest
 #pragma unroll
         for (int u = 0; u < 16; ++u) {
             const int i = threadIdx.x + 256 * u;
-            if (i < hidden) store_from_float(out, (size_t)row * hidden + i, (held[u] - mean) * inv * scale[u]);
+            if (i < hidden) {
+                const float normed = (held[u] - mean) * inv * scale[u];
+                store_from_float(out, (size_t)row * hidden + i, bias ? normed + bias[i] : normed);
+            }
         }
     } else {
-        for (int i = threadIdx.x; i < hidden; i += 256)
-            store_from_float(out, (size_t)row * hidden + i, (source[i] - mean) * inv * weight[i]);
+        for (int i = threadIdx.x; i < hidden; i += 256) {
+            const float normed = (source[i] - mean) * inv * weight[i];
+            store_from_float(out, (size_t)row * hidden + i, bias ? normed + bias[i] : normed);
+        }
     }
 }
 
-extern "C" int fw_layernorm_rows(const float* x, const float* weight, void* out, int out_dtype, const int32_t* row_index,
+extern "C" int fw_layernorm_rows(const float* x, const float* weight, const float* bias, void* out, int out_dtype, const int32_t* row_index,
                                  int rows, int hidden, float eps, void* stream) {
     FW_REQUIRE(rows >= 0 && hidden > 0, "layernorm_rows: bad sizes rows=%d hidden=%d", rows, hidden);
     FW_REQUIRE(eps > 0.0f, "layernorm_rows: eps must be positive");
     if (rows == 0) return 0;
     if (out_dtype == FW_F32)
-        layernorm_rows_kernel<float><<<rows, 256, 0, (hipStream_t)stream>>>(x, weight, (float*)out, row_index, hidden, eps);
+        layernorm_rows_kernel<float><<<rows, 256, 0, (hipStream_t)stream>>>(x, weight, bias, (float*)out, row_index, hidden, eps);
     else if (out_dtype == FW_BF16)
-        layernorm_rows_kernel<bf16_t><<<rows, 256, 0, (hipStream_t)stream>>>(x, weight, (bf16_t*)out, row_index, hidden, eps);
+        layernorm_rows_kernel<bf16_t><<<rows, 256, 0, (hipStream_t)stream>>>(x, weight, bias, (bf16_t*)out, row_index, hidden, eps);
     else
         FW_REQUIRE(false, "layernorm_rows: unknown out dtype %d", out_dtype);
     FW_LAUNCH_CHECK("layernorm_rows");

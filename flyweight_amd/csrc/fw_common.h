@@ -169,6 +169,23 @@ __device__ __forceinline__ float fw_gated_unit(float g, float u, float limit, fl
     return g * (z >= 0.0f ? 1.0f / (1.0f + e) : e / (1.0f + e)) * (u + shift);
 }
 
+// z Phi(z), Phi the normal distribution's cumulative function: the exact gelu
+__device__ __forceinline__ float fw_gelu(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+
+// A product that stores gelu(sum) in bfloat16 is the storing product with this output type (dtype code
+// FW_BF16_GELU): the unit is formed from the float32 sum and rounded once.
+#define FW_BF16_GELU 2
+struct gelu_bf16_t {
+    uint16_t bits;
+};
+template <> __device__ __forceinline__ float load_as_float<gelu_bf16_t>(const gelu_bf16_t* p, size_t i) { return bf16_bits_to_float(p[i].bits); }
+template <> __device__ __forceinline__ void store_from_float<gelu_bf16_t>(gelu_bf16_t* p, size_t i, float v) {
+    p[i].bits = float_to_bf16_bits(fw_gelu(v));
+}
+// what a store of this output type does to a float32 sum before it is rounded (for stores that pack several values)
+template <typename T> __device__ __forceinline__ float fw_before_store(float v) { return v; }
+template <> __device__ __forceinline__ float fw_before_store<gelu_bf16_t>(float v) { return fw_gelu(v); }
+
 // The first key that a row at position `pos` may see: with a window the last `window` keys (itself
 // among them), with a chunk only the keys of its own chunk (chunks counted from position 0 of the
 // sequence); 0 switches either off. Never falls as the position rises.

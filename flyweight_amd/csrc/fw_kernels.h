@@ -35,7 +35,8 @@ int fw_gemm_generic(const void* a, int a_dtype, const void* w, int w_dtype, cons
                     void* out, int out_dtype, int out_mode, int M, int N, int K, void* stream);
 
 // bfloat16 matrix products on the matrix cores, float32 accumulation. a [M][K], w [N][K], K a
-// multiple of 8. mode 0: out = a . w^T (+ bias) stored as out_dtype; mode 1: out (float32) +=
+// multiple of 8. mode 0: out = a . w^T (+ bias) stored as out_dtype (also 2, here and in every storing product below:
+// gelu(a . w^T (+ bias)), the error-function form, in bfloat16); mode 1: out (float32) +=
 // a . w^T (+ bias); mode 2 (SwiGLU): w is [2N][K], gate rows then up rows, out [M][N] bfloat16 =
 // silu(a . gate^T) * (a . up^T). fw_gemm_skinny streams w once for M <= 64 (decode);
 // fw_gemm_mfma tiles both operands through LDS (prompts).
@@ -131,7 +132,7 @@ int fw_shortconv(const void* bcx, int in_dtype, void* out, int out_dtype, const 
 // 1: channel 2i with channel 2i + 1; the tables are the same), q out, k and v appended to the pages of
 // the row's segment. qkv [rows][(nh + nkv) hd + nkv vd]: values may have a size vd of their own.
 // k_pages [pages][nkv][P][hd]; v_pages [pages][nkv][vd][P]. block_table [segments][table_stride].
-int fw_qk_norm_rope_kv_write(const void* qkv, int in_dtype, void* q_out, int dtype, const float* q_norm_weight,
+int fw_qk_norm_rope_kv_write(const void* qkv, int in_dtype, int row_stride, void* q_out, int dtype, const float* q_norm_weight,
                              const float* k_norm_weight, float eps, const float* cos_table,
                              const float* sin_table, int rotary_dim, void* k_pages, void* v_pages,
                              const int32_t* block_table, int table_stride, const int32_t* row_seg,
@@ -194,6 +195,35 @@ int fw_attention_decode_fused(const float* qkv, const float* q_norm_weight, cons
                               float scale, int window, int chunk, float softcap, int interleaved, int q_only, int keep_first,
                               const float* sinks, const float* slopes, const float* q_row_scale, int page_size, int num_pages, void* stream);
 
+// ---- attention whose weights are sigmoids and whose heads mix them ---------------------------------
+// a_g(i, j) = sigmoid(q_g . k * scale + bias[g]) for the visible keys j of row i (the last `window`; 0: all), each on its own;
+// out_h(i) = sigmoid(gate[i][h v_dim ..]) * sum_j (sum_g mix[h][g] a_g(i, j)) v_j, v of h's key/value head. bias [heads],
+// mix [heads][heads], gate [rows][gate_stride] (null: none) float32; pages and batch arrays as above.
+// The plain kernel takes up to 256 heads of up to 1,024 channels, float32 or bfloat16.
+int fw_sigmoid_attention_generic(const void* q, void* out, int dtype, const void* k_pages, const void* v_pages,
+                                 const int32_t* block_table, int table_stride, const int32_t* row_seg, const int32_t* row_pos,
+                                 int rows, int num_heads, int num_kv_heads, int head_dim, int v_dim, float scale, int window,
+                                 const float* bias, const float* mix, const float* gate, int gate_stride, int page_size,
+                                 int num_pages, void* stream);
+// The matrix-core kernels (bfloat16): whether they take these sizes (up to 16 heads, channels in steps of 16 up to 256).
+int fw_sigmoid_attention_fits(int num_heads, int head_dim, int v_dim);
+// Prompt portions; tiles as for fw_attention_prefill.
+int fw_sigmoid_attention_prefill(const void* q, void* out, const void* k_pages, const void* v_pages, const int32_t* block_table,
+                                 int table_stride, const int32_t* tile_seg, const int32_t* tile_row0, int tiles,
+                                 const int32_t* seg_row0, const int32_t* row_pos, int rows, int num_heads, int num_kv_heads,
+                                 int head_dim, int v_dim, float scale, int window, const float* bias, const float* mix,
+                                 const float* gate, int gate_stride, int page_size, int num_pages, void* stream);
+// One row per request: from finished bfloat16 queries q, or (q null) from the raw projections qkv (float32 rows of qkv_stride:
+// q | k | v), whose queries and keys are divided by their root mean square per head (qk_norm; eps under the root) and whose
+// keys and values are stored first (write_kv). max_splits workgroups of pages_per_split pages cover what a row sees;
+// partial: float32 [rows][max_splits][heads * v_dim]; tickets: an int32 per row, zero before and after.
+int fw_sigmoid_attention_decode(const void* q, const float* qkv, int qkv_stride, int qk_norm, float eps, int write_kv, void* out,
+                                float* partial, int max_splits, int pages_per_split, int max_context, int* tickets,
+                                int tickets_len, void* k_pages, void* v_pages, const int32_t* block_table, int table_stride,
+                                const int32_t* row_seg, const int32_t* row_pos, int rows, int num_heads, int num_kv_heads,
+                                int head_dim, int v_dim, float scale, int window, const float* bias, const float* mix,
+                                const float* gate, int gate_stride, int page_size, int num_pages, void* stream);
+
 // ids[r] = argmax(logits[r]) with ties to the lowest id, also written to also[r] if that is not null;
 // advance[r] += 1 if that is not null; workspace: rows * 64 64-bit words
 int fw_argmax_rows(const float* logits, int32_t* ids, int32_t* also, int32_t* advance, void* workspace, int rows, int vocab,
@@ -221,7 +251,7 @@ int fw_sample_rows(const float* logits, const float* settings, unsigned long lon
 
 // Layer norm with a weight and no bias: out[r] = (x[src] - mean) / sqrt(mean((x[src] - mean)^2) + eps) * w,
 // src = row_index ? row_index[r] : r.
-int fw_layernorm_rows(const float* x, const float* weight, void* out, int out_dtype, const int32_t* row_index,
+int fw_layernorm_rows(const float* x, const float* weight, const float* bias, void* out, int out_dtype, const int32_t* row_index,
                       int rows, int hidden, float eps, void* stream);
 
 // out[r][j] = gelu_tanh(z[r][j]) * table[ids[r]][col0 + j] for j < width; z float32 [rows][z_stride],
@@ -268,13 +298,18 @@ int fw_gated_head_norm(const float* o, const void* gate, int gate_dtype, int gat
 int fw_norm_scale_add(float* x, const float* a, const float* b, float scale_a, float scale_b, const float* weight,
                       int one_centered, float eps, float mult, void* rounded, int rounded_dtype, int rows,
                       int hidden, void* stream);
-// A sublayer between two norms: x[r] += norm(a[r]) * weight (RMS: a / sqrt(mean(a^2) + eps); centered: the
+// A sublayer between two norms: x[r] += mult * (norm(a[r]) * weight + bias) (bias may be null; RMS: a / sqrt(mean(a^2) + eps); centered: the
 // row's mean taken off first), and what reads x next, formed from the new row in the same pass:
 // next_kind 0 nothing, 1 x rounded to next_dtype, 2 the RMS norm of x times next_weight, 3 the same with
-// the mean taken off (next_eps under its root); next_out [rows][hidden] of next_dtype.
-int fw_norm_add_norm(float* x, const float* a, const float* weight, int centered, float eps, int next_kind,
-                     const float* next_weight, float next_eps, void* next_out, int next_dtype, int rows, int hidden,
-                     void* stream);
+// the mean taken off (next_eps under its root; next_bias, if not null, is added); next_out [rows][hidden] of next_dtype, its
+// rows next_stride apart (0: hidden).
+int fw_norm_add_norm(float* x, const float* a, const float* weight, const float* bias, float mult, int centered, float eps,
+                     int next_kind, const float* next_weight, const float* next_bias, float next_eps, void* next_out, int next_dtype,
+                     int next_stride, int rows, int hidden, void* stream);
+// x (float32 [rows][hidden]) into columns col0 .. of out [rows][out_stride] of out_dtype, with `twice` once more behind them
+int fw_place_rows(const float* x, void* out, int out_dtype, int rows, int hidden, int out_stride, int col0, int twice, void* stream);
+// out = gelu(z), the error-function form; z float32, count elements
+int fw_gelu_rows(const float* z, void* out, int out_dtype, long long count, void* stream);
 // out (bfloat16) = x (float32), count elements
 int fw_round_rows(const float* x, void* out, long long count, void* stream);
 // gate_up [rows][2 I]: out[r][i] = g sigmoid(alpha g) (u + shift), g = min(gate, limit),
@@ -290,21 +325,21 @@ int fw_clamped_glu(const void* gate_up, int in_dtype, void* out, int out_dtype, 
 // (2i, 2i + 1) of its first `turn` turned by the row's angles (tables [rows][turn / 2]), stored behind the latent in the key layout only.
 int fw_latent_norm_write(const float* raw, int raw_stride, int col0, const float* weight, float eps, void* k_pages,
                          void* v_pages, int dtype, const int32_t* block_table, int table_stride, const int32_t* row_seg,
-                         const int32_t* row_pos, int rows, int rank, int rot, int turn, const float* cos_table, const float* sin_table,
+                         const int32_t* row_pos, int rows, int rank, int rot, int turn, int interleaved, const float* cos_table, const float* sin_table,
                          int page_size, int num_pages, void* stream);
 // A map per head: out[r][h N + n] = sum_k in[r][h K + k] * w[h][n][k], with a gate (may be null) times
-// sigmoid(gate[r][h N + n]). in [rows][in_stride], w [heads][N][K], gate float32 [rows][gate_stride],
+// sigmoid(gate[r][h N + n]), or with gate_per_head sigmoid(gate[r][h]). in [rows][in_stride], w [heads][N][K], gate float32 [rows][gate_stride],
 // out [rows][heads N]. in_head / out_head / out_stride (0: K, N, heads * out_head): a head's inputs lie in_head apart
 // and its outputs out_head apart in rows out_stride wide, where a head's vector holds more than the map reads or writes.
 int fw_head_linear(const void* in, int in_dtype, int in_stride, const void* w, int w_dtype, const float* gate, int gate_stride,
-                   void* out, int out_dtype, int rows, int heads, int N, int K, int in_head, int out_head, int out_stride,
+                   int gate_per_head, void* out, int out_dtype, int rows, int heads, int N, int K, int in_head, int out_head, int out_stride,
                    void* stream);
-// Channels col0 .. col0 + rot - 1 of every head's vector (heads in_head apart in rows in_stride wide) turned, neighbouring
-// channels (2i, 2i + 1) of the first `turn` by the row's angles (tables [rows][turn / 2]), and stored from channel out_col0 of the head's
+// Channels col0 .. col0 + rot - 1 of every head's vector (heads in_head apart in rows in_stride wide) turned (interleaved:
+// channels (2i, 2i + 1), else (i, i + turn / 2)) in the first `turn` by the row's angles (tables [rows][turn / 2]), and stored from channel out_col0 of the head's
 // vector in out (heads out_head apart in rows out_stride wide).
 int fw_rotate_place(const void* in, int in_dtype, int in_stride, int in_head, int col0, const float* cos_table,
                     const float* sin_table, void* out, int out_dtype, int out_stride, int out_head, int out_col0, int rows,
-                    int heads, int rot, int turn, void* stream);
+                    int heads, int rot, int turn, int interleaved, void* stream);
 
 // ---- a recurrence with a decay per key channel formed by the token ("wkv") --------------------------------
 // Token shift: h = rmsnorm(x) * (w or 1 + w) (norm_weight null: h = x); out[s][r] = h[r] + (h[r - 1] - h[r]) * mu[s],
@@ -326,10 +361,11 @@ int fw_wkv_recurrence(const float* r, const float* k, const float* v, int rkv_st
 // chosen / weight [rows][top]: the `top` largest of logits[r] + bias (float32 [rows][experts]; ties: the lowest
 // id; bias may be null), largest first, and the softmax over those alone. groups > 1: the experts form that many equal
 // groups of neighbours, a group's score is its best expert's, and only experts of the `keep` best groups (ties: the
-// lowest group) can be chosen. score_all: the weights are the softmax over ALL experts at the chosen ones, divided by
-// their sum + 1e-20.
+// lowest group) can be chosen; group_pair: a group's score is the sum of its two best experts' scores. scores 0: the weights as
+// said; 1: the softmax over ALL experts at the chosen ones, divided by their sum + 1e-20; 2: each expert's own sigmoid
+// at the chosen ones, divided by their sum + 1e-20.
 int fw_moe_route(const float* logits, const float* bias, int32_t* chosen, float* weight, int rows, int experts, int top,
-                 int groups, int keep, int score_all, void* stream);
+                 int groups, int keep, int group_pair, int scores, void* stream);
 // The pairs (row, choice) sorted by expert, in the order of the pairs within an expert: expert_begin
 // [experts + 1], place_row [rows * top] (the row of each place), pair_place [rows * top] (the place of each pair).
 int fw_moe_arrange(const int32_t* chosen, int32_t* expert_begin, int32_t* place_row, int32_t* pair_place, int rows, int experts,

@@ -376,7 +376,8 @@ extern "C" int fw_gemm_decode(int prologue, const void* a, const float* norm_wei
     FW_REQUIRE(epilogue != DG_ACCUMULATE || out_dtype == FW_F32, "gemm_decode: accumulation needs a float32 destination");
     FW_REQUIRE(epilogue != DG_ACCUMULATE || prologue == 0, "gemm_decode: the accumulating product takes bfloat16 activations");
     FW_REQUIRE(epilogue != DG_SWIGLU || out_dtype == FW_BF16, "gemm_decode: SwiGLU stores bfloat16");
-    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16, "gemm_decode: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && epilogue == DG_STORE && prologue == 0),
+               "gemm_decode: unknown out dtype %d (gelu goes with a plain storing product)", out_dtype);
     FW_REQUIRE(epilogue != DG_CONV || (taps && state && seg_slot && kernel_size >= 2 && kernel_size <= DG_MAX_TAPS),
                "gemm_decode: the convolution epilogue needs taps, state, slots and a kernel size in 2..%d", DG_MAX_TAPS);
     FW_REQUIRE(((uintptr_t)a % 16 == 0) && ((uintptr_t)w % 16 == 0) && ((uintptr_t)norm_weight % 16 == 0),
@@ -404,7 +405,8 @@ extern "C" int fw_gemm_decode(int prologue, const void* a, const float* norm_wei
 #define DG_STORE_CASE(RT, ROWS)                                                                     \
     if (prologue == 1) { if (out_dtype == FW_F32) DG_TRY(RT, 8, ROWS, 1, DG_STORE, float); else DG_TRY(RT, 8, ROWS, 1, DG_STORE, bf16_t); } \
     else if (prologue == 2) { if (out_dtype == FW_F32) DG_TRY(RT, 8, ROWS, 2, DG_STORE, float); else DG_TRY(RT, 8, ROWS, 2, DG_STORE, bf16_t); } \
-    else { if (out_dtype == FW_F32) DG_TRY(RT, 8, ROWS, 0, DG_STORE, float); else DG_TRY(RT, 8, ROWS, 0, DG_STORE, bf16_t); }
+    else { if (out_dtype == FW_F32) DG_TRY(RT, 8, ROWS, 0, DG_STORE, float); \
+           else if (out_dtype == FW_BF16_GELU) DG_TRY(RT, 8, ROWS, 0, DG_STORE, gelu_bf16_t); else DG_TRY(RT, 8, ROWS, 0, DG_STORE, bf16_t); }
         if (N >= 16384) { DG_STORE_CASE(2, 16) } else if (narrow) { DG_STORE_CASE(1, 8) } else { DG_STORE_CASE(1, 16) }
 #undef DG_STORE_CASE
     } else if (epilogue == DG_SWIGLU) {

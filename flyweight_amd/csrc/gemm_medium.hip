@@ -331,7 +331,7 @@ __global__ __launch_bounds__(GM_THREADS) void gemm_medium_kernel(const MediumArg
             const int n = n_first + r;
             if (MODE == GM_SWIGLU) v[r] = fw_gated_unit(acc[0][mt][r] * inv, acc[1][mt][r] * inv, p.glu_limit, p.glu_alpha, p.glu_shift,
                                                         [](float g) { return gm_silu(g); });
-            else v[r] = acc[0][mt][r] * inv + ((p.bias && n < N) ? p.bias[n] : 0.0f);
+            else v[r] = fw_before_store<TO>(acc[0][mt][r] * inv + ((p.bias && n < N) ? p.bias[n] : 0.0f));
         }
         if (mine) {
             if constexpr (sizeof(TO) == 4) {
@@ -452,6 +452,7 @@ static void medium_launch_as(const MediumArgs& args, int out_dtype, int mode, di
     if (mode == GM_SWIGLU) gemm_medium_kernel<MT, FW, GM_SWIGLU, bf16_t, ROTATE, WT><<<grid, GM_THREADS, 0, stream>>>(args);
     else if (mode == GM_ACCUMULATE) gemm_medium_kernel<MT, FW, GM_ACCUMULATE, float, ROTATE, WT><<<grid, GM_THREADS, 0, stream>>>(args);
     else if (out_dtype == FW_F32) gemm_medium_kernel<MT, FW, GM_STORE, float, ROTATE, WT><<<grid, GM_THREADS, 0, stream>>>(args);
+    else if (out_dtype == FW_BF16_GELU) gemm_medium_kernel<MT, FW, GM_STORE, gelu_bf16_t, ROTATE, WT><<<grid, GM_THREADS, 0, stream>>>(args);
     else gemm_medium_kernel<MT, FW, GM_STORE, bf16_t, ROTATE, WT><<<grid, GM_THREADS, 0, stream>>>(args);
 }
 
@@ -481,7 +482,7 @@ extern "C" int fw_gemm_medium(const void* a, const void* w, int w_tiled, const f
     FW_REQUIRE(!w_tiled || K % 32 == 0, "gemm_medium: weights in operand tiles need K (%d) to be a multiple of 32", K);
     FW_REQUIRE(mode != GM_ACCUMULATE || out_dtype == FW_F32, "gemm_medium: accumulation needs a float32 destination");
     FW_REQUIRE(mode != GM_SWIGLU || (out_dtype == FW_BF16 && bias == nullptr), "gemm_medium: SwiGLU stores bfloat16 and takes no bias");
-    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16, "gemm_medium: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == GM_STORE), "gemm_medium: unknown out dtype %d", out_dtype);
     FW_REQUIRE(((uintptr_t)a % 16 == 0) && ((uintptr_t)w % 16 == 0) && ((uintptr_t)out % 16 == 0) && ((uintptr_t)workspace % 16 == 0),
                "gemm_medium: operands must be 16-byte aligned");
     FW_REQUIRE((next_activations == nullptr) == (next_squares == nullptr) && (next_activations == nullptr) == (next_norm_weight == nullptr),

@@ -323,7 +323,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
                         for (int h = 0; h < 2; ++h) {
                             const int r = 4 * q + 2 * h;
-                            const float upper = acc[i][j][r] + b, lower = acc[i][j][r + 1] + b;
+                            const float upper = fw_before_store<TO>(acc[i][j][r] + b), lower = fw_before_store<TO>(acc[i][j][r + 1] + b);
                             const float got = from_neighbour(odd ? upper : lower);
                             const uint32_t word = odd ? pack_bf16x2(got, lower) : pack_bf16x2(upper, got);
                             *reinterpret_cast<uint32_t*>(pair + (size_t)(i * 32 + 8 * q + 2 * h + (odd ? 1 : 0)) * N) = word;
@@ -434,7 +434,7 @@ extern "C" int fw_gemm_mfma_big(const void* a, const void* w, const float* bias,
     FW_REQUIRE(mode >= 0 && mode <= 2, "gemm_mfma_big: unknown mode %d", mode);
     FW_REQUIRE(mode != MB_ACCUMULATE || out_dtype == FW_F32, "gemm_mfma_big: accumulation needs a float32 destination");
     FW_REQUIRE(mode != MB_SWIGLU || (out_dtype == FW_BF16 && bias == nullptr), "gemm_mfma_big: SwiGLU stores bfloat16 and takes no bias");
-    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16, "gemm_mfma_big: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == MB_STORE), "gemm_mfma_big: unknown out dtype %d", out_dtype);
     FW_REQUIRE(((uintptr_t)a % 16 == 0) && ((uintptr_t)w % 16 == 0), "gemm_mfma_big: operands must be 16-byte aligned");
     FW_REQUIRE((long long)fw_ceil_div(M, BT / 2) * fw_ceil_div(N, BT / 2) < (1ll << 30), "gemm_mfma_big: too many tiles");
     hipStream_t s = (hipStream_t)stream;
@@ -443,6 +443,7 @@ extern "C" int fw_gemm_mfma_big(const void* a, const void* w, const float* bias,
     if (mode == MB_SWIGLU) status = launch_big<MB_SWIGLU, bf16_t>(a, w, nullptr, out, M, N, K, s);
     else if (mode == MB_ACCUMULATE) status = launch_planned<MB_ACCUMULATE, float>(plan, a, w, bias, out, M, N, K, s);
     else if (out_dtype == FW_F32) status = launch_planned<MB_STORE, float>(plan, a, w, bias, out, M, N, K, s);
+    else if (out_dtype == FW_BF16_GELU) status = launch_planned<MB_STORE, gelu_bf16_t>(plan, a, w, bias, out, M, N, K, s);
     else status = launch_planned<MB_STORE, bf16_t>(plan, a, w, bias, out, M, N, K, s);
     if (status != 0) return status;
     FW_LAUNCH_CHECK("gemm_mfma_big");

@@ -301,7 +301,7 @@ extern "C" int fw_gemm_mfma_deep(const void* a, const void* w, const float* bias
     FW_REQUIRE(mode == MD_STORE || mode == MD_ACCUMULATE, "gemm_mfma_deep: mode %d is not served", mode);
     FW_REQUIRE(columns == 128 || columns == 64, "gemm_mfma_deep: tiles have 128 or 64 columns, not %d", columns);
     FW_REQUIRE(mode != MD_ACCUMULATE || out_dtype == FW_F32, "gemm_mfma_deep: accumulation needs a float32 destination");
-    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16, "gemm_mfma_deep: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == MD_STORE), "gemm_mfma_deep: unknown out dtype %d", out_dtype);
     FW_REQUIRE(((uintptr_t)a % 16 == 0) && ((uintptr_t)w % 16 == 0), "gemm_mfma_deep: operands must be 16-byte aligned");
     FW_REQUIRE((long long)fw_ceil_div(M, DT) * fw_ceil_div(N, 64) < (1ll << 30), "gemm_mfma_deep: too many tiles");
     hipStream_t s = (hipStream_t)stream;
@@ -309,10 +309,12 @@ extern "C" int fw_gemm_mfma_deep(const void* a, const void* w, const float* bias
     if (columns == 128) {
         if (mode == MD_ACCUMULATE) status = launch_deep<MD_ACCUMULATE, float, 4>(a, w, bias, out, M, N, K, s);
         else if (out_dtype == FW_F32) status = launch_deep<MD_STORE, float, 4>(a, w, bias, out, M, N, K, s);
+        else if (out_dtype == FW_BF16_GELU) status = launch_deep<MD_STORE, gelu_bf16_t, 4>(a, w, bias, out, M, N, K, s);
         else status = launch_deep<MD_STORE, bf16_t, 4>(a, w, bias, out, M, N, K, s);
     } else {
         if (mode == MD_ACCUMULATE) status = launch_deep<MD_ACCUMULATE, float, 2>(a, w, bias, out, M, N, K, s);
         else if (out_dtype == FW_F32) status = launch_deep<MD_STORE, float, 2>(a, w, bias, out, M, N, K, s);
+        else if (out_dtype == FW_BF16_GELU) status = launch_deep<MD_STORE, gelu_bf16_t, 2>(a, w, bias, out, M, N, K, s);
         else status = launch_deep<MD_STORE, bf16_t, 2>(a, w, bias, out, M, N, K, s);
     }
     if (status != 0) return status;

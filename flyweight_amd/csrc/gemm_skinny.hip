@@ -151,6 +151,8 @@ static void launch_mode(const void* a, const void* w, const float* bias, void* o
         gemm_skinny_kernel<MT, RT, WAVES, SK_ACCUMULATE, float><<<blocks, threads, 0, stream>>>(pa, pw, bias, (float*)out, M, N, K, 0);
     else if (out_dtype == FW_F32)
         gemm_skinny_kernel<MT, RT, WAVES, SK_STORE, float><<<blocks, threads, 0, stream>>>(pa, pw, bias, (float*)out, M, N, K, 0);
+    else if (out_dtype == FW_BF16_GELU)
+        gemm_skinny_kernel<MT, RT, WAVES, SK_STORE, gelu_bf16_t><<<blocks, threads, 0, stream>>>(pa, pw, bias, (gelu_bf16_t*)out, M, N, K, 0);
     else
         gemm_skinny_kernel<MT, RT, WAVES, SK_STORE, bf16_t><<<blocks, threads, 0, stream>>>(pa, pw, bias, (bf16_t*)out, M, N, K, 0);
 }
@@ -174,7 +176,7 @@ extern "C" int fw_gemm_skinny(const void* a, const void* w, const float* bias, v
     FW_REQUIRE(mode >= 0 && mode <= 2, "gemm_skinny: unknown mode %d", mode);
     FW_REQUIRE(mode != SK_ACCUMULATE || out_dtype == FW_F32, "gemm_skinny: accumulation needs a float32 destination");
     FW_REQUIRE(mode != SK_SWIGLU || (out_dtype == FW_BF16 && bias == nullptr), "gemm_skinny: SwiGLU stores bfloat16 and takes no bias");
-    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16, "gemm_skinny: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == SK_STORE), "gemm_skinny: unknown out dtype %d", out_dtype);
     FW_REQUIRE(((uintptr_t)a % 16 == 0) && ((uintptr_t)w % 16 == 0), "gemm_skinny: operands must be 16-byte aligned");
     hipStream_t s = (hipStream_t)stream;
     switch ((M + 15) / 16) {

@@ -13,14 +13,15 @@
 // c = raw / sqrt(mean(raw^2) + eps) * weight goes to both layouts of the cache's one head:
 // k_pages [page][1][64][rank + rot] (a token's channels together) and v_pages [page][1][rank][64].
 // rot > 0: the next rot columns of raw are a key part of the token's own that every head shares; it is not
-// normed, neighbouring channels (2i, 2i + 1) of its first `turn` turn by the row's angles (tables [rows][turn / 2]), and
+// normed, channels of its first `turn` turn in pairs by the row's angles (tables [rows][turn / 2]; interleaved: channels
+// (2i, 2i + 1), else (i, i + turn / 2)), and
 // it is stored behind the latent in the key layout only (a key has rank + rot channels, a value rank).
 template <typename T>
 __global__ __launch_bounds__(256) void latent_norm_write_kernel(
     const float* __restrict__ raw, int raw_stride, int col0, const float* __restrict__ weight, float eps,
     T* __restrict__ k_pages, T* __restrict__ v_pages, const int32_t* __restrict__ block_table, int table_stride,
     const int32_t* __restrict__ row_seg, const int32_t* __restrict__ row_pos, int rank, int rot, int turn,
-    const float* __restrict__ cos_table, const float* __restrict__ sin_table) {
+    int interleaved, const float* __restrict__ cos_table, const float* __restrict__ sin_table) {
     __shared__ float scratch[16];
     const int row = blockIdx.x;
     const float* source = raw + (size_t)row * raw_stride + col0;
@@ -43,17 +44,20 @@ __global__ __launch_bounds__(256) void latent_norm_write_kernel(
             store_from_float(key, rank + j, mine);
             continue;
         }
-        const float other = source[rank + (j ^ 1)];
-        const float c = cos_table[(size_t)row * (turn / 2) + (j >> 1)], sn = sin_table[(size_t)row * (turn / 2) + (j >> 1)];
+        const int half = turn / 2;
+        const bool second = interleaved ? (j & 1) != 0 : j >= half;
+        const float other = source[rank + (interleaved ? j ^ 1 : (second ? j - half : j + half))];
+        const int pair = interleaved ? j >> 1 : (second ? j - half : j);
+        const float c = cos_table[(size_t)row * half + pair], sn = sin_table[(size_t)row * half + pair];
         // one rounding of other * sin, then one fused step: the same in every kernel that rotates
-        store_from_float(key, rank + j, fmaf(mine, c, (j & 1) ? other * sn : -(other * sn)));
+        store_from_float(key, rank + j, fmaf(mine, c, second ? other * sn : -(other * sn)));
     }
 }
 
 extern "C" int fw_latent_norm_write(const float* raw, int raw_stride, int col0, const float* weight, float eps, void* k_pages,
                                     void* v_pages, int dtype, const int32_t* block_table, int table_stride,
                                     const int32_t* row_seg, const int32_t* row_pos, int rows, int rank, int rot, int turn,
-                                    const float* cos_table, const float* sin_table, int page_size, int num_pages, void* stream) {
+                                    int interleaved, const float* cos_table, const float* sin_table, int page_size, int num_pages, void* stream) {
     FW_REQUIRE(rows >= 0 && rank > 0 && col0 >= 0 && rot >= 0 && col0 + rank + rot <= raw_stride, "latent_norm_write: columns %d..%d of rows %d wide", col0,
                col0 + rank + rot, raw_stride);
     FW_REQUIRE(turn >= 0 && turn <= rot && turn % 2 == 0 && (turn == 0 || (cos_table && sin_table)),
@@ -65,10 +69,10 @@ extern "C" int fw_latent_norm_write(const float* raw, int raw_stride, int col0, 
     hipStream_t s = (hipStream_t)stream;
     if (dtype == FW_F32)
         latent_norm_write_kernel<float><<<rows, 256, 0, s>>>(raw, raw_stride, col0, weight, eps, (float*)k_pages, (float*)v_pages,
-                                                             block_table, table_stride, row_seg, row_pos, rank, rot, turn, cos_table, sin_table);
+                                                             block_table, table_stride, row_seg, row_pos, rank, rot, turn, interleaved, cos_table, sin_table);
     else if (dtype == FW_BF16)
         latent_norm_write_kernel<bf16_t><<<rows, 256, 0, s>>>(raw, raw_stride, col0, weight, eps, (bf16_t*)k_pages, (bf16_t*)v_pages,
-                                                              block_table, table_stride, row_seg, row_pos, rank, rot, turn, cos_table, sin_table);
+                                                              block_table, table_stride, row_seg, row_pos, rank, rot, turn, interleaved, cos_table, sin_table);
     else
         FW_REQUIRE(false, "latent_norm_write: unknown dtype %d", dtype);
     FW_LAUNCH_CHECK("latent_norm_write");
@@ -76,7 +80,8 @@ extern "C" int fw_latent_norm_write(const float* raw, int raw_stride, int col0, 
 }
 
 // ---- a map per head ------------------------------------------------------------------------------------
-// out[r][h N + n] = sum_k in[r][h K + k] * w[h][n][k], then with a gate (float32) times sigmoid(gate[r][h N + n]).
+// out[r][h N + n] = sum_k in[r][h K + k] * w[h][n][k], then with a gate (float32) times sigmoid(gate[r][h N + n])
+// (gate_per_head: times sigmoid(gate[r][h]), one number for a head's outputs).
 // in [rows][in_stride], w [heads][N][K], out [rows][heads N]. A head's inputs may lie in_head apart (K of them used) and
 // its outputs out_head apart in rows out_stride wide (a head's vector holds more than the map reads or writes). Float32 sums, each output summed over k
 // in order by one thread: a function of the row alone.
@@ -84,7 +89,7 @@ extern "C" int fw_latent_norm_write(const float* raw, int raw_stride, int col0, 
 #define HL_K 16             // k values staged at a time
 template <typename TI, typename TW, typename TO>
 __global__ __launch_bounds__(256) void head_linear_kernel(const TI* __restrict__ in, int in_stride, const TW* __restrict__ w,
-                                                         const float* __restrict__ gate, int gate_stride, TO* __restrict__ out,
+                                                         const float* __restrict__ gate, int gate_stride, int gate_per_head, TO* __restrict__ out,
                                                          int rows, int heads, int N, int K, int in_head, int out_head, int out_stride) {
     __shared__ float a_tile[HL_K][HL_TILE + 1], w_tile[HL_K][HL_TILE + 1];
     const int head = blockIdx.z;
@@ -128,7 +133,7 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const TI* __restrict__
             if (col >= N) continue;
             float value = acc[i][j];
             if (gate) {
-                const float z = gate[(size_t)row * gate_stride + (size_t)head * N + col];
+                const float z = gate[(size_t)row * gate_stride + (gate_per_head ? (size_t)head : (size_t)head * N + col)];
                 value *= 1.0f / (1.0f + expf(-z));
             }
             store_from_float(out, (size_t)row * out_stride + (size_t)head * out_head + col, value);
@@ -195,7 +200,7 @@ typedef __attribute__((ext_vector_type(4))) float hl_f32x4;
 typedef __attribute__((ext_vector_type(4))) uint32_t hl_u32x4;
 template <int NT, bool WIDE>
 __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const uint16_t* __restrict__ in, int in_stride, const uint16_t* __restrict__ w,
-                                                              const float* __restrict__ gate, int gate_stride, uint16_t* __restrict__ out,
+                                                              const float* __restrict__ gate, int gate_stride, int gate_per_head, uint16_t* __restrict__ out,
                                                               int rows, int heads, int N, int K, int in_head, int out_head, int out_stride) {
     const int head = blockIdx.z;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, i16 = lane & 15, g = lane >> 4;
@@ -234,7 +239,8 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const uint16_t* _
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             value[r] = acc[t][r];
-            if (gate && n0 + r < N) value[r] *= 1.0f / (1.0f + expf(-gate[(size_t)row * gate_stride + (size_t)head * N + n0 + r]));
+            if (gate && n0 + r < N)
+                value[r] *= 1.0f / (1.0f + expf(-gate[(size_t)row * gate_stride + (gate_per_head ? (size_t)head : (size_t)head * N + n0 + r)]));
         }
         uint16_t* dest = out + (size_t)row * out_stride + (size_t)head * out_head + n0;
         if (n0 + 3 < N && N % 4 == 0) {
@@ -250,7 +256,7 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const uint16_t* _
 }
 
 extern "C" int fw_head_linear(const void* in, int in_dtype, int in_stride, const void* w, int w_dtype, const float* gate,
-                              int gate_stride, void* out, int out_dtype, int rows, int heads, int N, int K, int in_head, int out_head,
+                              int gate_stride, int gate_per_head, void* out, int out_dtype, int rows, int heads, int N, int K, int in_head, int out_head,
                               int out_stride, void* stream) {
     FW_REQUIRE(rows >= 0 && heads > 0 && heads <= 65535 && N > 0 && K > 0, "head_linear: bad sizes rows=%d heads=%d N=%d K=%d", rows, heads, N, K);
     if (in_head <= 0) in_head = K;
@@ -259,7 +265,8 @@ extern "C" int fw_head_linear(const void* in, int in_dtype, int in_stride, const
     FW_REQUIRE(in_head >= K && in_stride >= (heads - 1) * in_head + K, "head_linear: rows %d wide do not hold %d heads %d apart of %d", in_stride, heads, in_head, K);
     FW_REQUIRE(out_head >= N && out_stride >= (heads - 1) * out_head + N, "head_linear: rows %d wide do not take %d heads %d apart of %d", out_stride, heads, out_head, N);
     FW_REQUIRE(gate == nullptr || (out_head == N && out_stride == heads * N), "head_linear: a gate goes with outputs side by side");
-    FW_REQUIRE(gate == nullptr || gate_stride >= heads * N, "head_linear: the gates' rows (%d wide) do not hold %d x %d", gate_stride, heads, N);
+    FW_REQUIRE(gate == nullptr || gate_stride >= (gate_per_head ? heads : heads * N), "head_linear: the gates' rows (%d wide) do not hold %d x %d", gate_stride, heads,
+               gate_per_head ? 1 : N);
     if (rows == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     if (in_dtype == FW_BF16 && w_dtype == FW_BF16 && out_dtype == FW_BF16 && K % 8 == 0 && in_stride % 8 == 0 && in_head % 8 == 0 &&
@@ -268,12 +275,12 @@ extern "C" int fw_head_linear(const void* in, int in_dtype, int in_stride, const
         if (rows <= 16) {
             dim3 wide(1, (N + 63) / 64, heads);
             FW_REQUIRE(wide.y <= 65535, "head_linear: too many columns (%d)", N);
-            head_linear_mfma_kernel<1, true><<<wide, 256, 0, s>>>((const uint16_t*)in, in_stride, (const uint16_t*)w, gate, gate_stride,
+            head_linear_mfma_kernel<1, true><<<wide, 256, 0, s>>>((const uint16_t*)in, in_stride, (const uint16_t*)w, gate, gate_stride, gate_per_head,
                                                                   (uint16_t*)out, rows, heads, N, K, in_head, out_head, out_stride);
         } else {
             dim3 tall((rows + 63) / 64, (N + 63) / 64, heads);
             FW_REQUIRE(tall.y <= 65535, "head_linear: too many columns (%d)", N);
-            head_linear_mfma_kernel<4, false><<<tall, 256, 0, s>>>((const uint16_t*)in, in_stride, (const uint16_t*)w, gate, gate_stride,
+            head_linear_mfma_kernel<4, false><<<tall, 256, 0, s>>>((const uint16_t*)in, in_stride, (const uint16_t*)w, gate, gate_stride, gate_per_head,
                                                                    (uint16_t*)out, rows, heads, N, K, in_head, out_head, out_stride);
         }
         FW_LAUNCH_CHECK("head_linear");
@@ -293,7 +300,7 @@ extern "C" int fw_head_linear(const void* in, int in_dtype, int in_stride, const
     dim3 grid((rows + HL_TILE - 1) / HL_TILE, (N + HL_TILE - 1) / HL_TILE, heads);
     FW_REQUIRE(grid.y <= 65535, "head_linear: too many columns (%d)", N);
 #define FW_HL_LAUNCH(TI, TW, TO)                                                                                          \
-    head_linear_kernel<TI, TW, TO><<<grid, 256, 0, s>>>((const TI*)in, in_stride, (const TW*)w, gate, gate_stride, \
+    head_linear_kernel<TI, TW, TO><<<grid, 256, 0, s>>>((const TI*)in, in_stride, (const TW*)w, gate, gate_stride, gate_per_head, \
                                                         (TO*)out, rows, heads, N, K, in_head, out_head, out_stride)
     if (in_dtype == FW_F32 && w_dtype == FW_F32 && out_dtype == FW_F32) FW_HL_LAUNCH(float, float, float);
     else if (in_dtype == FW_BF16 && w_dtype == FW_BF16 && out_dtype == FW_BF16) FW_HL_LAUNCH(bf16_t, bf16_t, bf16_t);
@@ -308,30 +315,34 @@ extern "C" int fw_head_linear(const void* in, int in_dtype, int in_stride, const
 
 // ---- a rotated part of every head's vector -------------------------------------------------------------------
 // in [rows][in_stride]: head h's vector begins at h * in_head and its channels col0 .. col0 + rot - 1 are turned
-// (neighbouring channels (2i, 2i + 1) of the first `turn` by the row's angles, tables [rows][turn / 2], float32; the rest pass) and stored at
+// (in pairs of the first `turn` by the row's angles, tables [rows][turn / 2], float32; interleaved: channels (2i, 2i + 1), else
+// (i, i + turn / 2); the rest pass) and stored at
 // out[r][h * out_head + out_col0 ..] in rows out_stride wide. A thread per (row, head, pair).
 template <typename TI, typename TO>
 __global__ __launch_bounds__(256) void rotate_place_kernel(const TI* __restrict__ in, int in_stride, int in_head, int col0,
                                                           const float* __restrict__ cos_table, const float* __restrict__ sin_table,
                                                           TO* __restrict__ out, int out_stride, int out_head, int out_col0, int heads,
-                                                          int rot, int turn) {
+                                                          int rot, int turn, int interleaved) {
     const int row = blockIdx.x, half = rot / 2, turned = turn / 2;
     for (int item = threadIdx.x; item < heads * half; item += blockDim.x) {
         const int head = item / half, pair = item % half;
         const TI* source = in + (size_t)row * in_stride + (size_t)head * in_head + col0;
-        const float u = load_as_float(source, 2 * pair), v = load_as_float(source, 2 * pair + 1);
+        // the pair's two channels; past the turned ones two neighbours that pass
+        const int first = interleaved || pair >= turned ? 2 * pair : pair;
+        const int second = interleaved || pair >= turned ? 2 * pair + 1 : pair + turned;
+        const float u = load_as_float(source, first), v = load_as_float(source, second);
         // a pair past the turned channels passes as it is (an angle of zero)
         const float c = pair < turned ? cos_table[(size_t)row * turned + pair] : 1.0f;
         const float sn = pair < turned ? sin_table[(size_t)row * turned + pair] : 0.0f;
         TO* dest = out + (size_t)row * out_stride + (size_t)head * out_head + out_col0;
-        store_from_float(dest, 2 * pair, fmaf(u, c, -(v * sn)));
-        store_from_float(dest, 2 * pair + 1, fmaf(v, c, u * sn));
+        store_from_float(dest, first, fmaf(u, c, -(v * sn)));
+        store_from_float(dest, second, fmaf(v, c, u * sn));
     }
 }
 
 extern "C" int fw_rotate_place(const void* in, int in_dtype, int in_stride, int in_head, int col0, const float* cos_table,
                                const float* sin_table, void* out, int out_dtype, int out_stride, int out_head, int out_col0, int rows,
-                               int heads, int rot, int turn, void* stream) {
+                               int heads, int rot, int turn, int interleaved, void* stream) {
     FW_REQUIRE(turn >= 0 && turn <= rot && turn % 2 == 0, "rotate_place: %d turned channels of %d", turn, rot);
     FW_REQUIRE(rows >= 0 && heads > 0 && rot > 0 && rot % 2 == 0, "rotate_place: bad sizes rows=%d heads=%d rot=%d", rows, heads, rot);
     FW_REQUIRE(col0 >= 0 && col0 + rot <= in_head && in_stride >= (heads - 1) * in_head + col0 + rot,
@@ -343,7 +354,7 @@ extern "C" int fw_rotate_place(const void* in, int in_dtype, int in_stride, int 
     hipStream_t s = (hipStream_t)stream;
 #define FW_RP_LAUNCH(TI, TO)                                                                                                      \
     rotate_place_kernel<TI, TO><<<rows, 256, 0, s>>>((const TI*)in, in_stride, in_head, col0, cos_table, sin_table, (TO*)out, out_stride, \
-                                                     out_head, out_col0, heads, rot, turn)
+                                                     out_head, out_col0, heads, rot, turn, interleaved)
     if (in_dtype == FW_F32 && out_dtype == FW_F32) FW_RP_LAUNCH(float, float);
     else if (in_dtype == FW_BF16 && out_dtype == FW_BF16) FW_RP_LAUNCH(bf16_t, bf16_t);
     else if (in_dtype == FW_F32 && out_dtype == FW_BF16) FW_RP_LAUNCH(float, bf16_t);

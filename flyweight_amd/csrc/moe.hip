@@ -18,11 +18,17 @@
 #define MOE_MAX_EXPERTS 1024
 #define MOE_MAX_TOP 64
 // groups > 1: the experts form that many equal groups of neighbours, a group's score is its best expert's, and only
-// experts of the `keep` best groups (ties: the lowest group) can be chosen. score_all: the weights are the softmax
-// over ALL experts at the chosen ones, divided by their sum + 1e-20 (else the softmax over the chosen alone).
+// experts of the `keep` best groups (ties: the lowest group) can be chosen. group_pair: a group's score is the sum of its
+// two best experts' scores instead (of its one's, where it has no second). scores 0: the weights are the softmax over the chosen
+// alone; 1: the softmax over ALL experts at the chosen ones, divided by their sum + 1e-20; 2: sigmoids of the
+// logits, each expert's on its own, at the chosen ones, divided by their sum + 1e-20.
+#define MOE_SOFTMAX_CHOSEN 0
+#define MOE_SOFTMAX_ALL 1
+#define MOE_SIGMOID 2
+__device__ __forceinline__ float moe_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ logits, const float* __restrict__ bias,
                                                       int32_t* __restrict__ chosen, float* __restrict__ weight, int experts, int top,
-                                                      int groups, int keep, int score_all) {
+                                                      int groups, int keep, int group_pair, int scores) {
     const int row = blockIdx.x, lane = threadIdx.x;
     float z[MOE_MAX_EXPERTS / 64];
 #pragma unroll
@@ -31,7 +37,7 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
         z[i] = e < experts ? logits[(size_t)row * experts + e] + (bias ? bias[e] : 0.0f) : -INFINITY;
     }
     float all_max = 0.0f, all_sum = 1.0f;
-    if (score_all) {    // the softmax's maximum and sum over every expert, before any is shut out
+    if (scores == MOE_SOFTMAX_ALL) {    // the softmax's maximum and sum over every expert, before any is shut out
         float m = -INFINITY;
 #pragma unroll
         for (int i = 0; i < MOE_MAX_EXPERTS / 64; ++i) m = fmaxf(m, z[i]);
@@ -43,7 +49,8 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
         all_sum = wave_sum(sum);
     }
     if (groups > 1 && keep < groups) {
-        // lane g holds the best logit of group g (the softmax is monotonic: the best score is the best logit's)
+        // lane g holds the score of group g: its best logit (scores grow with their logits: the best score is the best
+        // logit's), or the sum of its two best scores
         const int per_group = experts / groups;
         float group_best = -INFINITY;
         for (int g = 0; g < groups; ++g) {
@@ -53,7 +60,28 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
                 const int e = lane + 64 * i;
                 if (e < experts && e / per_group == g) m = fmaxf(m, z[i]);
             }
+            const float mine = m;
             m = wave_max(m);
+            if (group_pair) {
+                // the second best: the lane that holds the best (the lowest such lane) offers its next one
+                const int holder = __ffsll((long long)__ballot(mine == m)) - 1;
+                float next = lane == holder ? -INFINITY : mine;
+                if (lane == holder) {
+                    bool taken = false;
+#pragma unroll
+                    for (int i = 0; i < MOE_MAX_EXPERTS / 64; ++i) {
+                        const int e = lane + 64 * i;
+                        if (e < experts && e / per_group == g) {
+                            if (!taken && z[i] == m) taken = true;
+                            else next = fmaxf(next, z[i]);
+                        }
+                    }
+                }
+                next = wave_max(next);
+                const float shift = scores == MOE_SIGMOID ? 0.0f : all_max, sum = scores == MOE_SIGMOID ? 1.0f : all_sum;
+                m = scores == MOE_SIGMOID ? moe_sigmoid(m) + (per_group > 1 ? moe_sigmoid(next) : 0.0f)
+                                          : expf(m - shift) / sum + (per_group > 1 ? expf(next - shift) / sum : 0.0f);
+            }
             if (lane == g) group_best = m;
         }
         unsigned long long kept = 0ull;
@@ -104,19 +132,21 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
         for (int i = 0; i < MOE_MAX_EXPERTS / 64; ++i)
             if (lane + 64 * i == best_id) z[i] = -INFINITY;
         if (round == 0) first = best;                   // the largest: the softmax's shift
-        const float e = score_all ? expf(best - all_max) / all_sum : expf(best - first);
+        const float e = scores == MOE_SIGMOID ? moe_sigmoid(best) : scores == MOE_SOFTMAX_ALL ? expf(best - all_max) / all_sum : expf(best - first);
         total += e;
         if (lane == round) {
             mine = e;
             chosen[(size_t)row * top + round] = best_id;
         }
     }
-    if (lane < top) weight[(size_t)row * top + lane] = mine / (score_all ? total + 1e-20f : total);
+    if (lane < top) weight[(size_t)row * top + lane] = mine / (scores != MOE_SOFTMAX_CHOSEN ? total + 1e-20f : total);
 }
 
 extern "C" int fw_moe_route(const float* logits, const float* bias, int32_t* chosen, float* weight, int rows, int experts, int top,
-                            int groups, int keep, int score_all, void* stream) {
+                            int groups, int keep, int group_pair, int scores, void* stream) {
     if (groups <= 0) groups = 1;
+    FW_REQUIRE(scores >= MOE_SOFTMAX_CHOSEN && scores <= MOE_SIGMOID && !(group_pair && scores == MOE_SOFTMAX_CHOSEN),
+               "moe_route: unknown scores %d, or groups scored by a pair of logits", scores);
     if (keep <= 0) keep = groups;
     FW_REQUIRE(groups <= 64 && experts % groups == 0 && keep <= groups, "moe_route: %d experts in %d groups (at most 64, equal ones) of which %d are kept",
                experts, groups, keep);
@@ -124,7 +154,7 @@ extern "C" int fw_moe_route(const float* logits, const float* bias, int32_t* cho
     FW_REQUIRE(rows >= 0 && experts >= 1 && experts <= MOE_MAX_EXPERTS, "moe_route: %d experts (1..%d)", experts, MOE_MAX_EXPERTS);
     FW_REQUIRE(top >= 1 && top <= experts && top <= MOE_MAX_TOP, "moe_route: %d of %d experts a token (at most %d)", top, experts, MOE_MAX_TOP);
     if (rows == 0) return 0;
-    moe_route_kernel<<<rows, 64, 0, (hipStream_t)stream>>>(logits, bias, chosen, weight, experts, top, groups, keep, score_all);
+    moe_route_kernel<<<rows, 64, 0, (hipStream_t)stream>>>(logits, bias, chosen, weight, experts, top, groups, keep, group_pair, scores);
     FW_LAUNCH_CHECK("moe_route");
     return 0;
 }

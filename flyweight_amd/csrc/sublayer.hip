@@ -104,6 +104,49 @@ extern "C" int fw_round_rows(const float* x, void* out, long long count, void* s
     return 0;
 }
 
+// The same into some columns of wider rows: out[r][col0 .. col0 + hidden - 1] = x[r], and with `twice` once more `hidden`
+// columns on (rows joined with themselves).
+template <typename T>
+__global__ __launch_bounds__(256) void place_rows_kernel(const float* __restrict__ x, T* __restrict__ out, int hidden, int out_stride,
+                                                        int col0, int twice) {
+    const int row = blockIdx.x;
+    T* to = out + (size_t)row * out_stride + col0;
+    for (int i = threadIdx.x; i < hidden; i += 256) {
+        const float v = x[(size_t)row * hidden + i];
+        store_from_float(to, i, v);
+        if (twice) store_from_float(to, hidden + i, v);
+    }
+}
+
+extern "C" int fw_place_rows(const float* x, void* out, int out_dtype, int rows, int hidden, int out_stride, int col0, int twice, void* stream) {
+    FW_REQUIRE(rows >= 0 && hidden > 0 && col0 >= 0 && col0 + (twice ? 2 : 1) * hidden <= out_stride,
+               "place_rows: %d columns from %d on do not fit rows of %d", (twice ? 2 : 1) * hidden, col0, out_stride);
+    if (rows == 0) return 0;
+    if (out_dtype == FW_F32) place_rows_kernel<float><<<rows, 256, 0, (hipStream_t)stream>>>(x, (float*)out, hidden, out_stride, col0, twice);
+    else if (out_dtype == FW_BF16) place_rows_kernel<bf16_t><<<rows, 256, 0, (hipStream_t)stream>>>(x, (bf16_t*)out, hidden, out_stride, col0, twice);
+    else FW_REQUIRE(false, "place_rows: unknown dtype %d", out_dtype);
+    FW_LAUNCH_CHECK("place_rows");
+    return 0;
+}
+
+// the error-function gelu of float32 sums, rounded once
+template <typename T>
+__global__ void gelu_rows_kernel(const float* __restrict__ z, T* __restrict__ out, long long count) {
+    for (long long i = blockIdx.x * (long long)blockDim.x + threadIdx.x; i < count; i += (long long)gridDim.x * blockDim.x)
+        store_from_float(out, (size_t)i, fw_gelu(z[i]));
+}
+
+extern "C" int fw_gelu_rows(const float* z, void* out, int out_dtype, long long count, void* stream) {
+    FW_REQUIRE(count >= 0, "gelu_rows: negative count");
+    if (count == 0) return 0;
+    const int blocks = (int)((count + 255) / 256 < 8192 ? (count + 255) / 256 : 8192);
+    if (out_dtype == FW_F32) gelu_rows_kernel<float><<<blocks, 256, 0, (hipStream_t)stream>>>(z, (float*)out, count);
+    else if (out_dtype == FW_BF16) gelu_rows_kernel<bf16_t><<<blocks, 256, 0, (hipStream_t)stream>>>(z, (bf16_t*)out, count);
+    else FW_REQUIRE(false, "gelu_rows: unknown dtype %d", out_dtype);
+    FW_LAUNCH_CHECK("gelu_rows");
+    return 0;
+}
+
 // Gated linear unit with clamped halves: g = min(gate, limit), u = clamp(up, -limit, limit),
 // out = g * sigmoid(alpha * g) * (u + shift). gate_up [rows][2 I]: gate columns, then up columns.
 template <typename TI, typename TO>
@@ -145,19 +188,22 @@ extern "C" int fw_clamped_glu(const void* gate_up, int in_dtype, void* out, int 
 // ---- a sublayer between two norms ---------------------------------------------------------------------
 // What joins a sublayer whose output passes a norm of its own to the residual stream, and hands the
 // stream to the next reader, in one pass over the row:
-//     x <- x + norm_a(a) * w            (norm_a: RMS, or with `centered` the mean taken off first)
+//     x <- x + mult * (norm_a(a) * w + bias)   (norm_a: RMS, or with `centered` the mean taken off first; bias null: none)
 //     next_out = next(x)                (next_kind 0: nothing; 1: x rounded to next_dtype; 2: RMS norm
-//                                        of x times next_weight; 3: the same with the mean taken off)
+//                                        of x times next_weight (+ next_bias); 3: the same with the mean taken off)
+// The rows of next_out may lie next_stride apart (they are then some columns of wider rows).
 // A norm here is v / sqrt(mean(v^2) + eps), v the values or their deviations from the row's mean. One
 // workgroup per row; a row of up to 256 * JOIN_HELD values stays in registers between the passes, a
 // wider one is read again. Every sum is a function of the row alone.
 #define JOIN_HELD 16
 template <typename T, bool HELD>
 __global__ __launch_bounds__(256) void norm_add_norm_kernel(
-    float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ weight, int centered, float eps,
-    int next_kind, const float* __restrict__ next_weight, float next_eps, T* __restrict__ next_out, int hidden) {
+    float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ weight, const float* __restrict__ bias, float mult,
+    int centered, float eps, int next_kind, const float* __restrict__ next_weight, const float* __restrict__ next_bias, float next_eps,
+    T* __restrict__ next_out, int next_stride, int hidden) {
     __shared__ float scratch[16];
     const size_t row0 = (size_t)blockIdx.x * hidden;
+    next_out += (size_t)blockIdx.x * next_stride;
     constexpr int N = HELD ? JOIN_HELD : 1;
     float held[N], was[N], scale[N];
     const float count = (float)hidden;
@@ -196,14 +242,16 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(
         for (int u = 0; u < N; ++u) {
             const int i = threadIdx.x + 256 * u;
             if (i < hidden) {
-                was[u] += (held[u] - mean) * inv * scale[u];
+                const float normed = (held[u] - mean) * inv * scale[u];
+                was[u] = fmaf(mult, bias ? normed + bias[i] : normed, was[u]);
                 x[row0 + i] = was[u];
                 new_sum += was[u];
             }
         }
     } else {
         for (int i = threadIdx.x; i < hidden; i += 256) {
-            const float updated = x[row0 + i] + (a[row0 + i] - mean) * inv * weight[i];
+            const float normed = (a[row0 + i] - mean) * inv * weight[i];
+            const float updated = fmaf(mult, bias ? normed + bias[i] : normed, x[row0 + i]);
             x[row0 + i] = updated;          // read again below by the thread that wrote it
             new_sum += updated;
         }
@@ -214,10 +262,10 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(
 #pragma unroll
             for (int u = 0; u < N; ++u) {
                 const int i = threadIdx.x + 256 * u;
-                if (i < hidden) store_from_float(next_out, row0 + i, was[u]);
+                if (i < hidden) store_from_float(next_out, i, was[u]);
             }
         } else {
-            for (int i = threadIdx.x; i < hidden; i += 256) store_from_float(next_out, row0 + i, x[row0 + i]);
+            for (int i = threadIdx.x; i < hidden; i += 256) store_from_float(next_out, i, x[row0 + i]);
         }
         return;
     }
@@ -240,17 +288,24 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(
 #pragma unroll
         for (int u = 0; u < N; ++u) {
             const int i = threadIdx.x + 256 * u;
-            if (i < hidden) store_from_float(next_out, row0 + i, (was[u] - next_mean) * next_inv * next_weight[i]);
+            if (i < hidden) {
+                const float normed = (was[u] - next_mean) * next_inv * next_weight[i];
+                store_from_float(next_out, i, next_bias ? normed + next_bias[i] : normed);
+            }
         }
     } else {
-        for (int i = threadIdx.x; i < hidden; i += 256)
-            store_from_float(next_out, row0 + i, (x[row0 + i] - next_mean) * next_inv * next_weight[i]);
+        for (int i = threadIdx.x; i < hidden; i += 256) {
+            const float normed = (x[row0 + i] - next_mean) * next_inv * next_weight[i];
+            store_from_float(next_out, i, next_bias ? normed + next_bias[i] : normed);
+        }
     }
 }
 
-extern "C" int fw_norm_add_norm(float* x, const float* a, const float* weight, int centered, float eps, int next_kind,
-                                const float* next_weight, float next_eps, void* next_out, int next_dtype, int rows,
-                                int hidden, void* stream) {
+extern "C" int fw_norm_add_norm(float* x, const float* a, const float* weight, const float* bias, float mult, int centered, float eps,
+                                int next_kind, const float* next_weight, const float* next_bias, float next_eps, void* next_out,
+                                int next_dtype, int next_stride, int rows, int hidden, void* stream) {
+    if (next_stride <= 0) next_stride = hidden;
+    FW_REQUIRE(next_stride >= hidden, "norm_add_norm: rows of %d do not fit %d apart", hidden, next_stride);
     FW_REQUIRE(rows >= 0 && hidden > 0, "norm_add_norm: bad sizes rows=%d hidden=%d", rows, hidden);
     FW_REQUIRE(eps > 0.0f, "norm_add_norm: eps must be positive");
     FW_REQUIRE(x && a && weight, "norm_add_norm: x, a and the weight are needed");
@@ -262,8 +317,8 @@ extern "C" int fw_norm_add_norm(float* x, const float* a, const float* weight, i
     hipStream_t s = (hipStream_t)stream;
     const bool held = hidden <= 256 * JOIN_HELD;
 #define FW_JOIN_LAUNCH(T, HELD)                                                                                             \
-    norm_add_norm_kernel<T, HELD><<<rows, 256, 0, s>>>(x, a, weight, centered, eps, next_kind, next_weight, next_eps, \
-                                                       (T*)next_out, hidden)
+    norm_add_norm_kernel<T, HELD><<<rows, 256, 0, s>>>(x, a, weight, bias, mult, centered, eps, next_kind, next_weight, \
+                                                       next_bias, next_eps, (T*)next_out, next_stride, hidden)
     if (next_kind == 0 || next_dtype == FW_F32) {
         if (held) FW_JOIN_LAUNCH(float, true);
         else FW_JOIN_LAUNCH(float, false);

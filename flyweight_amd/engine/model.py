@@ -14,6 +14,7 @@ from ..config import ModelSpec, load_config
 from ..config.spec import ConfigError
 from ..kernels import ops
 from ..parts import Linear, build_part
+from ..parts.input_join import InputJoin
 from ..parts.norm import LazyNorm
 from ..parts.base import _REGISTRIES
 from ..weights.loader import TensorDecl, load_tensors
@@ -43,6 +44,7 @@ class CausalLM:
                 raise ConfigError(f"unknown block arrangement '{layer.arrangement}'")
             self.layers.append(_REGISTRIES["block"][layer.arrangement](layer))
         self.final_norm = build_part("norm", spec.final_norm)
+        self.input_join = InputJoin(spec.input_join) if spec.input_join is not None else None
         self.bound = False
 
     # ----- tensors ----------------------------------------------------------------------
@@ -53,6 +55,8 @@ class CausalLM:
             declared[spec.position_table_name] = TensorDecl((spec.max_positions, spec.hidden_size))
         for block in self.layers:
             declared.update(block.tensors())
+        if self.input_join is not None:
+            declared.update(self.input_join.tensors())
         declared.update(self.final_norm.tensors())
         if spec.lm_head_name is not None:
             declared[spec.lm_head_name] = TensorDecl((spec.vocab_size, spec.hidden_size))
@@ -68,6 +72,8 @@ class CausalLM:
         self.head = Linear(head)
         for block in self.layers:
             block.bind(tensors, dtype, device)
+        if self.input_join is not None:
+            self.input_join.bind(tensors, dtype, device)
         self.final_norm.bind(tensors, dtype, device)
         self.bound = True
 
@@ -126,9 +132,18 @@ class CausalLM:
         # what it gives and what the launches give stay bit for bit the same.)
         every_row = bool(ctx.all_decode)
         prepared = None
+        joined = self.input_join.start(x) if any(entry.joins_input for entry in schedule) else None
         for at, entry in enumerate(schedule):
-            # the norm that reads the residual after this layer, for the layer's last product
-            if at + 1 < len(schedule):
+            if entry.joins_input:
+                x = self.input_join.forward(x, joined)
+                prepared = None
+            elif joined is not None:
+                joined.current = False      # the layer changes the stream
+            # what reads the residual after this layer, for the layer's last product or sum: the map that joins the
+            # model's input again, or a norm
+            if at + 1 < len(schedule) and schedule[at + 1].joins_input:
+                norm_after = joined
+            elif at + 1 < len(schedule):
                 norm_after = self.layers[schedule[at + 1].layer].first_norm()
             else:
                 norm_after = self.final_norm if every_row else None

@@ -16,11 +16,11 @@ import torch
 
 from . import build as _build
 
-F32, BF16 = 0, 1
+F32, BF16, BF16_GELU = 0, 1, 2     # (the last: what a storing product leaves as gelu of its float32 sums)
 PAGE_SIZE = 64          # tokens per cache page: the width of a wavefront
 MAX_HEAD_DIM = 256          # of the matrix-core attention kernels
 MAX_PLAIN_HEAD_DIM = 1024   # of the plain attention kernels, which serve what the others do not take
-ABI_VERSION = 16
+ABI_VERSION = 17
 
 _lib = None
 
@@ -151,6 +151,11 @@ def _dev_rows(t: torch.Tensor, name: str) -> None:
         raise KernelError("kernels run on the GPU only; got a CPU tensor")
     if t.dim() != 2 or t.stride(1) != 1:
         raise KernelError(f"{name} must be a matrix with contiguous rows")
+
+
+def _stride(t: torch.Tensor) -> int:
+    """Elements between the rows of a matrix (of a single row: its width)."""
+    return t.stride(0) if t.shape[0] > 1 else max(t.shape[1], t.stride(0))
 
 
 def _p(t: Optional[torch.Tensor]) -> ctypes.c_void_p:
@@ -351,11 +356,13 @@ def qk_norm_rope_kv_write(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, 
                           row_seg: torch.Tensor, row_pos: torch.Tensor, write_kv: bool = True,
                           v_dim: Optional[int] = None, interleaved: bool = False, q_only: bool = False,
                           q_row_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """The output and the cache take the pages' dtype; ``qkv`` may be float32 beside bfloat16 pages.
+    """The output and the cache take the pages' dtype; ``qkv`` may be float32 beside bfloat16 pages, and its rows may lie
+    apart (some columns of wider rows).
     ``q_row_scale`` (float32 [rows]): a factor on each row's finished queries.
     ``v_dim``: the size of a value head where it is not ``head_dim``. ``interleaved``: channel 2i turns
     with channel 2i + 1 instead of channel i with channel i + rotary_dim / 2."""
-    _dev(qkv, q_norm_weight, k_norm_weight, cos, sin, k_pages, v_pages, block_table, row_seg, row_pos)
+    _dev(q_norm_weight, k_norm_weight, cos, sin, k_pages, v_pages, block_table, row_seg, row_pos)
+    _dev_rows(qkv, "qkv")
     rows, width = qkv.shape
     v_dim = head_dim if v_dim is None else int(v_dim)
     expected = num_heads * head_dim if q_only else (num_heads + num_kv_heads) * head_dim + num_kv_heads * v_dim
@@ -380,7 +387,7 @@ def qk_norm_rope_kv_write(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, 
     q_out = torch.empty((rows, num_heads * head_dim), dtype=k_pages.dtype, device=qkv.device)
     _row_scale(q_row_scale, rows)
     _check(library().fw_qk_norm_rope_kv_write(
-        _p(qkv), _code(qkv.dtype), _p(q_out), _code(k_pages.dtype), _p(q_norm_weight), _p(k_norm_weight), ctypes.c_float(eps), _p(cos), _p(sin),
+        _p(qkv), _code(qkv.dtype), _stride(qkv), _p(q_out), _code(k_pages.dtype), _p(q_norm_weight), _p(k_norm_weight), ctypes.c_float(eps), _p(cos), _p(sin),
         rotary_dim, _p(k_pages), _p(v_pages), _p(block_table), block_table.shape[1], _p(row_seg), _p(row_pos), rows,
         num_heads, num_kv_heads, head_dim, v_dim, PAGE_SIZE, pages, int(write_kv), int(interleaved), int(q_only), _p(q_row_scale), _stream()))
     return q_out
@@ -708,7 +715,7 @@ def gemm_medium(a: torch.Tensor, w: torch.Tensor, epilogue: int, *, bias: Option
                 out_dtype: Optional[torch.dtype] = None, accumulate_into: Optional[torch.Tensor] = None,
                 squares: Optional[torch.Tensor] = None, eps: float = 0.0,
                 next_norm_weight: Optional[torch.Tensor] = None, next_one_centered: bool = False,
-                w_tiled: Optional[torch.Tensor] = None, glu: Optional[tuple] = None):
+                w_tiled: Optional[torch.Tensor] = None, glu: Optional[tuple] = None, gelu: bool = False):
     """The medium product with the fused decode product's conventions (EPILOGUE_STORE /
     ACCUMULATE / SWIGLU): returns the output, or for an accumulation with ``next_norm_weight``
     what the norm after it needs. ``glu`` (with EPILOGUE_SWIGLU): (limit, alpha, shift) of a gated
@@ -734,7 +741,9 @@ def gemm_medium(a: torch.Tensor, w: torch.Tensor, epilogue: int, *, bias: Option
         return accumulate_into if left is None else left
     out_dtype = torch.bfloat16 if epilogue == EPILOGUE_SWIGLU else (out_dtype or torch.bfloat16)
     out = torch.empty((M, N), dtype=out_dtype, device=a.device)
-    gemm_medium_into(a, w, bias, out, _code(out_dtype), epilogue, N, squares=squares, eps=eps, w_tiled=w_tiled, glu=glu)
+    if gelu and (epilogue != EPILOGUE_STORE or out_dtype != torch.bfloat16):
+        raise KernelError("gemm_medium: gelu goes with a storing product of bfloat16")
+    gemm_medium_into(a, w, bias, out, BF16_GELU if gelu else _code(out_dtype), epilogue, N, squares=squares, eps=eps, w_tiled=w_tiled, glu=glu)
     return out
 
 
@@ -769,10 +778,15 @@ def _fast_ok(a: torch.Tensor, w: torch.Tensor) -> bool:
 # ---- dispatch: which kernel serves a call ------------------------------------------------
 def gemm(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None,
          out_dtype: Optional[torch.dtype] = None, accumulate_into: Optional[torch.Tensor] = None,
-         w_tiled: Optional[torch.Tensor] = None) -> torch.Tensor:
+         w_tiled: Optional[torch.Tensor] = None, gelu: bool = False) -> torch.Tensor:
     """a [M, K] . w [N, K]^T (+ bias): bfloat16 operands go to the matrix-core kernels,
     everything else (float32, mixed) to the generic float32 one. ``w_tiled``: ``w`` once more in
-    operand tiles (``tile_weights``), for the kernels of few rows that read it so."""
+    operand tiles (``tile_weights``), for the kernels of few rows that read it so. ``gelu``: the error-function gelu of
+    the float32 sums, rounded once (the matrix-core products form it as they store)."""
+    if gelu and accumulate_into is not None:
+        raise KernelError("gemm: gelu goes with a product that stores")
+    if gelu and (not _fast_ok(a, w) or (out_dtype or a.dtype) != torch.bfloat16):
+        return gelu_rows(gemm(a, w, bias, out_dtype=torch.float32, w_tiled=w_tiled), out_dtype or a.dtype)
     if not _fast_ok(a, w):
         return gemm_generic(a, w, bias, out_dtype=out_dtype, accumulate_into=accumulate_into)
     _dev(a, w, bias, accumulate_into)
@@ -790,7 +804,7 @@ def gemm(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None,
         return accumulate_into
     out_dtype = out_dtype or a.dtype
     out = torch.empty((M, N), dtype=out_dtype, device=a.device)
-    _fast_gemm(a, w, bias, out, _code(out_dtype), 0, N, w_tiled)
+    _fast_gemm(a, w, bias, out, BF16_GELU if gelu else _code(out_dtype), 0, N, w_tiled)
     return out
 
 
@@ -839,9 +853,10 @@ def gemm_decode(a: torch.Tensor, w: torch.Tensor, epilogue: int, *, bias: Option
                 conv_bias: Optional[torch.Tensor] = None, state: Optional[torch.Tensor] = None,
                 seg_slot: Optional[torch.Tensor] = None, squares: Optional[torch.Tensor] = None,
                 next_norm_weight: Optional[torch.Tensor] = None, next_one_centered: bool = False,
-                w_tiled: Optional[torch.Tensor] = None, glu: Optional[tuple] = None):
+                w_tiled: Optional[torch.Tensor] = None, glu: Optional[tuple] = None, gelu: bool = False):
     """One kernel for (optional RMS norm of float32 rows) -> product with bfloat16 ``w`` -> epilogue.
-    ``glu`` (with EPILOGUE_SWIGLU): (limit, alpha, shift) of a gated unit with clamped halves.
+    ``glu`` (with EPILOGUE_SWIGLU): (limit, alpha, shift) of a gated unit with clamped halves. ``gelu`` (EPILOGUE_STORE,
+    bfloat16, no norm in front): the error-function gelu of the sums is stored.
     With ``norm_weight`` ``a`` holds float32 rows (gathered through ``row_index`` if given), else
     bfloat16 activations. With ``next_norm_weight`` the accumulating epilogue also leaves what
     the norm after it needs, and the call returns (activations x * w_next, sums of squares);
@@ -902,11 +917,13 @@ def gemm_decode(a: torch.Tensor, w: torch.Tensor, epilogue: int, *, bias: Option
         next_activations = torch.empty((rows, N), dtype=torch.bfloat16, device=a.device)
         next_squares = torch.empty((library().fw_gemm_decode_accumulate_tiles(N), 16), dtype=torch.float32, device=a.device)
     prologue = 1 if normed else (2 if squares is not None else 0)
+    if gelu and (epilogue != EPILOGUE_STORE or out_dtype != torch.bfloat16 or prologue):
+        raise KernelError("gemm_decode: gelu goes with a plain storing product of bfloat16")
     w_tiled = _tiled_for(w, w_tiled)
     _check(library().fw_gemm_decode(
         prologue, _p(a), _p(norm_weight), _p(row_index), ctypes.c_float(eps), int(one_centered),
         _p(w if w_tiled is None else w_tiled), int(w_tiled is not None), _p(bias),
-        _p(target), _code(out_dtype), int(epilogue), rows, N, K, _p(taps), _p(conv_bias), _p(state), _p(seg_slot),
+        _p(target), BF16_GELU if gelu else _code(out_dtype), int(epilogue), rows, N, K, _p(taps), _p(conv_bias), _p(state), _p(seg_slot),
         int(kernel_size), _p(next_norm_weight), int(next_one_centered), _p(next_activations), _p(next_squares),
         _p(squares), 0 if squares is None else squares.shape[0], *_glu(glu), _stream()))
     if next_norm_weight is not None:
@@ -1121,6 +1138,154 @@ def attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,
                              ctx.row_pos, scale, window, v_dim=v_dim, chunk=chunk, softcap=softcap, keep_first=keep_first, sinks=sinks, slopes=slopes)
 
 
+# ---- attention whose weights are sigmoids and whose heads mix them ------------------------------------------
+SIGMOID_MAX_HEADS = 256         # of the plain kernel (the matrix-core kernels: see sigmoid_attention_is_tiled)
+SIGMOID_DECODE_WORKGROUPS = 512     # two per compute unit: up to here every page of a row gets a workgroup of its own
+
+
+def sigmoid_attention_is_tiled(num_heads: int, head_dim: int, v_dim: int) -> bool:
+    """Whether bfloat16 runs on the matrix-core kernels: up to 16 heads, sizes in steps of 16, all heads of 16 rows in LDS."""
+    return bool(library().fw_sigmoid_attention_fits(int(num_heads), int(head_dim), int(v_dim)))
+
+
+def _sigmoid_checks(num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, k_pages: torch.Tensor, v_pages: torch.Tensor,
+                    block_table: torch.Tensor, row_seg: Optional[torch.Tensor], row_pos: torch.Tensor, rows: int, bias: torch.Tensor,
+                    mix: torch.Tensor, gate: Optional[torch.Tensor]):
+    _dev(k_pages, v_pages, block_table, row_seg, row_pos, bias, mix)
+    pages = _check_pages(k_pages, v_pages, num_kv_heads, head_dim, k_pages.dtype, v_dim)
+    for name, t in (("block_table", block_table), ("row_seg", row_seg), ("row_pos", row_pos)):
+        if t is not None:
+            _want(t, torch.int32, name)
+    if block_table.dim() != 2 or (row_seg is not None and row_seg.numel() < rows) or row_pos.numel() < rows:
+        raise KernelError("sigmoid_attention: batch index arrays are too short")
+    for name, t, shape in (("bias", bias, (num_heads,)), ("mix", mix, (num_heads, num_heads))):
+        _want(t, torch.float32, name)
+        if t.shape != shape:
+            raise KernelError(f"sigmoid_attention: {name} is {tuple(t.shape)}, expected {shape}")
+    if gate is not None:
+        _dev_rows(gate, "gate")
+        if gate.dtype != torch.float32 or gate.shape != (rows, num_heads * v_dim):
+            raise KernelError(f"sigmoid_attention: the gate is {tuple(gate.shape)} {gate.dtype}, expected {(rows, num_heads * v_dim)} float32")
+    return pages
+
+
+def sigmoid_attention_generic(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, k_pages: torch.Tensor,
+                              v_pages: torch.Tensor, block_table: torch.Tensor, row_seg: torch.Tensor, row_pos: torch.Tensor,
+                              scale: float, window: int, bias: torch.Tensor, mix: torch.Tensor,
+                              gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """a_g = sigmoid(q_g . k * scale + bias[g]) over the visible keys, heads mixed by ``mix`` [heads, heads], the weighted
+    sums of the values times sigmoid(``gate``) (float32 [rows, heads * v_dim], rows may lie apart; None: no gate)."""
+    rows = q.shape[0]
+    _dev(q)
+    if q.shape != (rows, num_heads * head_dim) or q.dtype != k_pages.dtype:
+        raise KernelError(f"sigmoid_attention: q is {tuple(q.shape)} {q.dtype}, expected {(rows, num_heads * head_dim)} {k_pages.dtype}")
+    pages = _sigmoid_checks(num_heads, num_kv_heads, head_dim, v_dim, k_pages, v_pages, block_table, row_seg, row_pos, rows, bias, mix, gate)
+    out = torch.empty((rows, num_heads * v_dim), dtype=q.dtype, device=q.device)
+    _check(library().fw_sigmoid_attention_generic(
+        _p(q), _p(out), _code(q.dtype), _p(k_pages), _p(v_pages), _p(block_table), block_table.shape[1], _p(row_seg), _p(row_pos), rows,
+        num_heads, num_kv_heads, head_dim, v_dim, ctypes.c_float(scale), int(window), _p(bias), _p(mix), _p(gate),
+        _stride(gate) if gate is not None else 0, PAGE_SIZE, pages, _stream()))
+    return out
+
+
+def sigmoid_attention_prefill(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, k_pages: torch.Tensor,
+                              v_pages: torch.Tensor, block_table: torch.Tensor, tile_seg: torch.Tensor, tile_row0: torch.Tensor,
+                              seg_row0: torch.Tensor, row_pos: torch.Tensor, scale: float, window: int, bias: torch.Tensor,
+                              mix: torch.Tensor, gate: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The same on the matrix cores for the rows of the given tiles (of up to 64 rows; ``attention_prefill``)."""
+    rows = q.shape[0]
+    _dev(q, tile_seg, tile_row0, seg_row0)
+    _want(q, torch.bfloat16, "q")
+    for name, t in (("tile_seg", tile_seg), ("tile_row0", tile_row0), ("seg_row0", seg_row0)):
+        _want(t, torch.int32, name)
+    if q.shape != (rows, num_heads * head_dim) or k_pages.dtype != torch.bfloat16 or tile_seg.numel() != tile_row0.numel():
+        raise KernelError(f"sigmoid_attention: q is {tuple(q.shape)}, pages {k_pages.dtype}, {tile_seg.numel()} / {tile_row0.numel()} tiles")
+    pages = _sigmoid_checks(num_heads, num_kv_heads, head_dim, v_dim, k_pages, v_pages, block_table, None, row_pos, rows, bias, mix, gate)
+    if out is None:
+        out = torch.empty((rows, num_heads * v_dim), dtype=q.dtype, device=q.device)
+    elif out.shape != (rows, num_heads * v_dim) or out.dtype != q.dtype or not out.is_contiguous():
+        raise KernelError("sigmoid_attention: out must be bfloat16 [rows, heads * v_dim]")
+    _check(library().fw_sigmoid_attention_prefill(
+        _p(q), _p(out), _p(k_pages), _p(v_pages), _p(block_table), block_table.shape[1], _p(tile_seg), _p(tile_row0), tile_seg.numel(),
+        _p(seg_row0), _p(row_pos), rows, num_heads, num_kv_heads, head_dim, v_dim, ctypes.c_float(scale), int(window), _p(bias), _p(mix),
+        _p(gate), _stride(gate) if gate is not None else 0, PAGE_SIZE, pages, _stream()))
+    return out
+
+
+def sigmoid_decode_splits(rows: int, max_context: int, window: int):
+    """(workgroups a row's visible pages are cut into at most, pages each of them takes)."""
+    blocks = (max_context + PAGE_SIZE - 1) // PAGE_SIZE
+    if window > 0:
+        blocks = min(blocks, (window + PAGE_SIZE - 2) // PAGE_SIZE + 1)
+    each = max(1, rows * blocks // SIGMOID_DECODE_WORKGROUPS)
+    return (blocks + each - 1) // each, each
+
+
+def sigmoid_attention_decode(num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, k_pages: torch.Tensor, v_pages: torch.Tensor,
+                             block_table: torch.Tensor, row_seg: torch.Tensor, row_pos: torch.Tensor, scale: float, window: int,
+                             bias: torch.Tensor, mix: torch.Tensor, max_context: int, gate: Optional[torch.Tensor] = None,
+                             q: Optional[torch.Tensor] = None, qkv: Optional[torch.Tensor] = None, qk_norm: bool = True, eps: float = 0.0,
+                             write_kv: bool = True, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """One row per request on the matrix cores; ``max_context`` bounds position + 1 of every row. From finished queries
+    ``q`` (bfloat16), or from the raw projections ``qkv`` (float32 [rows, q | k | v], rows may lie apart): queries and keys of a
+    head divided by their root mean square (``qk_norm``, ``eps``) and the new keys and values stored (``write_kv``) in the same
+    kernel."""
+    if (q is None) == (qkv is None):
+        raise KernelError("sigmoid_attention: finished queries or raw projections, one of the two")
+    rows = (q if q is not None else qkv).shape[0]
+    if q is not None:
+        _dev(q)
+        _want(q, torch.bfloat16, "q")
+        if q.shape != (rows, num_heads * head_dim):
+            raise KernelError(f"sigmoid_attention: q is {tuple(q.shape)}, expected {(rows, num_heads * head_dim)}")
+    else:
+        _dev_rows(qkv, "qkv")
+        _want(qkv, torch.float32, "qkv")
+        expected = (num_heads + num_kv_heads) * head_dim + num_kv_heads * v_dim
+        if qkv.shape != (rows, expected):
+            raise KernelError(f"sigmoid_attention: qkv is {tuple(qkv.shape)}, expected {(rows, expected)}")
+    if k_pages.dtype != torch.bfloat16:
+        raise KernelError("sigmoid_attention: the matrix-core kernels work on a bfloat16 cache")
+    pages = _sigmoid_checks(num_heads, num_kv_heads, head_dim, v_dim, k_pages, v_pages, block_table, row_seg, row_pos, rows, bias, mix, gate)
+    splits, each = sigmoid_decode_splits(rows, max_context, window)
+    partial = torch.empty((rows, splits, num_heads * v_dim), dtype=torch.float32, device=k_pages.device) if splits > 1 else None
+    tickets = _medium_counters(k_pages.device, rows)
+    if out is None:
+        out = torch.empty((rows, num_heads * v_dim), dtype=torch.bfloat16, device=k_pages.device)
+    elif out.shape != (rows, num_heads * v_dim) or out.dtype != torch.bfloat16 or not out.is_contiguous():
+        raise KernelError("sigmoid_attention: out must be bfloat16 [rows, heads * v_dim]")
+    _check(library().fw_sigmoid_attention_decode(
+        _p(q), _p(qkv), _stride(qkv) if qkv is not None else 0, int(qk_norm), ctypes.c_float(eps), int(write_kv), _p(out), _p(partial), splits,
+        each, int(max_context), _p(tickets), tickets.numel(), _p(k_pages), _p(v_pages), _p(block_table), block_table.shape[1], _p(row_seg),
+        _p(row_pos), rows, num_heads, num_kv_heads, head_dim, v_dim, ctypes.c_float(scale), int(window), _p(bias), _p(mix), _p(gate),
+        _stride(gate) if gate is not None else 0, PAGE_SIZE, pages, _stream()))
+    return out
+
+
+def sigmoid_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, k_pages: torch.Tensor,
+                      v_pages: torch.Tensor, block_table: torch.Tensor, ctx, scale: float, window: int, bias: torch.Tensor,
+                      mix: torch.Tensor, gate: Optional[torch.Tensor] = None, tile_seg: Optional[torch.Tensor] = None,
+                      tile_row0: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The step's rows: bfloat16 in sizes the matrix-core kernels take goes to the decode kernel for segments of one row
+    (all of them, or those a mixed step begins with) and to the tiled kernel for the rest; everything else to the plain one."""
+    if q.dtype != torch.bfloat16 or not sigmoid_attention_is_tiled(num_heads, head_dim, v_dim):
+        return sigmoid_attention_generic(q, num_heads, num_kv_heads, head_dim, v_dim, k_pages, v_pages, block_table, ctx.row_seg, ctx.row_pos,
+                                         scale, window, bias, mix, gate)
+    rows = q.shape[0]
+    single = rows if ctx.all_decode else getattr(ctx, "decode_prefix", 0)
+    out = torch.empty((rows, num_heads * v_dim), dtype=q.dtype, device=q.device)
+    if single:
+        sigmoid_attention_decode(num_heads, num_kv_heads, head_dim, v_dim, k_pages, v_pages, block_table, ctx.row_seg, ctx.row_pos, scale,
+                                 window, bias, mix, ctx.max_context, gate=gate[:single] if gate is not None else None, q=q[:single],
+                                 out=out[:single])
+    if single < rows:
+        if tile_seg is None or tile_row0 is None:
+            raise KernelError("sigmoid_attention: the tiled kernel needs the step's query tiles")
+        sigmoid_attention_prefill(q, num_heads, num_kv_heads, head_dim, v_dim, k_pages, v_pages, block_table, tile_seg[single:],
+                                  tile_row0[single:], ctx.seg_row0, ctx.row_pos, scale, window, bias, mix, gate, out=out)
+    return out
+
+
 # ---- the gated delta rule -----------------------------------------------------------------------------
 def delta_prepare(proj: torch.Tensor, beta_col: int, a: torch.Tensor, taps: torch.Tensor, conv_state: torch.Tensor,
                   A_log: torch.Tensor, dt_bias: torch.Tensor, row_seg: torch.Tensor, seg_row0: torch.Tensor,
@@ -1261,38 +1426,41 @@ NEXT_NOTHING, NEXT_ROUNDED, NEXT_RMS, NEXT_CENTERED = 0, 1, 2, 3
 
 
 def layernorm_rows(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype,
-                   row_index: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """(x - mean) / sqrt(mean((x - mean)^2) + eps) * weight over float32 rows (gathered through
+                   row_index: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """(x - mean) / sqrt(mean((x - mean)^2) + eps) * weight (+ bias) over float32 rows (gathered through
     ``row_index`` if given), in ``out_dtype``."""
-    _dev(x, weight, row_index)
+    _dev(x, weight, row_index, bias)
     _want(x, torch.float32, "x")
-    _want(weight, torch.float32, "weight")
     hidden = x.shape[-1]
-    if weight.shape != (hidden,):
-        raise KernelError(f"layernorm: weight is {tuple(weight.shape)}, row width is {hidden}")
+    for name, t in (("weight", weight), ("bias", bias)):
+        if t is not None:
+            _want(t, torch.float32, name)
+            if t.shape != (hidden,):
+                raise KernelError(f"layernorm: {name} is {tuple(t.shape)}, row width is {hidden}")
     rows = x.numel() // hidden if row_index is None else row_index.numel()
     if row_index is not None:
         _want(row_index, torch.int32, "row_index")
     out = torch.empty((rows, hidden), dtype=out_dtype, device=x.device)
-    _check(library().fw_layernorm_rows(_p(x), _p(weight), _p(out), _code(out_dtype), _p(row_index), rows, hidden,
+    _check(library().fw_layernorm_rows(_p(x), _p(weight), _p(bias), _p(out), _code(out_dtype), _p(row_index), rows, hidden,
                                        ctypes.c_float(eps), _stream()))
     return out
 
 
 def norm_add_norm_(x: torch.Tensor, a: torch.Tensor, weight: torch.Tensor, centered: bool, eps: float, *,
-                   next_kind: int = NEXT_NOTHING, next_weight: Optional[torch.Tensor] = None, next_eps: float = 0.0,
-                   next_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
-    """x += norm(a) * weight in place (float32 rows; ``centered``: the row's mean is taken off before its
-    root mean square). What reads x next is formed from the new rows in the same kernel and returned:
-    ``NEXT_ROUNDED`` the rows in ``next_dtype``, ``NEXT_RMS`` / ``NEXT_CENTERED`` their norm with
-    ``next_weight`` and ``next_eps``; ``NEXT_NOTHING`` returns None."""
-    _dev(x, a, weight, next_weight)
+                   bias: Optional[torch.Tensor] = None, mult: float = 1.0, next_kind: int = NEXT_NOTHING,
+                   next_weight: Optional[torch.Tensor] = None, next_bias: Optional[torch.Tensor] = None, next_eps: float = 0.0,
+                   next_dtype: Optional[torch.dtype] = None, next_out: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """x += mult * (norm(a) * weight + bias) in place (float32 rows; ``bias`` optional; ``centered``: the row's mean is
+    taken off before its root mean square). What reads x next is formed from the new rows in the same kernel and
+    returned: ``NEXT_ROUNDED`` the rows in ``next_dtype``, ``NEXT_RMS`` / ``NEXT_CENTERED`` their norm with ``next_weight``,
+    ``next_bias`` (optional) and ``next_eps``, into ``next_out`` if given (rows may lie apart); ``NEXT_NOTHING`` returns None."""
+    _dev(x, a, weight, bias, next_weight, next_bias)
     rows, hidden = x.shape
     for name, t in (("x", x), ("a", a)):
         _want(t, torch.float32, name)
         if t.shape != (rows, hidden):
             raise KernelError(f"norm_add_norm: {name} is {tuple(t.shape)}, expected {(rows, hidden)}")
-    for name, t in (("weight", weight), ("next_weight", next_weight)):
+    for name, t in (("weight", weight), ("bias", bias), ("next_weight", next_weight), ("next_bias", next_bias)):
         if t is not None:
             _want(t, torch.float32, name)
             if t.shape != (hidden,):
@@ -1303,10 +1471,35 @@ def norm_add_norm_(x: torch.Tensor, a: torch.Tensor, weight: torch.Tensor, cente
         raise KernelError("norm_add_norm: the norm that follows needs its weight")
     out = None
     if next_kind != NEXT_NOTHING:
-        out = torch.empty((rows, hidden), dtype=next_dtype or torch.float32, device=x.device)
-    _check(library().fw_norm_add_norm(_p(x), _p(a), _p(weight), int(centered), ctypes.c_float(eps), int(next_kind), _p(next_weight),
-                                      ctypes.c_float(next_eps), _p(out), _code(out.dtype) if out is not None else F32, rows, hidden,
+        out = next_out
+        if out is None:
+            out = torch.empty((rows, hidden), dtype=next_dtype or torch.float32, device=x.device)
+        _dev_rows(out, "next_out")
+        if out.shape != (rows, hidden) or (next_dtype is not None and out.dtype != next_dtype):
+            raise KernelError(f"norm_add_norm: next_out is {tuple(out.shape)} {out.dtype}, expected {(rows, hidden)} {next_dtype}")
+    _check(library().fw_norm_add_norm(_p(x), _p(a), _p(weight), _p(bias), ctypes.c_float(mult), int(centered), ctypes.c_float(eps),
+                                      int(next_kind), _p(next_weight), _p(next_bias), ctypes.c_float(next_eps), _p(out),
+                                      _code(out.dtype) if out is not None else F32, _stride(out) if out is not None else 0, rows, hidden,
                                       _stream()))
+    return out
+
+
+def place_rows(x: torch.Tensor, out: torch.Tensor, col0: int = 0, twice: bool = False) -> torch.Tensor:
+    """float32 rows into columns ``col0`` .. of the wider rows ``out``, in its dtype; ``twice``: once more behind them."""
+    _dev(x, out)
+    _want(x, torch.float32, "x")
+    if x.dim() != 2 or out.dim() != 2 or out.shape[0] != x.shape[0]:
+        raise KernelError(f"place_rows: {tuple(x.shape)} into {tuple(out.shape)}")
+    _check(library().fw_place_rows(_p(x), _p(out), _code(out.dtype), x.shape[0], x.shape[1], out.shape[1], int(col0), int(twice), _stream()))
+    return out
+
+
+def gelu_rows(z: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """z Phi(z) (the error-function gelu) of float32 values, in ``out_dtype``."""
+    _dev(z)
+    _want(z, torch.float32, "z")
+    out = torch.empty(z.shape, dtype=out_dtype, device=z.device)
+    _check(library().fw_gelu_rows(_p(z), _p(out), _code(out_dtype), ctypes.c_longlong(z.numel()), _stream()))
     return out
 
 
@@ -1328,11 +1521,12 @@ def gelu_gate_rows(z: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, col0
 # ---- attention over a cached latent ------------------------------------------------------------------------
 def latent_norm_write(raw: torch.Tensor, weight: torch.Tensor, eps: float, k_pages: torch.Tensor, v_pages: torch.Tensor,
                       block_table: torch.Tensor, row_seg: torch.Tensor, row_pos: torch.Tensor, rot: int = 0,
-                      cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None, turn: Optional[int] = None) -> None:
+                      cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None, turn: Optional[int] = None,
+                      interleaved: bool = True) -> None:
     """The step's latents ``raw`` (float32 [rows, rank + rot]; a view of some columns of wider rows will do): the first
     rank columns RMS-normed times ``weight`` and stored at each row's position in a cache of one key/value head; the last
-    ``rot`` columns (a key part all heads share) turned by the row's angles (neighbouring channels paired; ``cos``, ``sin``
-    float32 [rows, rot / 2]) and stored behind the latent in the keys' layout, whose head then has rank + rot channels."""
+    ``rot`` columns (a key part all heads share) turned by the row's angles (``interleaved``: neighbouring channels paired,
+    else channel i with channel i + turn / 2; ``cos``, ``sin`` float32 [rows, turn / 2]) and stored behind the latent in the keys' layout, whose head then has rank + rot channels."""
     _dev(weight, k_pages, v_pages, block_table, row_seg, row_pos, cos, sin)
     _dev_rows(raw, "raw")
     _want(raw, torch.float32, "raw")
@@ -1352,14 +1546,14 @@ def latent_norm_write(raw: torch.Tensor, weight: torch.Tensor, eps: float, k_pag
         raise KernelError("latent_norm_write: batch index arrays are too short")
     _check(library().fw_latent_norm_write(_p(raw), raw.stride(0) if rows > 1 else max(rank + int(rot), raw.stride(0)), 0, _p(weight),
                                           ctypes.c_float(eps), _p(k_pages), _p(v_pages), _code(k_pages.dtype), _p(block_table),
-                                          block_table.shape[1], _p(row_seg), _p(row_pos), rows, rank, int(rot), turn, _p(cos), _p(sin),
+                                          block_table.shape[1], _p(row_seg), _p(row_pos), rows, rank, int(rot), turn, int(interleaved), _p(cos), _p(sin),
                                           PAGE_SIZE, pages, _stream()))
 
 
 def head_linear(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, gate: Optional[torch.Tensor] = None,
                 in_head: Optional[int] = None, out: Optional[torch.Tensor] = None, out_head: Optional[int] = None) -> torch.Tensor:
     """A map per head: ``x`` [rows, heads K] (rows may lie apart), ``w`` [heads, N, K] -> [rows, heads N], with
-    ``gate`` (float32 [rows, heads N], rows may lie apart) times its sigmoid. ``in_head``: a head's vector in ``x`` holds
+    ``gate`` (float32 [rows, heads N], or [rows, heads]: one number a head; rows may lie apart) times its sigmoid. ``in_head``: a head's vector in ``x`` holds
     that many channels of which the map reads the first K; ``out`` with ``out_head``: the results go to the first N
     channels of each head's vector of ``out_head`` channels in the rows of ``out``."""
     _dev(w)
@@ -1371,8 +1565,8 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, gate: 
         raise KernelError(f"head_linear: x is {tuple(x.shape)}, the weight {tuple(w.shape)}, a head's vector {in_head}")
     if gate is not None:
         _dev_rows(gate, "gate")
-        if gate.shape != (rows, heads * N) or gate.dtype != torch.float32:
-            raise KernelError(f"head_linear: the gate is {tuple(gate.shape)} {gate.dtype}, expected {(rows, heads * N)} float32")
+        if gate.shape not in ((rows, heads * N), (rows, heads)) or gate.dtype != torch.float32:
+            raise KernelError(f"head_linear: the gate is {tuple(gate.shape)} {gate.dtype}, expected {(rows, heads * N)} or {(rows, heads)} float32")
     out_head = N if out_head is None else int(out_head)
     if out is None:
         out = torch.empty((rows, heads * out_head), dtype=out_dtype, device=x.device)
@@ -1385,15 +1579,16 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, gate: 
         return t.stride(0) if rows > 1 else max(width, t.stride(0))
 
     _check(library().fw_head_linear(_p(x), _code(x.dtype), stride(x, heads * in_head), _p(w), _code(w.dtype), _p(gate),
-                                    stride(gate, heads * N) if gate is not None else 0, _p(out), _code(out_dtype), rows, heads, N, K,
+                                    stride(gate, gate.shape[1]) if gate is not None else 0,
+                                    int(gate is not None and gate.shape[1] == heads and N > 1), _p(out), _code(out_dtype), rows, heads, N, K,
                                     in_head, out_head, heads * out_head, _stream()))
     return out
 
 
 def rotate_place(x: torch.Tensor, heads: int, col0: int, rot: int, cos: torch.Tensor, sin: torch.Tensor, out: torch.Tensor,
-                 out_col0: int, turn: Optional[int] = None) -> torch.Tensor:
+                 out_col0: int, turn: Optional[int] = None, interleaved: bool = True) -> torch.Tensor:
     """Channels col0 .. col0 + rot - 1 of every head's vector in ``x`` [rows, heads * in_head], neighbouring channels
-    turned by the row's angles (``cos``, ``sin`` float32 [rows, rot / 2]), stored from channel ``out_col0`` of the head's
+    (``interleaved``; else channels i and i + turn / 2) turned by the row's angles (``cos``, ``sin`` float32 [rows, rot / 2]), stored from channel ``out_col0`` of the head's
     vector in ``out`` [rows, heads * out_head]."""
     _dev(x, cos, sin, out)
     rows = x.shape[0]
@@ -1405,7 +1600,7 @@ def rotate_place(x: torch.Tensor, heads: int, col0: int, rot: int, cos: torch.Te
             raise KernelError(f"rotate_place: {turn} turned channels need float32 tables {(rows, turn // 2)}")
     _check(library().fw_rotate_place(_p(x), _code(x.dtype), x.shape[1], x.shape[1] // heads, int(col0), _p(cos), _p(sin), _p(out),
                                      _code(out.dtype), out.shape[1], out.shape[1] // heads, int(out_col0), rows, heads, int(rot), turn,
-                                     _stream()))
+                                     int(interleaved), _stream()))
     return out
 
 
@@ -1481,12 +1676,20 @@ def wkv_recurrence(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, a: torch.T
 
 
 # ---- a mixture of feed-forward units chosen per token ------------------------------------------------------------
+MOE_SCORES = ("softmax_chosen", "softmax_all", "sigmoid")
+
+
 def moe_route(logits: torch.Tensor, bias: Optional[torch.Tensor], top: int, groups: int = 1, keep: int = 1,
-              score_all: bool = False):
+              score_all: bool = False, scores: Optional[str] = None, group_pair: bool = False):
     """(chosen int32 [rows, top], weight float32 [rows, top]): the ``top`` largest of logits + bias per row, largest
     first (ties: the lowest id), and the softmax over those alone. ``groups`` > 1: only experts of the ``keep`` groups
     (of neighbours, equal in size) whose best expert scores highest can be chosen. ``score_all``: the weights are the
-    softmax over all experts at the chosen ones, divided by their sum + 1e-20."""
+    softmax over all experts at the chosen ones, divided by their sum + 1e-20. ``scores`` names the same choice
+    ("softmax_chosen", "softmax_all") or "sigmoid": each expert's own sigmoid at the chosen ones, divided by their sum + 1e-20.
+    ``group_pair``: a group's score is the sum of its two best experts' scores (not with "softmax_chosen")."""
+    scores = scores or ("softmax_all" if score_all else "softmax_chosen")
+    if scores not in MOE_SCORES or (group_pair and scores == "softmax_chosen"):
+        raise KernelError(f"moe_route: scores {scores!r} (known: {', '.join(MOE_SCORES)}; groups by pairs: {group_pair})")
     _dev(logits, bias)
     _want(logits, torch.float32, "logits")
     rows, experts = logits.shape
@@ -1495,7 +1698,7 @@ def moe_route(logits: torch.Tensor, bias: Optional[torch.Tensor], top: int, grou
     chosen = torch.empty((rows, top), dtype=torch.int32, device=logits.device)
     weight = torch.empty((rows, top), dtype=torch.float32, device=logits.device)
     _check(library().fw_moe_route(_p(logits), _p(bias), _p(chosen), _p(weight), rows, experts, int(top), int(groups), int(keep),
-                                  int(score_all), _stream()))
+                                  int(group_pair), MOE_SCORES.index(scores), _stream()))
     return chosen, weight
 
 

@@ -8,11 +8,11 @@ arrangement (post-norm, parallel mixer and feed-forward) is another class regist
 read x itself (rounded to the activation dtype for their products), the norm stands on a
 sublayer's OUTPUT, and m is a fixed factor. The feed-forward may be absent.
 
-``sandwich_norm_residual``: x <- x + post1(mixer(pre1(x))); x <- x + post2(ffn(pre2(x))), a norm before
-and a norm behind every sublayer; then, where the layer has one, the tokens' own input
+``sandwich_norm_residual``: x <- x + m * post1(mixer(pre1(x))); x <- x + m * post2(ffn(pre2(x))), a norm before
+and a norm behind every sublayer and m a fixed factor (1 unless given); then, where the layer has one, the tokens' own input
 (``parts/token_input.py``): x <- x + rms(y(x, token)) * w. The feed-forward may be absent. Every sum into
-x also forms what reads x next (the next norm's output, or x rounded) in the same kernel.
-
+x also forms what reads x next (the next norm's output, or x rounded, also in its place beside the model's input: see
+``parts/input_join.py``) in the same kernel.
 
 ``parallel_residual``: with h = norm1(x), x <- x + (mixer(h) + ffn(h)): one norm, and both sublayers read its
 output. The feed-forward may be absent.
@@ -23,6 +23,7 @@ from __future__ import annotations
 from ..config.spec import ConfigError
 from ..kernels import ops
 from .base import Block, build_part, register_block
+from .input_join import JoinedRows
 from .norm import LazyNorm, NormedRows
 from .token_input import TokenInput
 
@@ -137,7 +138,8 @@ class OutputNormResidualBlock(Block):
 @register_block("sandwich_norm_residual")
 class SandwichNormResidualBlock(Block):
     """``LayerSpec.params``: ``mixer_post_norm`` and ``ffn_post_norm`` (PartSpecs of norms), ``token_input``
-    (PartSpec of a :class:`TokenInput`, or absent). The norms may be RMS or layer norms, each on its own."""
+    (PartSpec of a :class:`TokenInput`, or absent), ``residual_mult`` (the factor m on both sublayers' normed outputs; the
+    tokens' own input takes none). The norms may be RMS or layer norms, each on its own."""
 
     def __init__(self, spec):
         self.spec = spec
@@ -147,6 +149,7 @@ class SandwichNormResidualBlock(Block):
         self.ffn = build_part("ffn", spec.ffn) if spec.ffn is not None else None
         self.ffn_norm = build_part("norm", spec.ffn_norm) if spec.ffn is not None else None
         self.ffn_post_norm = build_part("norm", spec.params["ffn_post_norm"]) if spec.ffn is not None else None
+        self.mult = float(spec.params.get("residual_mult", 1.0))
         given = spec.params.get("token_input")
         self.token_input = TokenInput(given) if given is not None else None
         for part in (self.mixer, self.ffn):
@@ -174,35 +177,40 @@ class SandwichNormResidualBlock(Block):
     @staticmethod
     def _reader(reader, dtype) -> dict:
         """What a kernel that sums into x is told about the next reader of x: a norm (its output), "rounded"
-        (x in the activation dtype) or None."""
+        (x in the activation dtype), rows in which x is to be joined with others (x in its columns of them) or None."""
         if reader is None:
             return {}
         if reader == "rounded":
             return {"next_kind": ops.NEXT_ROUNDED, "next_dtype": dtype}
-        next_weight, next_eps, next_centered = reader.row_norm()
-        return {"next_kind": ops.NEXT_CENTERED if next_centered else ops.NEXT_RMS, "next_weight": next_weight, "next_eps": next_eps,
-                "next_dtype": dtype}
+        if isinstance(reader, JoinedRows):
+            return {"next_kind": ops.NEXT_ROUNDED, "next_dtype": reader.rows.dtype, "next_out": reader.place}
+        norm = reader.row_norm()
+        return {"next_kind": ops.NEXT_CENTERED if norm.centered else ops.NEXT_RMS, "next_weight": norm.weight, "next_bias": norm.bias,
+                "next_eps": norm.eps, "next_dtype": dtype}
 
-    def _join(self, x, rows, norm, reader, dtype):
-        """x += norm(rows); returns what ``reader`` sees of the new x (None for no reader)."""
-        weight, eps, centered = norm.row_norm()
-        return ops.norm_add_norm_(x, rows, weight, centered, eps, **self._reader(reader, dtype))
+    def _join(self, x, rows, norm, reader, dtype, mult=1.0):
+        """x += mult * norm(rows); returns what ``reader`` sees of the new x (None for no reader)."""
+        own = norm.row_norm()
+        return ops.norm_add_norm_(x, rows, own.weight, own.centered, own.eps, bias=own.bias, mult=mult, **self._reader(reader, dtype))
 
     def forward(self, x, ctx, cache, prepared=None, norm_after=None):
         """``x`` [rows, hidden] float32 is updated in place."""
         dtype = self.mixer_norm.dtype
-        # a norm that follows this block is formed with the block's last sum only if it is of a form the kernel knows
-        after = norm_after if hasattr(norm_after, "row_norm") and norm_after.row_norm() is not None else None
+        # what follows this block is formed with the block's last sum only if it is of a form the kernel knows
+        known = isinstance(norm_after, JoinedRows) or (hasattr(norm_after, "row_norm") and norm_after.row_norm() is not None)
+        after = norm_after if known else None
         h = LazyNorm(self.mixer_norm, x, ctx, prepared=prepared).tensor()
         last = self.ffn is None and self.token_input is None
         reader = after if last else (self.ffn_norm if self.ffn is not None else "rounded")     # the token input's product reads x rounded
-        h = self._join(x, self.mixer.output(h, ctx, cache), self.mixer_post_norm, reader, dtype)
+        h = self._join(x, self.mixer.output(h, ctx, cache), self.mixer_post_norm, reader, dtype, self.mult)
         if self.ffn is not None:
             reader = after if self.token_input is None else "rounded"
-            h = self._join(x, self.ffn.output(h, ctx), self.ffn_post_norm, reader, dtype)
+            h = self._join(x, self.ffn.output(h, ctx), self.ffn_post_norm, reader, dtype, self.mult)
         if self.token_input is not None:
             h = self._join(x, self.token_input.output(h, ctx), self.token_input, after, dtype)
-        return NormedRows(after, h) if after is not None and h is not None else None
+        if after is None or h is None:
+            return None
+        return after.placed() if isinstance(after, JoinedRows) else NormedRows(after, h)
 
 
 @register_block("parallel_residual")

@@ -145,6 +145,15 @@ class Linear:
                                    w_tiled=self.tiled, **self._norm_arguments(a))
         return ops.gemm_swiglu(self._tensor_of(a), self.weight, w_tiled=self.tiled)
 
+    def gelu(self, a: torch.Tensor) -> torch.Tensor:
+        """gelu(a . W^T (+ bias)), the error-function form, in a's dtype."""
+        if a.dtype == torch.bfloat16:
+            if self._medium(a):
+                return ops.gemm_medium(a, self.weight, ops.EPILOGUE_STORE, bias=self.bias, out_dtype=a.dtype, w_tiled=self.tiled, gelu=True)
+            if self._fused(a, self.out_features, ops.EPILOGUE_STORE):
+                return ops.gemm_decode(a, self.weight, ops.EPILOGUE_STORE, bias=self.bias, out_dtype=a.dtype, w_tiled=self.tiled, gelu=True)
+        return ops.gemm(a, self.weight, self.bias, out_dtype=a.dtype, w_tiled=self.tiled, gelu=True)
+
     def clamped_glu(self, a: Input, limit: float, alpha: float, shift: float) -> torch.Tensor:
         """The weight holds gate rows then up rows: g * sigmoid(alpha g) * (u + shift) with g = min(gate,
         limit), u = clamp(up, -limit, limit). In the products of few rows the unit is the product's

@@ -11,7 +11,9 @@ pairs as tiles of one grouped product, so nothing crosses to the host and a deco
 ``router_scores`` "softmax_all": the scores are the softmax over all experts, and the chosen experts' scores divided by
 their sum (+ 1e-20) are the weights (the choice is the same: the largest scores are the largest logits).
 ``router_groups`` (count, keep): the experts form ``count`` equal groups of neighbours, a group's score is its best
-expert's, and only experts of the ``keep`` best groups can be chosen. ``unit`` "clamped" with ``limit`` (and ``alpha``,
+expert's, and only experts of the ``keep`` best groups can be chosen; ``group_score`` "pair": a group's score is the sum of
+its two best experts' scores instead. ``router_scores`` "sigmoid": every expert scores sigmoid(z) on its own, and the
+chosen scores divided by their sum (+ 1e-20) are the weights. ``unit`` "clamped" with ``limit`` (and ``alpha``,
 ``shift``): an expert is W_down (g sigmoid(alpha g) (u + shift)) with g = min(W_gate h, limit), u = clamp(W_up h, -limit,
 limit); the shared unit is then of the same form with ``shared_limit``. Registered as ``moe_swiglu`` and ``moe_glu``.
 """
@@ -47,13 +49,16 @@ class MoeSwiGLU(FeedForward):
         self.intermediate = int(spec["intermediate_size"])
         self.shared_intermediate = int(spec.get("shared_intermediate_size") or 0)
         self.router_bias = bool(spec.get("router_bias", True))
-        self.score_all = spec.get("router_scores", "softmax_chosen") == "softmax_all"
+        self.scores = str(spec.get("router_scores", "softmax_chosen"))
+        self.group_pair = spec.get("group_score", "best") == "pair"
         self.groups, self.keep_groups = (int(n) for n in (spec.get("router_groups") or (1, 1)))
         self.clamped = spec.get("unit", "swiglu") == "clamped"
         self.glu = (float(spec["limit"]), float(spec.get("alpha", 1.702)), float(spec.get("shift", 1.0))) if self.clamped else None
         self.names = {**_DEFAULT_NAMES, **dict(spec.get("names", {}))}
-        if spec.get("router_scores", "softmax_chosen") not in ("softmax_chosen", "softmax_all") or spec.get("unit", "swiglu") not in ("swiglu", "clamped"):
-            raise ConfigError("a mixture's router scores are 'softmax_chosen' or 'softmax_all', its units 'swiglu' or 'clamped'")
+        if self.scores not in ops.MOE_SCORES or spec.get("unit", "swiglu") not in ("swiglu", "clamped"):
+            raise ConfigError(f"a mixture's router scores are one of {', '.join(ops.MOE_SCORES)}, its units 'swiglu' or 'clamped'")
+        if spec.get("group_score", "best") not in ("best", "pair") or (self.group_pair and self.scores == "softmax_chosen"):
+            raise ConfigError("a group's score is 'best' or 'pair' (a pair of scores that do not depend on the choice)")
         if self.groups < 1 or self.groups > 64 or self.experts % self.groups or not 1 <= self.keep_groups <= self.groups \
                 or self.top > self.keep_groups * (self.experts // self.groups):
             raise ConfigError(f"{self.experts} experts in {self.groups} groups (equal ones, at most 64) of which {self.keep_groups} "
@@ -117,7 +122,7 @@ class MoeSwiGLU(FeedForward):
     def route(self, h: torch.Tensor):
         """(chosen [rows, top], weight [rows, top]) of the rows ``h``."""
         logits = self.router.forward(h, out_dtype=torch.float32)
-        return ops.moe_route(logits, self.bias, self.top, self.groups, self.keep_groups, self.score_all)
+        return ops.moe_route(logits, self.bias, self.top, self.groups, self.keep_groups, scores=self.scores, group_pair=self.group_pair)
 
     def forward(self, h, residual, ctx):
         rows = (h.tensor() if isinstance(h, LazyNorm) else h)

@@ -1,16 +1,26 @@
 """RMS norm: y = x * rsqrt(mean(x^2) + eps) * w, sums in float32; the weight multiplies
 directly (native/include/flyweight_v2_qwen_kernels.hpp:425-447 with one_centered = 0).
-Layer norm with a weight and no bias: the row's mean is taken off first, y = (x - m) * rsqrt(mean((x - m)^2) + eps) * w."""
+Layer norm: the row's mean is taken off first, y = (x - m) * rsqrt(mean((x - m)^2) + eps) * w, plus a bias vector where
+the design has one."""
 
 from __future__ import annotations
 
-from typing import Dict, Optional
+from typing import Dict, NamedTuple, Optional
 
 import torch
 
 from ..kernels import ops
 from ..weights.loader import TensorDecl
 from .base import Norm, register_norm
+
+
+class RowNorm(NamedTuple):
+    """A norm over a whole row as a kernel applies it beside other work on the row: v / sqrt(mean(v^2) + eps) * weight
+    (+ bias), v the row, or with ``centered`` the row less its mean."""
+    weight: torch.Tensor
+    eps: float
+    centered: bool
+    bias: Optional[torch.Tensor] = None
 
 
 class Prepared:
@@ -93,9 +103,9 @@ class RMSNorm(Norm):
         return self.weight, self.eps, self.one_centered
 
     def row_norm(self):
-        """(weight, eps, centered) for a kernel that applies the norm beside other work on the row, or
-        None where the norm is not of that plain form."""
-        return None if self.one_centered else (self.weight, self.eps, False)
+        """The norm for a kernel that applies it beside other work on the row, or None where the norm is
+        not of that plain form."""
+        return None if self.one_centered else RowNorm(self.weight, self.eps, False)
 
     def forward(self, x: torch.Tensor, ctx, row_index: Optional[torch.Tensor] = None) -> torch.Tensor:
         return ops.rmsnorm_rows(x, self.weight, self.eps, self.dtype, row_index=row_index,
@@ -104,27 +114,33 @@ class RMSNorm(Norm):
 
 @register_norm("layernorm")
 class LayerNorm(Norm):
-    """(x - mean) / sqrt(variance + eps) * w, the variance the mean of the squared deviations; no bias."""
+    """(x - mean) / sqrt(variance + eps) * w, the variance the mean of the squared deviations; with ``bias`` + b, the
+    tensor of the weight's name with ".b" behind it."""
     graph_safe = True
 
     def __init__(self, spec):
         super().__init__(spec)
         self.size = int(spec["size"])
         self.eps = float(spec["eps"])
+        self.has_bias = bool(spec.get("bias", False))
 
     @property
     def tensor_name(self) -> str:
         return self.spec.get("tensor") or self.prefix + "weight"
 
     def tensors(self) -> Dict[str, TensorDecl]:
-        return {self.tensor_name: TensorDecl((self.size,), role="vector", init="norm")}
+        declared = {self.tensor_name: TensorDecl((self.size,), role="vector", init="norm")}
+        if self.has_bias:
+            declared[self.tensor_name + ".b"] = TensorDecl((self.size,), role="vector", init="bias")
+        return declared
 
     def bind(self, tensors, dtype, device) -> None:
         super().bind(tensors, dtype, device)
         self.weight = tensors[self.tensor_name]
+        self.bias = tensors[self.tensor_name + ".b"] if self.has_bias else None
 
     def row_norm(self):
-        return self.weight, self.eps, True
+        return RowNorm(self.weight, self.eps, True, self.bias)
 
     def forward(self, x: torch.Tensor, ctx, row_index: Optional[torch.Tensor] = None) -> torch.Tensor:
-        return ops.layernorm_rows(x, self.weight, self.eps, self.dtype, row_index=row_index)
+        return ops.layernorm_rows(x, self.weight, self.eps, self.dtype, row_index=row_index, bias=self.bias)

@@ -22,6 +22,7 @@ from ..kernels import ops
 from ..weights.loader import TensorDecl
 from .base import Part
 from .linear import Linear
+from .norm import RowNorm
 
 
 class TokenInput(Part):
@@ -53,7 +54,7 @@ class TokenInput(Part):
         self.weight = tensors[self.prefix + "norm"]
 
     def row_norm(self):
-        return self.weight, self.eps, False
+        return RowNorm(self.weight, self.eps, False)
 
     def gathered_tensors(self):
         """What the part reads by the row (a step's accounting does not count it among the weights it streams)."""
