@@ -190,6 +190,33 @@ def telapel_configs(size: dict):
     return telapel, dalerax_configs(size)[0]
 
 
+# Zaluvik (windowed attention whose weights are sigmoids that the heads mix, windowed softmax attention over a cached latent
+# with a rotated key part and a gate per head, a gelu unit or a mixture of gated units among the best groups of experts
+# with a shared unit, a layer norm with bias before and behind every sublayer; the second layer runs twice, the model's
+# input joined ahead of each pass) at the two sizes of TELAPEL_SIZES, beside the engine's closest existing model: a Telapel
+# of as many layer runs, the same width, vocabulary, latent, experts and windows.
+ZALUVIK_SIZES = {name: dict(size) for name, size in TELAPEL_SIZES.items()}
+
+
+def zaluvik_configs(size: dict):
+    """(Zaluvik configuration, Telapel configuration of equal size)."""
+    from flyweight_amd.config import config_from_dict
+    moe = {"kind": "moe", "router": {"experts": size["experts"], "top": size["top"], "groups": {"count": size["groups"], "keep": size["keep"]}},
+           "expert": {"ff": size["expert_ff"]}, "shared": {"ff": size["shared_ff"]}}
+    attention = {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": size["dim"], "vdim": size["vdim"],
+                 "scale": 2.0 * size["dim"] ** -0.5, "mask": {"size": size["window"]}}
+    latent = {"heads": size["heads"], "dim": size["latent_dim"], "rot_dim": size["rot_dim"], "vdim": size["vdim"], "kv_rank": size["kv_rank"],
+              "scale": (size["latent_dim"] + size["rot_dim"]) ** -0.5, "mask": {"size": size["window"]},
+              "rot": {"base": 10000.0, "dims": size["rot_dim"]}}
+    layers = [{"type": "attention", "mixer": attention, "mlp": {"kind": "dense", "ff": size["ff"]}},
+              {"type": "latent_attention", "mixer": latent, "mlp": moe},
+              {"type": "attention", "mixer": attention, "mlp": moe}]
+    zaluvik = config_from_dict({"architecture": "Zaluvik", "vocab": size["vocab"], "width": size["width"], "norm": {"eps": 1e-6},
+                                "embedding": {"scale": 1.0}, "residual_mult": 0.5, "layers": layers,
+                                "loop": {"start": 1, "stop": 2, "times": 2}})
+    return zaluvik, telapel_configs(size)[0]
+
+
 def kernel_times(torch, run) -> dict:
     """Entry point of the kernel library -> microseconds of GPU time per call, over one call of ``run``
     (launched kernel by kernel, every call bracketed by two events)."""
@@ -562,11 +589,11 @@ def main() -> int:
     parser.add_argument("--only", choices=("decode", "prefill"), help="run one phase and print no JSON (for profiling)")
     parser.add_argument("--drawn", action="store_true", help="with --only decode: the requests draw their tokens "
                         "(temperature 0.8, top_k 40, top_p 0.95, min_p 0.05) instead of taking the most likely one")
-    parser.add_argument("--workload", choices=("headline",) + tuple(WORKLOADS) + ("koketar", "vavelorn", "dalerax", "telapel"), default="headline",
+    parser.add_argument("--workload", choices=("headline",) + tuple(WORKLOADS) + ("koketar", "vavelorn", "dalerax", "telapel", "zaluvik"), default="headline",
                         help="headline: the LFM2-1.2B decode and prefill figures; long-context, mixed: a whole serving run; "
                              "koketar: prefill and decode of Koketar beside LFM2 at equal sizes, kernel by kernel; "
                              "vavelorn: the same of Vavelorn beside Koketar; dalerax: the same of Dalerax beside Koketar; "
-                             "telapel: the same of Telapel beside Dalerax")
+                             "telapel: the same of Telapel beside Dalerax; zaluvik: the same of Zaluvik beside Telapel")
     parser.add_argument("--requests", type=int, help="requests of a serving workload (default: as the workload names)")
     args = parser.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
@@ -580,8 +607,11 @@ def main() -> int:
     from flyweight_amd import Model
     from flyweight_amd.config import config_from_dict
 
-    if args.workload in ("koketar", "vavelorn", "dalerax", "telapel"):
-        if args.workload == "telapel":
+    if args.workload in ("koketar", "vavelorn", "dalerax", "telapel", "zaluvik"):
+        if args.workload == "zaluvik":
+            record = koketar_run(torch, args, families=("zaluvik", "telapel"), sizes=ZALUVIK_SIZES, configs_of=zaluvik_configs,
+                                 title="Zaluvik", beside="Zaluvik beside Telapel at equal width, layer runs, vocabulary, latent, experts and windows")
+        elif args.workload == "telapel":
             record = koketar_run(torch, args, families=("telapel", "dalerax"), sizes=TELAPEL_SIZES, configs_of=telapel_configs,
                                  title="Telapel", beside="Telapel beside Dalerax at equal width, depth, vocabulary, experts and windows")
         elif args.workload == "dalerax":

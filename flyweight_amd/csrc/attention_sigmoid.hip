@@ -28,6 +28,8 @@ __device__ __forceinline__ uint32_t sg_pack(float lo, float hi) {
 }
 // a factor on an output channel: sigmoid of the gate's raw value
 __device__ __forceinline__ float sg_gate(float z) { return 1.0f / (1.0f + expf(-z)); }
+// the same by the hardware's 2^x and reciprocal (about 1e-7 of the result), for results that are rounded to bfloat16
+__device__ __forceinline__ float sg_gate_quick(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-z * LOG2E_F)); }
 
 // ---- the plain kernel: any sizes, float32 arithmetic ------------------------------------------------
 // A workgroup per (row, run of output heads). Per page: a wave's lanes are the page's keys and its heads
@@ -155,26 +157,36 @@ extern "C" int fw_sigmoid_attention_generic(const void* q, void* out, int dtype,
 // ---- prompt portions on the matrix cores --------------------------------------------------------------
 // A workgroup of eight waves takes 16 query rows of one segment, all heads, and walks the visible keys
 // 128 at a time. Of those a wave first takes 16: per head g it forms S^T[key][row] = K Q^T
-// (v_mfma_f32_16x16x32_bf16, the key/value head's keys loaded once per group straight into operand registers,
-// the queries from LDS), so that a lane holds the scores of 4 keys x 1 row of EVERY head, turns them
-// into sigmoids, and mixes the heads where they are: v_mfma_f32_4x4x1f32 multiplies a 4 x 1 column of the mix (4
-// output heads, one g) by 64 lanes' weights of g, sixteen blocks side by side, which is a mix in exact
+// (v_mfma_f32_16x16x32_bf16, the key/value head's keys loaded once per group straight into operand registers, one
+// key/value head ahead of the work, the queries from LDS), so that a lane holds the scores of 4 keys x 1 row of EVERY
+// head, turns them into sigmoids, and mixes the heads where they are: v_mfma_f32_4x4x1f32 multiplies a 4 x 1 column
+// of the mix (4 output heads, one g) by 64 lanes' weights of g, sixteen blocks side by side, which is a mix in exact
 // float32 that moves nothing between lanes and leaves the vector unit to the sigmoids. The mixed
 // weights, rounded to bfloat16, go to LDS [head][row][128 keys]; behind a barrier the waves share out
-// the (head, half of the channels) pairs and add V^T P^T (v_mfma_f32_16x16x32_bf16, values straight from
-// the cache) to accumulators that stay in registers to the end, where the gate joins.
-// HB: heads in fours (num_heads <= 4 HB; heads beyond have a zero column and row in the mix and are not stored).
+// the heads (and, with few heads, the halves of their channels) and add V^T P^T (v_mfma_f32_16x16x32_bf16, values
+// straight from the cache, one run of tiles ahead) to accumulators that stay in registers to the end, where the gate joins.
+// gridDim.y workgroups share the steps of 128 keys of a tile where the tiles alone would not fill the chip: parts
+// of a row's keys add up, so each leaves its float32 sums and the one that arrives last (a ticket per tile; nobody
+// waits) adds them in the order of the keys.
+// HB: heads in fours (num_heads <= 4 HB; heads beyond have a zero column and row in the mix and are not stored). GS: a
+// divisor of the heads on one key/value head (4, 2 or 1); the scores of that many heads are formed side by side.
+// What is the same for a whole wave is kept in scalar registers (its number, pages, heads), and a lane's place
+// in a page as one 32-bit offset: the vector registers are all taken by what is in flight.
 #define SG_WAVES 8
 #define SG_STEP 128
 #define SG_PAD 8
-template <int HD, int HB>
+template <int HD, int HB, int GS>
 __global__ __launch_bounds__(64 * SG_WAVES) void sigmoid_attention_prefill_kernel(
-    const uint16_t* __restrict__ q, uint16_t* __restrict__ out, const uint16_t* __restrict__ k_pages,
+    const uint16_t* __restrict__ q, uint16_t* __restrict__ out, float* partial, int* tickets, const uint16_t* __restrict__ k_pages,
     const uint16_t* __restrict__ v_pages, const int32_t* __restrict__ block_table, int table_stride,
     const int32_t* __restrict__ tile_seg, const int32_t* __restrict__ tile_row0, const int32_t* __restrict__ seg_row0,
     const int32_t* __restrict__ row_pos, int num_heads, int num_kv_heads, int head_dim, int v_dim, float scale_log2, int window,
     const float* __restrict__ bias, const float* __restrict__ mix, const float* __restrict__ gate, int gate_stride) {
-    constexpr int HP = 4 * HB;                  // heads with padding
+    constexpr int HP = 4 * HB;                          // heads with padding
+    constexpr int SLOTS = (HB + 1) / 2;                 // heads of a wave in the weighted sums
+    constexpr int HALVES = HB == 1 ? 1 : 2;             // halves of a head's channels a wave takes
+    constexpr int TILES = HD / 32;                      // tiles of 16 channels in a half
+    constexpr bool AHEAD = HD <= 128;                   // values are asked for a run of tiles ahead where registers allow
     constexpr int Q_STRIDE = HD + SG_PAD, P_STRIDE = SG_STEP + SG_PAD;
     extern __shared__ __attribute__((aligned(16))) unsigned char sg_raw[];
     uint16_t* lds_q = reinterpret_cast<uint16_t*>(sg_raw);                          // [heads][16 rows][Q_STRIDE]
@@ -182,6 +194,7 @@ __global__ __launch_bounds__(64 * SG_WAVES) void sigmoid_attention_prefill_kerne
     // the mix as the lanes read it: [4 output heads][4 g's][output head % 4][g % 4]
     float* lds_mix = reinterpret_cast<float*>(lds_p + (size_t)num_heads * 16 * P_STRIDE);
     float* lds_bias = lds_mix + HP * HP;                                            // [HP], times log2(e)
+    int* ticket_shared = reinterpret_cast<int*>(lds_bias + HP);
 
     const int tile = blockIdx.x >> 2, sub = blockIdx.x & 3;
     const int seg = tile_seg[tile];
@@ -189,8 +202,49 @@ __global__ __launch_bounds__(64 * SG_WAVES) void sigmoid_attention_prefill_kerne
     const int seg_end = seg_row0[seg + 1];
     if (row0 >= seg_end) return;                // the whole workgroup
     const int rows = seg_end - row0 < 16 ? seg_end - row0 : 16;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, i16 = lane & 15, g4 = lane >> 4;
+    const int pos_lo = row_pos[row0], pos_hi = row_pos[row0 + rows - 1];
+    const int all_first = fw_first_visible(pos_lo, window, 0) / PAGE, last_block = pos_hi / PAGE;
+    // this workgroup's share of the tile's steps
+    const int all_steps = (last_block - all_first) / 2 + 1;
+    const int share = (all_steps + (int)gridDim.y - 1) / (int)gridDim.y, parts = (all_steps + share - 1) / share;
+    const int first_block = all_first + (int)blockIdx.y * share * 2;
+    if (first_block > last_block) return;       // the whole workgroup
+    const int end_block = first_block + 2 * share - 1 < last_block ? first_block + 2 * share - 1 : last_block;
+    const int tid = threadIdx.x, lane = tid & 63, i16 = lane & 15, g4 = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int group = num_heads / num_kv_heads;
+    const int32_t* table = block_table + (size_t)seg * table_stride;
+    auto page_of = [&](int block) { return table[block <= end_block ? block : end_block]; };
+
+    // A lane's place in a head's page of keys, in bytes. Channels past head_dim (whole runs of 32, or the last
+    // run's upper half: head_dim is a multiple of 16) are read from channels that are there, and are zero by the time
+    // they are used.
+    const uint32_t key_offset = (uint32_t)(((wave & 3) * 16 + i16) * head_dim + g4 * 8) * 2u;
+    const uint32_t key_offset_tail = g4 >= 2 ? key_offset - 32u : key_offset;
+    const int whole_runs = head_dim / 32;
+    auto load_keys = [&](u32x4 (&kf)[HD / 32], int page, int kvh) {
+        const char* keys = reinterpret_cast<const char*>(k_pages + ((size_t)page * num_kv_heads + kvh) * PAGE * head_dim);
+#pragma unroll
+        for (int dc = 0; dc < HD / 32; ++dc) {
+            const char* from = keys + (dc * 32 < head_dim ? dc * 64 : 0);
+            kf[dc] = *reinterpret_cast<const u32x4*>(from + (dc < whole_runs ? key_offset : key_offset_tail));
+        }
+    };
+    u32x4 kf_next[HD / 32];
+    bf16x8 kf[HD / 32];
+    auto take_keys = [&]() {
+#pragma unroll
+        for (int dc = 0; dc < HD / 32; ++dc) {
+            u32x4 bits = kf_next[dc];
+            if (dc >= whole_runs) {             // uniform, and never with a full head_dim
+                const bool in = dc * 32 + g4 * 8 < head_dim;
+                bits = u32x4{in ? bits[0] : 0u, in ? bits[1] : 0u, in ? bits[2] : 0u, in ? bits[3] : 0u};
+            }
+            kf[dc] = __builtin_bit_cast(bf16x8, bits);
+        }
+    };
+    int page_a = page_of(first_block), page_b = page_of(first_block + 1);       // the step's two pages
+    load_keys(kf_next, wave >> 2 ? page_b : page_a, 0);
 
     // queries of the 16 rows, head by head; channels past head_dim and rows past the end are zero
     for (int run = tid; run < num_heads * 16 * (HD / 8); run += 64 * SG_WAVES) {
@@ -204,58 +258,88 @@ __global__ __launch_bounds__(64 * SG_WAVES) void sigmoid_attention_prefill_kerne
         lds_mix[item] = (h < num_heads && g < num_heads) ? mix[(size_t)h * num_heads + g] : 0.0f;
     }
     if (tid < HP) lds_bias[tid] = tid < num_heads ? bias[tid] * LOG2E_F : 0.0f;
-    __syncthreads();
+    fw_lds_barrier();
 
     const bool row_there = i16 < rows;
     const int my_pos = row_pos[row0 + (row_there ? i16 : 0)];
-    const int pos_lo = row_pos[row0], pos_hi = row_pos[row0 + rows - 1];
     const int my_first = fw_first_visible(my_pos, window, 0);
-    const int first_block = fw_first_visible(pos_lo, window, 0) / PAGE, last_block = pos_hi / PAGE;
-    const int32_t* table = block_table + (size_t)seg * table_stride;
-
-    f32x4 acc[HB][HD / 32];
+    // the heads of this wave's weighted sums (one past the last computes along and is not stored)
+    int head_of[SLOTS], kv_of[SLOTS];
 #pragma unroll
-    for (int n = 0; n < HB; ++n)
+    for (int n = 0; n < SLOTS; ++n) {
+        const int head = HB == 1 ? wave >> 1 : wave * SLOTS + n;
+        head_of[n] = head < num_heads ? head : num_heads - 1;
+        kv_of[n] = head_of[n] / group;
+    }
+    const int half0 = HB == 1 ? (wave & 1) : 0;
+    // (v_dim is a multiple of 16: a tile of channels is there or not; one past the last is the last again, not stored)
+    const uint32_t value_offset = (uint32_t)(i16 * PAGE + g4 * 8) * 2u;
+    const int last_tile = v_dim / 16 - 1;
+    auto load_values = [&](u32x4 (&v)[TILES], int page, int kb, int half, int kvh) {
+        const char* values = reinterpret_cast<const char*>(v_pages + ((size_t)page * num_kv_heads + kvh) * v_dim * PAGE + (kb & 1) * 32);
 #pragma unroll
-        for (int t = 0; t < HD / 32; ++t) acc[n][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int t = 0; t < TILES; ++t) {
+            const int at = (half0 + half) * TILES + t, there = at < last_tile ? at : last_tile;
+            v[t] = *reinterpret_cast<const u32x4*>(values + (size_t)there * 16 * PAGE * 2 + value_offset);
+        }
+    };
 
-    for (int block0 = first_block; block0 <= last_block; block0 += 2) {
+    f32x4 acc[SLOTS][HALVES][TILES];
+#pragma unroll
+    for (int n = 0; n < SLOTS; ++n)
+#pragma unroll
+        for (int half = 0; half < HALVES; ++half)
+#pragma unroll
+            for (int t = 0; t < TILES; ++t) acc[n][half][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+    for (int block0 = first_block; block0 <= end_block; block0 += 2) {
         // -- weights of this wave's 16 keys, every head
         const int my_block = block0 + (wave >> 2);
-        const int key0 = my_block * PAGE + (wave & 3) * 16;         // a wave past the last page sees nothing and stores zeros
-        const int page_k = table[my_block <= last_block ? my_block : last_block];
+        const int key0 = my_block * PAGE + (wave & 3) * 16;
+        const int next_a = page_of(block0 + 2), next_b = page_of(block0 + 3);
         float w[HP][4];
-        bf16x8 kf[HD / 32];
-        int kvh = -1;
+        int kvh = -1, left = 0;                 // heads left on this key/value head
 #pragma unroll
-        for (int g = 0; g < HP; ++g) {
-            const int head = g < num_heads ? g : num_heads - 1;
-            const int wanted = head / group;
-            if (wanted != kvh) {                // uniform: the next key/value head's keys
-                kvh = wanted;
-                const uint16_t* key = k_pages + (((size_t)page_k * num_kv_heads + kvh) * PAGE + (wave & 3) * 16 + i16) * head_dim + g4 * 8;
-#pragma unroll
-                for (int dc = 0; dc < HD / 32; ++dc) {
-                    kf[dc] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
-                    if (dc * 32 + g4 * 8 < head_dim) kf[dc] = *reinterpret_cast<const bf16x8*>(key + dc * 32);
-                }
+        for (int g0 = 0; g0 < HP; g0 += GS) {
+            if (left == 0 && g0 < num_heads) {  // uniform: the next key/value head's keys, and the ones after them asked for
+                ++kvh;
+                left = group;
+                take_keys();
+                const bool last = kvh + 1 >= num_kv_heads;
+                load_keys(kf_next, wave >> 2 ? (last ? next_b : page_b) : (last ? next_a : page_a), last ? 0 : kvh + 1);
             }
-            const uint16_t* query = lds_q + ((size_t)head * 16 + i16) * Q_STRIDE + g4 * 8;
-            f32x4 s = {0.f, 0.f, 0.f, 0.f};
+            left -= GS;
+            f32x4 s[GS];
+#pragma unroll
+            for (int u = 0; u < GS; ++u) s[u] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int dc = 0; dc < HD / 32; ++dc)
-                s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[dc], *reinterpret_cast<const bf16x8*>(query + dc * 32), s, 0, 0, 0);
-            const float b = lds_bias[g];
 #pragma unroll
-            for (int r = 0; r < 4; ++r)         // sigmoid by the hardware's 2^x and reciprocal; 2^x = infinity gives 0
-                w[g][r] = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-fmaf(s[r], scale_log2, b)));
+                for (int u = 0; u < GS; ++u) {
+                    const int head = g0 + u < num_heads ? g0 + u : num_heads - 1;
+                    const bf16x8 query = *reinterpret_cast<const bf16x8*>(lds_q + ((size_t)head * 16 + i16) * Q_STRIDE + g4 * 8 + dc * 32);
+                    s[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[dc], query, s[u], 0, 0, 0);
+                }
+#pragma unroll
+            for (int u = 0; u < GS; ++u) {
+                const float b = lds_bias[g0 + u];
+#pragma unroll
+                for (int r = 0; r < 4; ++r)     // sigmoid by the hardware's 2^x and reciprocal; 2^x = infinity gives 0
+                    w[g0 + u][r] = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-fmaf(s[u][r], scale_log2, b)));
+            }
         }
+        u32x4 v[TILES], v_next[AHEAD ? TILES : 1];
+        if constexpr (AHEAD) load_values(v_next, page_a, 0, 0, kv_of[0]);        // they travel while the heads are mixed
+        // all of the wave's keys seen by all of its rows (all but the pages at the window's edge and the diagonal): no mask
+        const bool whole = __all(row_there && key0 >= my_first && key0 + 15 <= my_pos) && my_block <= end_block;
+        if (!whole) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int key = key0 + g4 * 4 + r;
-            const bool seen = row_there && key >= my_first && key <= my_pos;
+            for (int r = 0; r < 4; ++r) {
+                const int key = key0 + g4 * 4 + r;
+                const bool seen = row_there && key >= my_first && key <= my_pos && my_block <= end_block;
 #pragma unroll
-            for (int g = 0; g < HP; ++g) w[g][r] = seen ? w[g][r] : 0.0f;
+                for (int g = 0; g < HP; ++g) w[g][r] = seen ? w[g][r] : 0.0f;
+            }
         }
         // -- the heads mixed, and stored as the next product reads them
 #pragma unroll
@@ -271,64 +355,117 @@ __global__ __launch_bounds__(64 * SG_WAVES) void sigmoid_attention_prefill_kerne
 #pragma unroll
                     for (int r = 0; r < 4; ++r) m[r] = __builtin_amdgcn_mfma_f32_4x4x1f32(t[g], w[gb * 4 + g][r], m[r], 0, 0, 0);
             }
-            fw_mfma_drain();
 #pragma unroll
-            for (int x = 0; x < 4; ++x)
-                if (hb * 4 + x < num_heads) {
-                    uint16_t* to = lds_p + ((size_t)(hb * 4 + x) * 16 + i16) * P_STRIDE + wave * 16 + g4 * 4;
-                    *reinterpret_cast<u32x2*>(to) = u32x2{sg_pack(m[0][x], m[1][x]), sg_pack(m[2][x], m[3][x])};
-                }
+            for (int x = 0; x < 4; ++x) {
+                const u32x2 packed = {sg_pack(m[0][x], m[1][x]), sg_pack(m[2][x], m[3][x])};
+                if (hb * 4 + x < num_heads)
+                    *reinterpret_cast<u32x2*>(lds_p + ((size_t)(hb * 4 + x) * 16 + i16) * P_STRIDE + wave * 16 + g4 * 4) = packed;
+            }
         }
-        __syncthreads();
-        // -- the weighted sums of this wave's (head, half of the channels) pairs
+        fw_lds_barrier();
+        // -- the weighted sums of this wave's heads
 #pragma unroll
         for (int kb = 0; kb < 4; ++kb) {
-            const int block = block0 + (kb >> 1);
-            if (block <= last_block) {          // uniform
-                const int page = table[block];
-                // values of keys nobody has written yet must not meet a weight of 0 as they are
-                const int last_written = pos_hi - block * PAGE - (kb & 1) * 32 - g4 * 8;     // in this lane's eight keys
-                uint32_t keep[4];
+            // values of keys nobody has written yet must not meet a weight of 0 as they are
+            const int last_written = pos_hi - (block0 + (kb >> 1)) * PAGE - (kb & 1) * 32 - g4 * 8;     // in this lane's eight keys
+            uint32_t keep[4];
 #pragma unroll
-                for (int word = 0; word < 4; ++word)
-                    keep[word] = 2 * word + 1 <= last_written ? 0xffffffffu : (2 * word <= last_written ? 0xffffu : 0u);
+            for (int word = 0; word < 4; ++word)
+                keep[word] = 2 * word + 1 <= last_written ? 0xffffffffu : (2 * word <= last_written ? 0xffffu : 0u);
+            bf16x8 pf[SLOTS];
 #pragma unroll
-                for (int n = 0; n < HB; ++n) {
-                    const int unit = wave * HB + n, head_here = unit >> 1;
-                    const int head = head_here < num_heads ? head_here : num_heads - 1;     // computed along, not stored
-                    const bf16x8 pf = *reinterpret_cast<const bf16x8*>(lds_p + ((size_t)head * 16 + i16) * P_STRIDE + kb * 32 + g4 * 8);
-                    const uint16_t* value = v_pages + ((size_t)page * num_kv_heads + head / group) * v_dim * PAGE + (kb & 1) * 32 + g4 * 8;
+            for (int n = 0; n < SLOTS; ++n)
+                pf[n] = *reinterpret_cast<const bf16x8*>(lds_p + ((size_t)head_of[n] * 16 + i16) * P_STRIDE + kb * 32 + g4 * 8);
 #pragma unroll
-                    for (int t = 0; t < HD / 32; ++t) {
-                        const int channel = (unit & 1) * (HD / 2) + t * 16 + i16;
-                        u32x4 v = *reinterpret_cast<const u32x4*>(value + (size_t)(channel < v_dim ? channel : v_dim - 1) * PAGE);
-                        v = u32x4{v[0] & keep[0], v[1] & keep[1], v[2] & keep[2], v[3] & keep[3]};
-                        acc[n][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v), pf, acc[n][t], 0, 0, 0);
+            for (int half = 0; half < HALVES; ++half) {
+                if constexpr (AHEAD) {
+#pragma unroll
+                    for (int t = 0; t < TILES; ++t) v[t] = v_next[t];
+                    if (kb < 3 || half + 1 < HALVES) {
+                        const int kb_next = half + 1 < HALVES ? kb : kb + 1;
+                        load_values(v_next, kb_next >> 1 ? page_b : page_a, kb_next, half + 1 < HALVES ? half + 1 : 0, kv_of[0]);
+                    }
+                } else {
+                    load_values(v, kb >> 1 ? page_b : page_a, kb, half, kv_of[0]);
+                }
+#pragma unroll
+                for (int n = 0; n < SLOTS; ++n) {
+                    if (n > 0 && kv_of[n] != kv_of[n - 1]) load_values(v, kb >> 1 ? page_b : page_a, kb, half, kv_of[n]);    // uniform
+#pragma unroll
+                    for (int t = 0; t < TILES; ++t) {
+                        const u32x4 clean = {v[t][0] & keep[0], v[t][1] & keep[1], v[t][2] & keep[2], v[t][3] & keep[3]};
+                        acc[n][half][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, clean), pf[n], acc[n][half][t], 0, 0, 0);
                     }
                 }
             }
         }
         fw_mfma_drain();
-        __syncthreads();        // the weights are read: the next step may store its own
+        fw_lds_barrier();       // the weights are read: the next step may store its own
+        page_a = next_a;
+        page_b = next_b;
+    }
+    const int channels = num_heads * v_dim;
+    if (parts > 1) {
+        // [tile of 16 rows][part][register][thread]: device-scope stores, which pass the caches that workgroups on other
+        // dies do not share
+        constexpr int HELD = SLOTS * HALVES * TILES * 4;
+        float* mine = partial + ((size_t)blockIdx.x * gridDim.y + blockIdx.y) * HELD * 512 + tid;
+#pragma unroll
+        for (int n = 0; n < SLOTS; ++n)
+#pragma unroll
+            for (int half = 0; half < HALVES; ++half)
+#pragma unroll
+                for (int t = 0; t < TILES; ++t)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        __hip_atomic_store(mine + (size_t)(((n * HALVES + half) * TILES + t) * 4 + r) * 512, acc[n][half][t][r], __ATOMIC_RELAXED,
+                                           __HIP_MEMORY_SCOPE_AGENT);
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+        if (tid == 0) *ticket_shared = __hip_atomic_fetch_add(tickets + blockIdx.x, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        __syncthreads();
+        if (*ticket_shared != parts - 1) return;
+        if (tid == 0) __hip_atomic_store(tickets + blockIdx.x, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+#pragma unroll
+        for (int n = 0; n < SLOTS; ++n)
+#pragma unroll
+            for (int half = 0; half < HALVES; ++half)
+#pragma unroll
+                for (int t = 0; t < TILES; ++t) acc[n][half][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int part = 0; part < parts; ++part) {
+            const float* from = partial + ((size_t)blockIdx.x * gridDim.y + part) * HELD * 512 + tid;
+#pragma unroll
+            for (int n = 0; n < SLOTS; ++n)
+#pragma unroll
+                for (int half = 0; half < HALVES; ++half)
+#pragma unroll
+                    for (int t = 0; t < TILES; ++t)
+#pragma unroll
+                        for (int r = 0; r < 4; ++r)
+                            acc[n][half][t][r] += __hip_atomic_load(from + (size_t)(((n * HALVES + half) * TILES + t) * 4 + r) * 512, __ATOMIC_RELAXED,
+                                                                    __HIP_MEMORY_SCOPE_AGENT);
+        }
     }
     if (!row_there) return;
 #pragma unroll
-    for (int n = 0; n < HB; ++n) {
-        const int unit = wave * HB + n, head = unit >> 1;
+    for (int n = 0; n < SLOTS; ++n) {
+        const int head = HB == 1 ? wave >> 1 : wave * SLOTS + n;
         if (head >= num_heads) continue;
 #pragma unroll
-        for (int t = 0; t < HD / 32; ++t) {
-            const int channel = (unit & 1) * (HD / 2) + t * 16 + g4 * 4;
-            if (channel >= v_dim) continue;     // v_dim is a multiple of 16
-            f32x4 o = acc[n][t];
-            if (gate) {
-                const float* z = gate + (size_t)(row0 + i16) * gate_stride + (size_t)head * v_dim + channel;
+        for (int half = 0; half < HALVES; ++half)
 #pragma unroll
-                for (int r = 0; r < 4; ++r) o[r] *= sg_gate(z[r]);
+            for (int t = 0; t < TILES; ++t) {
+                const int channel = (half0 + half) * (HD / 2) + t * 16 + g4 * 4;
+                if (channel >= v_dim) continue;     // v_dim is a multiple of 16
+                f32x4 o = acc[n][half][t];
+                if (gate) {
+                    const float* z = gate + (size_t)(row0 + i16) * gate_stride + (size_t)head * v_dim + channel;
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) o[r] *= sg_gate_quick(z[r]);
+                }
+                *reinterpret_cast<u32x2*>(out + (size_t)(row0 + i16) * channels + (size_t)head * v_dim + channel) =
+                    u32x2{sg_pack(o[0], o[1]), sg_pack(o[2], o[3])};
             }
-            *reinterpret_cast<u32x2*>(out + ((size_t)(row0 + i16) * num_heads + head) * v_dim + channel) =
-                u32x2{sg_pack(o[0], o[1]), sg_pack(o[2], o[3])};
-        }
     }
 }
 
@@ -340,13 +477,15 @@ static int sg_tiled_check(const char* name, int num_heads, int head_dim, int v_d
 }
 static int sg_prefill_lds(int num_heads, int widest_class) {
     const int heads_padded = (num_heads + 3) / 4 * 4;
-    return num_heads * 16 * (widest_class + SG_PAD + SG_STEP + SG_PAD) * 2 + (heads_padded * heads_padded + heads_padded) * 4;
+    return num_heads * 16 * (widest_class + SG_PAD + SG_STEP + SG_PAD) * 2 + (heads_padded * heads_padded + heads_padded + 1) * 4;
 }
 static int sg_class(int head_dim, int v_dim) {
     const int widest = head_dim > v_dim ? head_dim : v_dim;
     return widest <= 32 ? 32 : widest <= 64 ? 64 : widest <= 128 ? 128 : 256;
 }
 #define SG_LDS_LIMIT (160 * 1024)
+#define SG_MAX_PARTS 8
+#define SG_FILL 256                 // workgroups that fill the chip (one to a compute unit at many heads)
 
 // 1 if the matrix-core kernels take these sizes (bfloat16): up to 16 heads, sizes in steps of 16 up to 256, and
 // the queries and weights of 16 rows of all heads within a compute unit's LDS
@@ -356,7 +495,30 @@ extern "C" int fw_sigmoid_attention_fits(int num_heads, int head_dim, int v_dim)
     return sg_prefill_lds(num_heads, sg_class(head_dim, v_dim)) <= SG_LDS_LIMIT ? 1 : 0;
 }
 
-extern "C" int fw_sigmoid_attention_prefill(const void* q, void* out, const void* k_pages, const void* v_pages,
+// Floats of workspace that a tile of 16 rows leaves per part (all of a workgroup's accumulators)
+static int sg_part_floats(int num_heads, int width) {
+    const int fours = (num_heads + 3) / 4;
+    return (fours + 1) / 2 * (fours == 1 ? 1 : 2) * (width / 32) * 4 * 512;
+}
+
+// What `tiles` tiles of 64 rows that see at most `max_keys` keys each need for `parts` workgroups to a tile of 16 rows: floats
+// of workspace (0: none) and zeroed counters. parts <= 0: as many as fill the chip; the number used is returned.
+extern "C" int fw_sigmoid_attention_prefill_plan(int tiles, int num_heads, int head_dim, int v_dim, int window, int max_context, int parts,
+                                                 long long* workspace_floats, int* counters) {
+    long long keys = max_context;
+    if (window > 0 && window + 16 < keys) keys = window + 16;
+    const int steps = (int)((keys + PAGE - 2) / PAGE + 1) / 2 + 1;
+    if (parts <= 0) parts = tiles > 0 ? SG_FILL / (tiles * 4) : 1;
+    if (parts > steps) parts = steps;
+    if (parts > SG_MAX_PARTS) parts = SG_MAX_PARTS;
+    if (parts < 1) parts = 1;
+    *workspace_floats = parts > 1 ? (long long)tiles * 4 * parts * sg_part_floats(num_heads, sg_class(head_dim, v_dim)) : 0;
+    *counters = parts > 1 ? tiles * 4 : 0;
+    return parts;
+}
+
+extern "C" int fw_sigmoid_attention_prefill(const void* q, void* out, float* partial, long long partial_floats, int* tickets,
+                                            int tickets_len, int parts, const void* k_pages, const void* v_pages,
                                             const int32_t* block_table, int table_stride, const int32_t* tile_seg,
                                             const int32_t* tile_row0, int tiles, const int32_t* seg_row0, const int32_t* row_pos, int rows,
                                             int num_heads, int num_kv_heads, int head_dim, int v_dim, float scale, int window,
@@ -371,28 +533,35 @@ extern "C" int fw_sigmoid_attention_prefill(const void* q, void* out, const void
     FW_REQUIRE(lds_bytes <= SG_LDS_LIMIT, "sigmoid_attention_prefill: %d heads of %d / %d channels need %d bytes of LDS", num_heads, head_dim,
                v_dim, lds_bytes);
     if (rows == 0 || tiles == 0) return 0;
-    dim3 grid((unsigned)tiles * 4);
-#define SG_LAUNCH(HD, HB)                                                                                                            \
+    FW_REQUIRE(parts >= 1 && parts <= SG_MAX_PARTS, "sigmoid_attention_prefill: %d parts (1..%d)", parts, SG_MAX_PARTS);
+    FW_REQUIRE(parts == 1 || (partial && tickets && partial_floats >= (long long)tiles * 4 * parts * sg_part_floats(num_heads, width) &&
+                              tickets_len >= tiles * 4), "sigmoid_attention_prefill: %d parts of %d tiles need more workspace or counters", parts, tiles);
+    dim3 grid((unsigned)tiles * 4, (unsigned)parts);
+#define SG_LAUNCH(HD, HB, GS)                                                                                                         \
     {                                                                                                                               \
         static int configured = 0;                                                                                                  \
         if (lds_bytes > configured) {                                                                                               \
-            hipError_t status = hipFuncSetAttribute((const void*)sigmoid_attention_prefill_kernel<HD, HB>,                           \
+            hipError_t status = hipFuncSetAttribute((const void*)sigmoid_attention_prefill_kernel<HD, HB, GS>,                       \
                                                     hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);                         \
             FW_REQUIRE(status == hipSuccess, "sigmoid_attention_prefill: cannot reserve %d bytes of LDS", lds_bytes);                \
             configured = lds_bytes;                                                                                                 \
         }                                                                                                                           \
-        sigmoid_attention_prefill_kernel<HD, HB><<<grid, 64 * SG_WAVES, lds_bytes, (hipStream_t)stream>>>(                           \
-            (const uint16_t*)q, (uint16_t*)out, (const uint16_t*)k_pages, (const uint16_t*)v_pages, block_table, table_stride,       \
+        sigmoid_attention_prefill_kernel<HD, HB, GS><<<grid, 64 * SG_WAVES, lds_bytes, (hipStream_t)stream>>>(                       \
+            (const uint16_t*)q, (uint16_t*)out, partial, tickets, (const uint16_t*)k_pages, (const uint16_t*)v_pages, block_table, table_stride, \
             tile_seg, tile_row0, seg_row0, row_pos, num_heads, num_kv_heads, head_dim, v_dim, scale * LOG2E_F, window, bias, mix,    \
             gate, gate_stride);                                                                                                     \
     }
+#define SG_BY_GROUP(HD, HB)                                                                                                         \
+    if (group % 4 == 0) SG_LAUNCH(HD, HB, 4) else if (group % 2 == 0) SG_LAUNCH(HD, HB, 2) else SG_LAUNCH(HD, HB, 1)
 #define SG_BY_HEADS(HD)                                                                                                             \
-    if (fours == 1) SG_LAUNCH(HD, 1) else if (fours == 2) SG_LAUNCH(HD, 2) else if (fours == 3) SG_LAUNCH(HD, 3) else SG_LAUNCH(HD, 4)
+    if (fours == 1) { SG_BY_GROUP(HD, 1) } else if (fours == 2) { SG_BY_GROUP(HD, 2) } else if (fours == 3) { SG_BY_GROUP(HD, 3) } else { SG_BY_GROUP(HD, 4) }
+    const int group = num_heads / num_kv_heads;
     if (width == 32) { SG_BY_HEADS(32) }
     else if (width == 64) { SG_BY_HEADS(64) }
     else if (width == 128) { SG_BY_HEADS(128) }
-    else { if (fours == 1) SG_LAUNCH(256, 1) else if (fours == 2) SG_LAUNCH(256, 2) else SG_LAUNCH(256, 3) }
+    else { if (fours == 1) SG_LAUNCH(256, 1, 1) else if (fours == 2) SG_LAUNCH(256, 2, 1) else SG_LAUNCH(256, 3, 1) }
 #undef SG_BY_HEADS
+#undef SG_BY_GROUP
 #undef SG_LAUNCH
     FW_LAUNCH_CHECK("sigmoid_attention_prefill");
     return 0;
@@ -598,7 +767,7 @@ __global__ __launch_bounds__(256) void sigmoid_attention_decode_kernel(
                 f32x4 o = acc[t];
                 if (gate) {
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) o[r] *= sg_gate(gate[(size_t)row * gate_stride + at + r]);
+                    for (int r = 0; r < 4; ++r) o[r] *= sg_gate_quick(gate[(size_t)row * gate_stride + at + r]);
                 }
                 *reinterpret_cast<u32x2*>(out + (size_t)row * channels + at) = u32x2{sg_pack(o[0], o[1]), sg_pack(o[2], o[3])};
             } else {
@@ -642,7 +811,7 @@ __global__ __launch_bounds__(256) void sigmoid_attention_decode_kernel(
         for (int u = 0; u < 4; ++u) {
             const int item = item0 + 256 * u;
             if (item < channels) {
-                const float factor = gate ? sg_gate(gate[(size_t)row * gate_stride + item]) : 1.0f;
+                const float factor = gate ? sg_gate_quick(gate[(size_t)row * gate_stride + item]) : 1.0f;
                 out[(size_t)row * channels + item] = float_to_bf16_bits(sum[u] * factor);
             }
         }

@@ -207,8 +207,12 @@ int fw_sigmoid_attention_generic(const void* q, void* out, int dtype, const void
                                  int num_pages, void* stream);
 // The matrix-core kernels (bfloat16): whether they take these sizes (up to 16 heads, channels in steps of 16 up to 256).
 int fw_sigmoid_attention_fits(int num_heads, int head_dim, int v_dim);
-// Prompt portions; tiles as for fw_attention_prefill.
-int fw_sigmoid_attention_prefill(const void* q, void* out, const void* k_pages, const void* v_pages, const int32_t* block_table,
+// Prompt portions; tiles as for fw_attention_prefill. `parts` workgroups share the keys of 16 rows (1..8): their number, the
+// floats of workspace and the zeroed counters (left zero) they need come from the plan (parts <= 0: as many as fill the chip).
+int fw_sigmoid_attention_prefill_plan(int tiles, int num_heads, int head_dim, int v_dim, int window, int max_context, int parts,
+                                      long long* workspace_floats, int* counters);
+int fw_sigmoid_attention_prefill(const void* q, void* out, float* partial, long long partial_floats, int* tickets, int tickets_len,
+                                 int parts, const void* k_pages, const void* v_pages, const int32_t* block_table,
                                  int table_stride, const int32_t* tile_seg, const int32_t* tile_row0, int tiles,
                                  const int32_t* seg_row0, const int32_t* row_pos, int rows, int num_heads, int num_kv_heads,
                                  int head_dim, int v_dim, float scale, int window, const float* bias, const float* mix,

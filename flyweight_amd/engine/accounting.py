@@ -66,20 +66,31 @@ def _chosen_parts(model) -> List:
 
 
 def step_weight_bytes(model, rows: int = 1) -> int:
-    """Bytes of every weight a decode step of ``rows`` tokens reads once: the layers, the final norm and
+    """Bytes of every weight a decode step of ``rows`` tokens reads, each counted once also where a layer runs
+    several times: the layers, the map of the model's input where there is one, the final norm and
     the head (a tied embedding table is read as the head; an untied one only by the row, which is not
     counted); of weights that tokens choose among, those that ``rows`` tokens are expected to choose.
     ``model``: a bound CausalLM."""
-    return _bytes(_tensors([model.layers, model.final_norm, model.head])) + sum(
+    return _bytes(_tensors([model.layers, model.input_join, model.final_norm, model.head])) + sum(
         int(part.chosen_weight_bytes(rows)) for part in _chosen_parts(model))
 
 
 def product_flops_per_token(model) -> int:
-    """Flops of the layers' matrix products for one token (the head is not among them: it runs
-    for wanted rows only)."""
-    linears = {id(item): item for item in _walk(model.layers, set()) if isinstance(item, Linear)}
-    return 2 * sum(linear.weight.numel() for linear in linears.values()) + sum(
-        int(part.chosen_flops_per_token()) for part in _chosen_parts(model))
+    """Flops of the layers' matrix products for one token, a layer counted as often as it runs (the head is
+    not among them: it runs for wanted rows only)."""
+    def of(item) -> int:
+        linears = {id(found): found for found in _walk(item, set()) if isinstance(found, Linear)}
+        return 2 * sum(linear.weight.numel() for linear in linears.values())
+
+    def chosen(part) -> int:
+        below = part.sub_parts() if hasattr(part, "sub_parts") else ()
+        return (int(part.chosen_flops_per_token()) if hasattr(part, "chosen_flops_per_token") else 0) + sum(chosen(inner) for inner in below)
+
+    by_layer = [of(block) + sum(chosen(part) for part in block.parts()) for block in model.layers]
+    total = sum(by_layer[entry.layer] for entry in model.spec.schedule)
+    if model.input_join is not None:
+        total += of(model.input_join) * sum(entry.joins_input for entry in model.spec.schedule)
+    return total
 
 
 def head_flops_per_row(model) -> int:

@@ -1140,7 +1140,7 @@ def attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,
 
 # ---- attention whose weights are sigmoids and whose heads mix them ------------------------------------------
 SIGMOID_MAX_HEADS = 256         # of the plain kernel (the matrix-core kernels: see sigmoid_attention_is_tiled)
-SIGMOID_DECODE_WORKGROUPS = 512     # two per compute unit: up to here every page of a row gets a workgroup of its own
+SIGMOID_DECODE_WORKGROUPS = 256     # one per compute unit: up to here every page of a row gets a workgroup of its own
 
 
 def sigmoid_attention_is_tiled(num_heads: int, head_dim: int, v_dim: int) -> bool:
@@ -1191,8 +1191,11 @@ def sigmoid_attention_generic(q: torch.Tensor, num_heads: int, num_kv_heads: int
 def sigmoid_attention_prefill(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, v_dim: int, k_pages: torch.Tensor,
                               v_pages: torch.Tensor, block_table: torch.Tensor, tile_seg: torch.Tensor, tile_row0: torch.Tensor,
                               seg_row0: torch.Tensor, row_pos: torch.Tensor, scale: float, window: int, bias: torch.Tensor,
-                              mix: torch.Tensor, gate: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """The same on the matrix cores for the rows of the given tiles (of up to 64 rows; ``attention_prefill``)."""
+                              mix: torch.Tensor, gate: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None,
+                              max_context: int = 0, parts: int = 0) -> torch.Tensor:
+    """The same on the matrix cores for the rows of the given tiles (of up to 64 rows; ``attention_prefill``).
+    ``max_context`` bounds position + 1 of every row (0: what the block table holds). ``parts``: workgroups that share the keys of
+    16 rows (0: as many as fill the chip)."""
     rows = q.shape[0]
     _dev(q, tile_seg, tile_row0, seg_row0)
     _want(q, torch.bfloat16, "q")
@@ -1205,8 +1208,14 @@ def sigmoid_attention_prefill(q: torch.Tensor, num_heads: int, num_kv_heads: int
         out = torch.empty((rows, num_heads * v_dim), dtype=q.dtype, device=q.device)
     elif out.shape != (rows, num_heads * v_dim) or out.dtype != q.dtype or not out.is_contiguous():
         raise KernelError("sigmoid_attention: out must be bfloat16 [rows, heads * v_dim]")
+    floats, counters = ctypes.c_longlong(0), ctypes.c_int(0)
+    parts = library().fw_sigmoid_attention_prefill_plan(tile_seg.numel(), num_heads, head_dim, v_dim, int(window),
+                                                        int(max_context) or block_table.shape[1] * PAGE_SIZE, int(parts),
+                                                        ctypes.byref(floats), ctypes.byref(counters))
+    partial = torch.empty((floats.value,), dtype=torch.float32, device=q.device) if parts > 1 else None
+    tickets = _medium_counters(q.device, counters.value)
     _check(library().fw_sigmoid_attention_prefill(
-        _p(q), _p(out), _p(k_pages), _p(v_pages), _p(block_table), block_table.shape[1], _p(tile_seg), _p(tile_row0), tile_seg.numel(),
+        _p(q), _p(out), _p(partial), ctypes.c_longlong(floats.value), _p(tickets), tickets.numel(), parts, _p(k_pages), _p(v_pages), _p(block_table), block_table.shape[1], _p(tile_seg), _p(tile_row0), tile_seg.numel(),
         _p(seg_row0), _p(row_pos), rows, num_heads, num_kv_heads, head_dim, v_dim, ctypes.c_float(scale), int(window), _p(bias), _p(mix),
         _p(gate), _stride(gate) if gate is not None else 0, PAGE_SIZE, pages, _stream()))
     return out
@@ -1282,7 +1291,8 @@ def sigmoid_attention(q: torch.Tensor, num_heads: int, num_kv_heads: int, head_d
         if tile_seg is None or tile_row0 is None:
             raise KernelError("sigmoid_attention: the tiled kernel needs the step's query tiles")
         sigmoid_attention_prefill(q, num_heads, num_kv_heads, head_dim, v_dim, k_pages, v_pages, block_table, tile_seg[single:],
-                                  tile_row0[single:], ctx.seg_row0, ctx.row_pos, scale, window, bias, mix, gate, out=out)
+                                  tile_row0[single:], ctx.seg_row0, ctx.row_pos, scale, window, bias, mix, gate, out=out,
+                                  max_context=ctx.max_context)
     return out
 
 
