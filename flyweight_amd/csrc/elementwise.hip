@@ -421,7 +421,7 @@ __global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __rest
     const int row = blockIdx.x;
     const float* source = x + (size_t)(row_index ? row_index[row] : row) * hidden;
     const bool held_all = hidden <= 256 * 16;
-    float held[16], scale[16];
+    float held[16], scale[16], shift[16];
     float sum = 0.0f;
     if (held_all) {
 #pragma unroll
@@ -429,6 +429,7 @@ __global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __rest
             const int i = threadIdx.x + 256 * u;
             held[u] = i < hidden ? source[i] : 0.0f;
             scale[u] = i < hidden ? weight[i] : 0.0f;
+            shift[u] = (bias && i < hidden) ? bias[i] : 0.0f;       // asked for with the rest, not behind the sums
             sum += held[u];
         }
     } else {
@@ -455,7 +456,7 @@ __global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __rest
             const int i = threadIdx.x + 256 * u;
             if (i < hidden) {
                 const float normed = (held[u] - mean) * inv * scale[u];
-                store_from_float(out, (size_t)row * hidden + i, bias ? normed + bias[i] : normed);
+                store_from_float(out, (size_t)row * hidden + i, bias ? normed + shift[u] : normed);
             }
         }
     } else {

@@ -195,109 +195,117 @@ extern "C" int fw_clamped_glu(const void* gate_up, int in_dtype, void* out, int 
 // A norm here is v / sqrt(mean(v^2) + eps), v the values or their deviations from the row's mean. One
 // workgroup per row; a row of up to 256 * JOIN_HELD values stays in registers between the passes, a
 // wider one is read again. Every sum is a function of the row alone.
+// A row that stays in registers asks for everything it will need at once (with few rows nothing else hides a
+// second trip to memory), meets over LDS alone, and writes x last (a barrier behind a store would wait for it).
 #define JOIN_HELD 16
-template <typename T, bool HELD>
-__global__ __launch_bounds__(256) void norm_add_norm_kernel(
+__device__ __forceinline__ float join_block_sum(float v, float* scratch) {      // 256 threads; scratch: 4 floats of its own
+    v = wave_sum(v);
+    if ((threadIdx.x & 63) == 0) scratch[threadIdx.x >> 6] = v;
+    fw_lds_barrier();
+    return ((scratch[0] + scratch[1]) + scratch[2]) + scratch[3];
+}
+template <typename T, int N>
+__global__ __launch_bounds__(256) void norm_add_norm_held_kernel(
+    float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ weight, const float* __restrict__ bias, float mult,
+    int centered, float eps, int next_kind, const float* __restrict__ next_weight, const float* __restrict__ next_bias, float next_eps,
+    T* __restrict__ next_out, int next_stride, int hidden) {
+    __shared__ float scratch[4][4];
+    const size_t row0 = (size_t)blockIdx.x * hidden;
+    const float count = (float)hidden;
+    float held[N], was[N], scale[N], shift[N], next_scale[N], next_shift[N];
+    float sum = 0.0f;
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+        const int i = threadIdx.x + 256 * u < hidden ? threadIdx.x + 256 * u : hidden - 1;      // past the end: read again, not used
+        held[u] = a[row0 + i];
+        was[u] = x[row0 + i];
+        scale[u] = weight[i];
+        shift[u] = bias ? bias[i] : 0.0f;
+        next_scale[u] = next_kind >= 2 ? next_weight[i] : 0.0f;
+        next_shift[u] = (next_kind >= 2 && next_bias) ? next_bias[i] : 0.0f;
+    }
+#pragma unroll
+    for (int u = 0; u < N; ++u) sum += threadIdx.x + 256 * u < hidden ? held[u] : 0.0f;
+    const float mean = centered ? join_block_sum(sum, scratch[0]) / count : 0.0f;
+    float squares = 0.0f;
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+        const float d = threadIdx.x + 256 * u < hidden ? held[u] - mean : 0.0f;
+        squares = fmaf(d, d, squares);
+    }
+    const float inv = 1.0f / sqrtf(join_block_sum(squares, scratch[1]) / count + eps);
+    float new_sum = 0.0f;
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+        const float normed = (held[u] - mean) * inv * scale[u];
+        was[u] = fmaf(mult, bias ? normed + shift[u] : normed, was[u]);
+        new_sum += threadIdx.x + 256 * u < hidden ? was[u] : 0.0f;
+    }
+    float next_mean = 0.0f, next_inv = 1.0f;
+    if (next_kind >= 2) {
+        next_mean = next_kind == 3 ? join_block_sum(new_sum, scratch[2]) / count : 0.0f;
+        float next_squares = 0.0f;
+#pragma unroll
+        for (int u = 0; u < N; ++u) {
+            const float d = threadIdx.x + 256 * u < hidden ? was[u] - next_mean : 0.0f;
+            next_squares = fmaf(d, d, next_squares);
+        }
+        next_inv = 1.0f / sqrtf(join_block_sum(next_squares, scratch[3]) / count + next_eps);
+    }
+    next_out += (size_t)blockIdx.x * next_stride;
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+        const int i = threadIdx.x + 256 * u;
+        if (i >= hidden) break;
+        x[row0 + i] = was[u];
+        if (next_kind == 1) store_from_float(next_out, i, was[u]);
+        if (next_kind >= 2) {
+            const float normed = (was[u] - next_mean) * next_inv * next_scale[u];
+            store_from_float(next_out, i, next_bias ? normed + next_shift[u] : normed);
+        }
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void norm_add_norm_wide_kernel(
     float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ weight, const float* __restrict__ bias, float mult,
     int centered, float eps, int next_kind, const float* __restrict__ next_weight, const float* __restrict__ next_bias, float next_eps,
     T* __restrict__ next_out, int next_stride, int hidden) {
     __shared__ float scratch[16];
     const size_t row0 = (size_t)blockIdx.x * hidden;
     next_out += (size_t)blockIdx.x * next_stride;
-    constexpr int N = HELD ? JOIN_HELD : 1;
-    float held[N], was[N], scale[N];
     const float count = (float)hidden;
     float sum = 0.0f;
-    if (HELD) {
-#pragma unroll
-        for (int u = 0; u < N; ++u) {
-            const int i = threadIdx.x + 256 * u;
-            const bool in = i < hidden;
-            held[u] = in ? a[row0 + i] : 0.0f;
-            was[u] = in ? x[row0 + i] : 0.0f;
-            scale[u] = in ? weight[i] : 0.0f;
-            sum += held[u];
-        }
-    } else {
-        for (int i = threadIdx.x; i < hidden; i += 256) sum += a[row0 + i];
-    }
+    for (int i = threadIdx.x; i < hidden; i += 256) sum += a[row0 + i];
     const float mean = centered ? block_sum(sum, scratch) / count : 0.0f;
     float squares = 0.0f;
-    if (HELD) {
-#pragma unroll
-        for (int u = 0; u < N; ++u) {
-            const float d = threadIdx.x + 256 * u < hidden ? held[u] - mean : 0.0f;
-            squares = fmaf(d, d, squares);
-        }
-    } else {
-        for (int i = threadIdx.x; i < hidden; i += 256) {
-            const float d = a[row0 + i] - mean;
-            squares = fmaf(d, d, squares);
-        }
+    for (int i = threadIdx.x; i < hidden; i += 256) {
+        const float d = a[row0 + i] - mean;
+        squares = fmaf(d, d, squares);
     }
     const float inv = 1.0f / sqrtf(block_sum(squares, scratch) / count + eps);
     float new_sum = 0.0f;
-    if (HELD) {
-#pragma unroll
-        for (int u = 0; u < N; ++u) {
-            const int i = threadIdx.x + 256 * u;
-            if (i < hidden) {
-                const float normed = (held[u] - mean) * inv * scale[u];
-                was[u] = fmaf(mult, bias ? normed + bias[i] : normed, was[u]);
-                x[row0 + i] = was[u];
-                new_sum += was[u];
-            }
-        }
-    } else {
-        for (int i = threadIdx.x; i < hidden; i += 256) {
-            const float normed = (a[row0 + i] - mean) * inv * weight[i];
-            const float updated = fmaf(mult, bias ? normed + bias[i] : normed, x[row0 + i]);
-            x[row0 + i] = updated;          // read again below by the thread that wrote it
-            new_sum += updated;
-        }
+    for (int i = threadIdx.x; i < hidden; i += 256) {
+        const float normed = (a[row0 + i] - mean) * inv * weight[i];
+        const float updated = fmaf(mult, bias ? normed + bias[i] : normed, x[row0 + i]);
+        x[row0 + i] = updated;          // read again below by the thread that wrote it
+        new_sum += updated;
     }
     if (next_kind == 0) return;
     if (next_kind == 1) {
-        if (HELD) {
-#pragma unroll
-            for (int u = 0; u < N; ++u) {
-                const int i = threadIdx.x + 256 * u;
-                if (i < hidden) store_from_float(next_out, i, was[u]);
-            }
-        } else {
-            for (int i = threadIdx.x; i < hidden; i += 256) store_from_float(next_out, i, x[row0 + i]);
-        }
+        for (int i = threadIdx.x; i < hidden; i += 256) store_from_float(next_out, i, x[row0 + i]);
         return;
     }
     const float next_mean = next_kind == 3 ? block_sum(new_sum, scratch) / count : 0.0f;
     float next_squares = 0.0f;
-    if (HELD) {
-#pragma unroll
-        for (int u = 0; u < N; ++u) {
-            const float d = threadIdx.x + 256 * u < hidden ? was[u] - next_mean : 0.0f;
-            next_squares = fmaf(d, d, next_squares);
-        }
-    } else {
-        for (int i = threadIdx.x; i < hidden; i += 256) {
-            const float d = x[row0 + i] - next_mean;
-            next_squares = fmaf(d, d, next_squares);
-        }
+    for (int i = threadIdx.x; i < hidden; i += 256) {
+        const float d = x[row0 + i] - next_mean;
+        next_squares = fmaf(d, d, next_squares);
     }
     const float next_inv = 1.0f / sqrtf(block_sum(next_squares, scratch) / count + next_eps);
-    if (HELD) {
-#pragma unroll
-        for (int u = 0; u < N; ++u) {
-            const int i = threadIdx.x + 256 * u;
-            if (i < hidden) {
-                const float normed = (was[u] - next_mean) * next_inv * next_weight[i];
-                store_from_float(next_out, i, next_bias ? normed + next_bias[i] : normed);
-            }
-        }
-    } else {
-        for (int i = threadIdx.x; i < hidden; i += 256) {
-            const float normed = (x[row0 + i] - next_mean) * next_inv * next_weight[i];
-            store_from_float(next_out, i, next_bias ? normed + next_bias[i] : normed);
-        }
+    for (int i = threadIdx.x; i < hidden; i += 256) {
+        const float normed = (x[row0 + i] - next_mean) * next_inv * next_weight[i];
+        store_from_float(next_out, i, next_bias ? normed + next_bias[i] : normed);
     }
 }
 
@@ -315,17 +323,20 @@ extern "C" int fw_norm_add_norm(float* x, const float* a, const float* weight, c
     FW_REQUIRE(next_kind == 0 || next_dtype == FW_F32 || next_dtype == FW_BF16, "norm_add_norm: unknown dtype %d", next_dtype);
     if (rows == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
-    const bool held = hidden <= 256 * JOIN_HELD;
-#define FW_JOIN_LAUNCH(T, HELD)                                                                                             \
-    norm_add_norm_kernel<T, HELD><<<rows, 256, 0, s>>>(x, a, weight, bias, mult, centered, eps, next_kind, next_weight, \
-                                                       next_bias, next_eps, (T*)next_out, next_stride, hidden)
+#define FW_JOIN_LAUNCH(KERNEL, T)                                                                                                    \
+    KERNEL<<<rows, 256, 0, s>>>(x, a, weight, bias, mult, centered, eps, next_kind, next_weight, next_bias, next_eps, (T*)next_out, \
+                                next_stride, hidden)
+#define FW_JOIN_BY_WIDTH(T)                                                                            \
+    if (hidden <= 256 * 4) FW_JOIN_LAUNCH((norm_add_norm_held_kernel<T, 4>), T);                       \
+    else if (hidden <= 256 * 8) FW_JOIN_LAUNCH((norm_add_norm_held_kernel<T, 8>), T);                  \
+    else if (hidden <= 256 * JOIN_HELD) FW_JOIN_LAUNCH((norm_add_norm_held_kernel<T, JOIN_HELD>), T); \
+    else FW_JOIN_LAUNCH((norm_add_norm_wide_kernel<T>), T)
     if (next_kind == 0 || next_dtype == FW_F32) {
-        if (held) FW_JOIN_LAUNCH(float, true);
-        else FW_JOIN_LAUNCH(float, false);
+        FW_JOIN_BY_WIDTH(float);
     } else {
-        if (held) FW_JOIN_LAUNCH(bf16_t, true);
-        else FW_JOIN_LAUNCH(bf16_t, false);
+        FW_JOIN_BY_WIDTH(bf16_t);
     }
+#undef FW_JOIN_BY_WIDTH
 #undef FW_JOIN_LAUNCH
     FW_LAUNCH_CHECK("norm_add_norm");
     return 0;
