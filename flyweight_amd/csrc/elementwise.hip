@@ -412,7 +412,43 @@ extern "C" int fw_fill_zero(void* ptr, long long bytes, void* stream) {
 // ---- layer norm with a weight and an optional bias ---------------------------------------------------
 // out[r] = (x[src] - mean) / sqrt(mean((x[src] - mean)^2) + eps) * w (+ bias), src = row_index ? row_index[r] : r.
 // The mean first, then the mean of the squared deviations from it (not E[x^2] - mean^2, which loses
-// digits where the mean is large beside the spread). A row of up to 4,096 values stays in registers.
+// digits where the mean is large beside the spread). A row of up to 4,096 values stays in registers and is
+// asked for at once with what scales and shifts it; a wider one is read again.
+template <typename T, int N>
+__global__ __launch_bounds__(256) void layernorm_rows_held_kernel(const float* __restrict__ x, const float* __restrict__ weight,
+                                                                  const float* __restrict__ bias, T* __restrict__ out,
+                                                                  const int32_t* __restrict__ row_index, int hidden, float eps) {
+    __shared__ float scratch[2][4];
+    const int row = blockIdx.x;
+    const float* source = x + (size_t)(row_index ? row_index[row] : row) * hidden;
+    float held[N], scale[N], shift[N];
+    float sum = 0.0f;
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+        const int i = threadIdx.x + 256 * u < hidden ? threadIdx.x + 256 * u : hidden - 1;      // past the end: read again, not used
+        held[u] = source[i];
+        scale[u] = weight[i];
+        shift[u] = bias ? bias[i] : 0.0f;
+    }
+#pragma unroll
+    for (int u = 0; u < N; ++u) sum += threadIdx.x + 256 * u < hidden ? held[u] : 0.0f;
+    const float mean = block_sum_by_lds(sum, scratch[0]) / (float)hidden;
+    float squares = 0.0f;
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+        const float d = threadIdx.x + 256 * u < hidden ? held[u] - mean : 0.0f;
+        squares = fmaf(d, d, squares);
+    }
+    const float inv = 1.0f / sqrtf(block_sum_by_lds(squares, scratch[1]) / (float)hidden + eps);
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+        const int i = threadIdx.x + 256 * u;
+        if (i >= hidden) break;
+        const float normed = (held[u] - mean) * inv * scale[u];
+        store_from_float(out, (size_t)row * hidden + i, bias ? normed + shift[u] : normed);
+    }
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __restrict__ x, const float* __restrict__ weight, const float* __restrict__ bias,
                                                              T* __restrict__ out, const int32_t* __restrict__ row_index,
@@ -420,50 +456,18 @@ __global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __rest
     __shared__ float scratch[16];
     const int row = blockIdx.x;
     const float* source = x + (size_t)(row_index ? row_index[row] : row) * hidden;
-    const bool held_all = hidden <= 256 * 16;
-    float held[16], scale[16], shift[16];
     float sum = 0.0f;
-    if (held_all) {
-#pragma unroll
-        for (int u = 0; u < 16; ++u) {
-            const int i = threadIdx.x + 256 * u;
-            held[u] = i < hidden ? source[i] : 0.0f;
-            scale[u] = i < hidden ? weight[i] : 0.0f;
-            shift[u] = (bias && i < hidden) ? bias[i] : 0.0f;       // asked for with the rest, not behind the sums
-            sum += held[u];
-        }
-    } else {
-        for (int i = threadIdx.x; i < hidden; i += 256) sum += source[i];
-    }
+    for (int i = threadIdx.x; i < hidden; i += 256) sum += source[i];
     const float mean = block_sum(sum, scratch) / (float)hidden;
     float squares = 0.0f;
-    if (held_all) {
-#pragma unroll
-        for (int u = 0; u < 16; ++u) {
-            const float d = threadIdx.x + 256 * u < hidden ? held[u] - mean : 0.0f;
-            squares = fmaf(d, d, squares);
-        }
-    } else {
-        for (int i = threadIdx.x; i < hidden; i += 256) {
-            const float d = source[i] - mean;
-            squares = fmaf(d, d, squares);
-        }
+    for (int i = threadIdx.x; i < hidden; i += 256) {
+        const float d = source[i] - mean;
+        squares = fmaf(d, d, squares);
     }
     const float inv = 1.0f / sqrtf(block_sum(squares, scratch) / (float)hidden + eps);
-    if (held_all) {
-#pragma unroll
-        for (int u = 0; u < 16; ++u) {
-            const int i = threadIdx.x + 256 * u;
-            if (i < hidden) {
-                const float normed = (held[u] - mean) * inv * scale[u];
-                store_from_float(out, (size_t)row * hidden + i, bias ? normed + shift[u] : normed);
-            }
-        }
-    } else {
-        for (int i = threadIdx.x; i < hidden; i += 256) {
-            const float normed = (source[i] - mean) * inv * weight[i];
-            store_from_float(out, (size_t)row * hidden + i, bias ? normed + bias[i] : normed);
-        }
+    for (int i = threadIdx.x; i < hidden; i += 256) {
+        const float normed = (source[i] - mean) * inv * weight[i];
+        store_from_float(out, (size_t)row * hidden + i, bias ? normed + bias[i] : normed);
     }
 }
 
@@ -472,12 +476,16 @@ extern "C" int fw_layernorm_rows(const float* x, const float* weight, const floa
     FW_REQUIRE(rows >= 0 && hidden > 0, "layernorm_rows: bad sizes rows=%d hidden=%d", rows, hidden);
     FW_REQUIRE(eps > 0.0f, "layernorm_rows: eps must be positive");
     if (rows == 0) return 0;
-    if (out_dtype == FW_F32)
-        layernorm_rows_kernel<float><<<rows, 256, 0, (hipStream_t)stream>>>(x, weight, bias, (float*)out, row_index, hidden, eps);
-    else if (out_dtype == FW_BF16)
-        layernorm_rows_kernel<bf16_t><<<rows, 256, 0, (hipStream_t)stream>>>(x, weight, bias, (bf16_t*)out, row_index, hidden, eps);
-    else
-        FW_REQUIRE(false, "layernorm_rows: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16, "layernorm_rows: unknown out dtype %d", out_dtype);
+#define FW_LN_LAUNCH(KERNEL, T) KERNEL<<<rows, 256, 0, (hipStream_t)stream>>>(x, weight, bias, (T*)out, row_index, hidden, eps)
+#define FW_LN_BY_WIDTH(T)                                                                          \
+    if (hidden <= 256 * 4) FW_LN_LAUNCH((layernorm_rows_held_kernel<T, 4>), T);                    \
+    else if (hidden <= 256 * 8) FW_LN_LAUNCH((layernorm_rows_held_kernel<T, 8>), T);               \
+    else if (hidden <= 256 * 16) FW_LN_LAUNCH((layernorm_rows_held_kernel<T, 16>), T);             \
+    else FW_LN_LAUNCH(layernorm_rows_kernel<T>, T)
+    if (out_dtype == FW_F32) { FW_LN_BY_WIDTH(float); } else { FW_LN_BY_WIDTH(bf16_t); }
+#undef FW_LN_BY_WIDTH
+#undef FW_LN_LAUNCH
     FW_LAUNCH_CHECK("layernorm_rows");
     return 0;
 }

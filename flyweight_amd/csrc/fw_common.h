@@ -156,6 +156,15 @@ __device__ __forceinline__ float block_sum(float v, float* scratch /* >= 16 floa
     return total;
 }
 
+// The same over 256 threads, the waves meeting over LDS alone (loads and stores on the way stay on the way);
+// the parts are added in the same order. Every sum of a kernel has four floats of its own.
+__device__ __forceinline__ float block_sum_by_lds(float v, float* scratch) {
+    v = wave_sum(v);
+    if ((threadIdx.x & 63) == 0) scratch[threadIdx.x >> 6] = v;
+    fw_lds_barrier();
+    return ((scratch[0] + scratch[1]) + scratch[2]) + scratch[3];
+}
+
 // A gated unit behind a product that holds gate and up of one feature: silu(g) * u (limit <= 0), or
 // with clamped halves g' = min(g, limit), u' = clamp(u, -limit, limit): g' * sigmoid(alpha g') * (u' + shift).
 // `silu` is the product's own form of silu(g) * u, so that the plain unit's results stay what they were.
@@ -172,6 +181,20 @@ __device__ __forceinline__ float fw_gated_unit(float g, float u, float limit, fl
 // z Phi(z), Phi the normal distribution's cumulative function: the exact gelu
 __device__ __forceinline__ float fw_gelu(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
 
+// The same for results that are rounded to bfloat16: the complement of the error function as a polynomial in 1 / (1 + p x)
+// times e^(-x^2) (Abramowitz and Stegun, Handbook of Mathematical Functions, 7.1.26: within 1.5e-7), which gives the
+// lower half of Phi without a difference of nearly equal numbers.
+__device__ __forceinline__ float fw_gelu_quick(float z) {
+    const float x = fabsf(z) * 0.70710678118654752f;
+    const float t = __builtin_amdgcn_rcpf(fmaf(0.3275911f, x, 1.0f));
+    float poly = fmaf(1.061405429f, t, -1.453152027f);
+    poly = fmaf(poly, t, 1.421413741f);
+    poly = fmaf(poly, t, -0.284496736f);
+    poly = fmaf(poly, t, 0.254829592f);
+    const float lower = 0.5f * poly * t * __builtin_amdgcn_exp2f(-x * x * 1.4426950408889634f);      // Phi(-|z|)
+    return z * (z < 0.0f ? lower : 1.0f - lower);
+}
+
 // A product that stores gelu(sum) in bfloat16 is the storing product with this output type (dtype code
 // FW_BF16_GELU): the unit is formed from the float32 sum and rounded once.
 #define FW_BF16_GELU 2
@@ -180,11 +203,11 @@ struct gelu_bf16_t {
 };
 template <> __device__ __forceinline__ float load_as_float<gelu_bf16_t>(const gelu_bf16_t* p, size_t i) { return bf16_bits_to_float(p[i].bits); }
 template <> __device__ __forceinline__ void store_from_float<gelu_bf16_t>(gelu_bf16_t* p, size_t i, float v) {
-    p[i].bits = float_to_bf16_bits(fw_gelu(v));
+    p[i].bits = float_to_bf16_bits(fw_gelu_quick(v));
 }
 // what a store of this output type does to a float32 sum before it is rounded (for stores that pack several values)
 template <typename T> __device__ __forceinline__ float fw_before_store(float v) { return v; }
-template <> __device__ __forceinline__ float fw_before_store<gelu_bf16_t>(float v) { return fw_gelu(v); }
+template <> __device__ __forceinline__ float fw_before_store<gelu_bf16_t>(float v) { return fw_gelu_quick(v); }
 
 // The first key that a row at position `pos` may see: with a window the last `window` keys (itself
 // among them), with a chunk only the keys of its own chunk (chunks counted from position 0 of the

@@ -198,12 +198,6 @@ extern "C" int fw_clamped_glu(const void* gate_up, int in_dtype, void* out, int 
 // A row that stays in registers asks for everything it will need at once (with few rows nothing else hides a
 // second trip to memory), meets over LDS alone, and writes x last (a barrier behind a store would wait for it).
 #define JOIN_HELD 16
-__device__ __forceinline__ float join_block_sum(float v, float* scratch) {      // 256 threads; scratch: 4 floats of its own
-    v = wave_sum(v);
-    if ((threadIdx.x & 63) == 0) scratch[threadIdx.x >> 6] = v;
-    fw_lds_barrier();
-    return ((scratch[0] + scratch[1]) + scratch[2]) + scratch[3];
-}
 template <typename T, int N>
 __global__ __launch_bounds__(256) void norm_add_norm_held_kernel(
     float* __restrict__ x, const float* __restrict__ a, const float* __restrict__ weight, const float* __restrict__ bias, float mult,
@@ -226,14 +220,14 @@ __global__ __launch_bounds__(256) void norm_add_norm_held_kernel(
     }
 #pragma unroll
     for (int u = 0; u < N; ++u) sum += threadIdx.x + 256 * u < hidden ? held[u] : 0.0f;
-    const float mean = centered ? join_block_sum(sum, scratch[0]) / count : 0.0f;
+    const float mean = centered ? block_sum_by_lds(sum, scratch[0]) / count : 0.0f;
     float squares = 0.0f;
 #pragma unroll
     for (int u = 0; u < N; ++u) {
         const float d = threadIdx.x + 256 * u < hidden ? held[u] - mean : 0.0f;
         squares = fmaf(d, d, squares);
     }
-    const float inv = 1.0f / sqrtf(join_block_sum(squares, scratch[1]) / count + eps);
+    const float inv = 1.0f / sqrtf(block_sum_by_lds(squares, scratch[1]) / count + eps);
     float new_sum = 0.0f;
 #pragma unroll
     for (int u = 0; u < N; ++u) {
@@ -243,14 +237,14 @@ __global__ __launch_bounds__(256) void norm_add_norm_held_kernel(
     }
     float next_mean = 0.0f, next_inv = 1.0f;
     if (next_kind >= 2) {
-        next_mean = next_kind == 3 ? join_block_sum(new_sum, scratch[2]) / count : 0.0f;
+        next_mean = next_kind == 3 ? block_sum_by_lds(new_sum, scratch[2]) / count : 0.0f;
         float next_squares = 0.0f;
 #pragma unroll
         for (int u = 0; u < N; ++u) {
             const float d = threadIdx.x + 256 * u < hidden ? was[u] - next_mean : 0.0f;
             next_squares = fmaf(d, d, next_squares);
         }
-        next_inv = 1.0f / sqrtf(join_block_sum(next_squares, scratch[3]) / count + next_eps);
+        next_inv = 1.0f / sqrtf(block_sum_by_lds(next_squares, scratch[3]) / count + next_eps);
     }
     next_out += (size_t)blockIdx.x * next_stride;
 #pragma unroll
