@@ -2,7 +2,7 @@
 
 Zaluvik is a decoder with a layer norm (weight and bias) before and behind every sublayer, x += m N1b(mixer(N1(x))), then
 x += m N2b(ff(N2(x))), with one factor m for the model (``residual_mult``). ``loop`` names a run of neighbouring layers
-(``start`` .. ``stop`` - 1) that is passed ``times`` times in a row with the same weights, each pass with pages of its own;
+(``start`` .. ``stop`` - 1) that every token passes ``times`` times, one set of weights, pages of its own for each pass;
 ahead of every pass the residual stream becomes ``loop.in`` times [stream; embedding output]. ``layers`` lists the layers, each
 with its ``type``: ``attention`` (grouped heads without positions whose weights are sigmoids that the heads mix, see
 ``parts/sigmoid_attention.py``) or ``latent_attention`` (softmax attention over a cached latent with a rotated key part that

@@ -819,7 +819,7 @@ __global__ __launch_bounds__(256) void sigmoid_attention_decode_kernel(
 }
 
 // One row per request. q: finished bfloat16 queries, or null with `qkv` (float32 [rows][qkv_stride]: q | k | v as the
-// projections leave them; qk_norm: q and k of a head are divided by their root mean square; write_kv: the new key
+// projections leave them; qk_norm: q and k of a head are brought to unit RMS; write_kv: the new key
 // and value are stored). partial: float32 workspace of rows * max_splits * heads * v_dim; tickets: a zeroed int32 per row, left
 // zero. max_context: no row's position reaches it; max_splits * pages_per_split covers the pages such a row sees.
 extern "C" int fw_sigmoid_attention_decode(const void* q, const float* qkv, int qkv_stride, int qk_norm, float eps, int write_kv, void* out,

@@ -218,7 +218,7 @@ int fw_sigmoid_attention_prefill(const void* q, void* out, float* partial, long 
                                  int head_dim, int v_dim, float scale, int window, const float* bias, const float* mix,
                                  const float* gate, int gate_stride, int page_size, int num_pages, void* stream);
 // One row per request: from finished bfloat16 queries q, or (q null) from the raw projections qkv (float32 rows of qkv_stride:
-// q | k | v), whose queries and keys are divided by their root mean square per head (qk_norm; eps under the root) and whose
+// q | k | v), whose queries and keys are brought to unit RMS per head (qk_norm; eps under the root) and whose
 // keys and values are stored first (write_kv). max_splits workgroups of pages_per_split pages cover what a row sees;
 // partial: float32 [rows][max_splits][heads * v_dim]; tickets: an int32 per row, zero before and after.
 int fw_sigmoid_attention_decode(const void* q, const float* qkv, int qkv_stride, int qk_norm, float eps, int write_kv, void* out,
@@ -365,7 +365,7 @@ int fw_wkv_recurrence(const float* r, const float* k, const float* v, int rkv_st
 // chosen / weight [rows][top]: the `top` largest of logits[r] + bias (float32 [rows][experts]; ties: the lowest
 // id; bias may be null), largest first, and the softmax over those alone. groups > 1: the experts form that many equal
 // groups of neighbours, a group's score is its best expert's, and only experts of the `keep` best groups (ties: the
-// lowest group) can be chosen; group_pair: a group's score is the sum of its two best experts' scores. scores 0: the weights as
+// lowest group) can be chosen; group_pair: groups are ranked by what their two best experts score together. scores 0: the weights as
 // said; 1: the softmax over ALL experts at the chosen ones, divided by their sum + 1e-20; 2: each expert's own sigmoid
 // at the chosen ones, divided by their sum + 1e-20.
 int fw_moe_route(const float* logits, const float* bias, int32_t* chosen, float* weight, int rows, int experts, int top,

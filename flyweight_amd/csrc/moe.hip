@@ -18,8 +18,8 @@
 #define MOE_MAX_EXPERTS 1024
 #define MOE_MAX_TOP 64
 // groups > 1: the experts form that many equal groups of neighbours, a group's score is its best expert's, and only
-// experts of the `keep` best groups (ties: the lowest group) can be chosen. group_pair: a group's score is the sum of its
-// two best experts' scores instead (of its one's, where it has no second). scores 0: the weights are the softmax over the chosen
+// experts of the `keep` best groups (ties: the lowest group) can be chosen. group_pair: groups are ranked by what their
+// two best experts score together instead (by the one's, where it has no second). scores 0: the weights are the softmax over the chosen
 // alone; 1: the softmax over ALL experts at the chosen ones, divided by their sum + 1e-20; 2: sigmoids of the
 // logits, each expert's on its own, at the chosen ones, divided by their sum + 1e-20.
 #define MOE_SOFTMAX_CHOSEN 0

@@ -1696,7 +1696,7 @@ def moe_route(logits: torch.Tensor, bias: Optional[torch.Tensor], top: int, grou
     (of neighbours, equal in size) whose best expert scores highest can be chosen. ``score_all``: the weights are the
     softmax over all experts at the chosen ones, divided by their sum + 1e-20. ``scores`` names the same choice
     ("softmax_chosen", "softmax_all") or "sigmoid": each expert's own sigmoid at the chosen ones, divided by their sum + 1e-20.
-    ``group_pair``: a group's score is the sum of its two best experts' scores (not with "softmax_chosen")."""
+    ``group_pair``: groups are ranked by what their two best experts score together (not with "softmax_chosen")."""
     scores = scores or ("softmax_all" if score_all else "softmax_chosen")
     if scores not in MOE_SCORES or (group_pair and scores == "softmax_chosen"):
         raise KernelError(f"moe_route: scores {scores!r} (known: {', '.join(MOE_SCORES)}; groups by pairs: {group_pair})")

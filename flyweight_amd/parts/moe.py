@@ -11,8 +11,8 @@ pairs as tiles of one grouped product, so nothing crosses to the host and a deco
 ``router_scores`` "softmax_all": the scores are the softmax over all experts, and the chosen experts' scores divided by
 their sum (+ 1e-20) are the weights (the choice is the same: the largest scores are the largest logits).
 ``router_groups`` (count, keep): the experts form ``count`` equal groups of neighbours, a group's score is its best
-expert's, and only experts of the ``keep`` best groups can be chosen; ``group_score`` "pair": a group's score is the sum of
-its two best experts' scores instead. ``router_scores`` "sigmoid": every expert scores sigmoid(z) on its own, and the
+expert's, and only experts of the ``keep`` best groups can be chosen; ``group_score`` "pair": groups are ranked by what their
+two best experts score together instead. ``router_scores`` "sigmoid": every expert scores sigmoid(z) on its own, and the
 chosen scores divided by their sum (+ 1e-20) are the weights. ``unit`` "clamped" with ``limit`` (and ``alpha``,
 ``shift``): an expert is W_down (g sigmoid(alpha g) (u + shift)) with g = min(W_gate h, limit), u = clamp(W_up h, -limit,
 limit); the shared unit is then of the same form with ``shared_limit``. Registered as ``moe_swiglu`` and ``moe_glu``.

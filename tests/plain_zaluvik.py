@@ -69,7 +69,7 @@ def mixed_heads(q: np.ndarray, keys: np.ndarray, values: np.ndarray, start: int,
                 mix: np.ndarray, window: Optional[int]) -> np.ndarray:
     """q [T, H, d] are the rows at positions start .. start + T - 1 of a sequence whose keys [N, G, d] and values
     [N, G, dv] are given from position 0 on. a_g(i, j) = sigmoid(q_g . k * scale + bias_g) for the visible keys;
-    head h weighs the values of its own key/value head with sum_g mix[h, g] a_g(i, j). Returns [T, H, dv]."""
+    head h weighs the values of key head h // (H / G) with sum_g mix[h, g] a_g(i, j). Returns [T, H, dv]."""
     T, H, _ = q.shape
     per = H // keys.shape[1]
     out = np.zeros((T, H, values.shape[2]))
