@@ -6,6 +6,7 @@ from .vavelorn import VavelornConfig
 from .dalerax import DaleraxConfig
 from .telapel import TelapelConfig
 from .zaluvik import ZaluvikConfig
+from .fevolorn import FevolornConfig
 from .registry import (architecture_name, config_from_dict, load_config,
                        register_architecture, registered_architectures)
 
@@ -16,9 +17,10 @@ register_architecture("Vavelorn", VavelornConfig)
 register_architecture("Dalerax", DaleraxConfig)
 register_architecture("Telapel", TelapelConfig)
 register_architecture("Zaluvik", ZaluvikConfig)
+register_architecture("Fevolorn", FevolornConfig)
 
 __all__ = [
     "ConfigError", "LayerSpec", "ModelSpec", "PartSpec", "ScheduleEntry", "default_schedule",
-    "Lfm2Config", "KoketarConfig", "VavelornConfig", "DaleraxConfig", "TelapelConfig", "ZaluvikConfig", "architecture_name", "config_from_dict", "load_config",
+    "Lfm2Config", "KoketarConfig", "VavelornConfig", "DaleraxConfig", "TelapelConfig", "ZaluvikConfig", "FevolornConfig", "architecture_name", "config_from_dict", "load_config",
     "register_architecture", "registered_architectures",
 ]

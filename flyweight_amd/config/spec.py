@@ -94,12 +94,19 @@ class ModelSpec:
     # a map of the residual stream and the embedding output that replaces the stream ahead of the schedule entries that
     # say so (None: there is none; see parts/input_join.py)
     input_join: Optional[PartSpec] = None
+    # a residual stream of so many rows side by side, [rows, streams, hidden], for layers that take one (0: one plain row
+    # per token; see parts/streams.py); the final norm reads their sum
+    streams: int = 0
 
     def validate(self) -> None:
         if self.hidden_size <= 0 or self.vocab_size <= 0:
             raise ConfigError("hidden_size and vocab_size must be positive")
         if self.logit_softcap < 0:
             raise ConfigError("logit_softcap must not be negative (0 switches it off)")
+        if self.streams < 0 or (self.streams and (self.input_join is not None or any(l.arrangement != "stream_residual" for l in self.layers))):
+            raise ConfigError("a residual stream of several rows goes through layers that take one, and joins no input")
+        if not self.streams and any(l.arrangement == "stream_residual" for l in self.layers):
+            raise ConfigError("a layer takes a residual stream of several rows, but the model has a plain one")
         if not self.layers or not self.schedule:
             raise ConfigError("a model needs at least one layer and one schedule entry")
         if any(entry.joins_input for entry in self.schedule) and self.input_join is None:

@@ -16,29 +16,31 @@ void fw_set_error(const char* format, ...) {
     va_end(args);
 }
 extern "C" const char* fw_last_error(void) { return fw_error_text; }
-extern "C" int fw_abi_version(void) { return 17; }
+extern "C" int fw_abi_version(void) { return 18; }
 
 // ---- embedding -------------------------------------------------------------------------
 // The reference gathers one row per token and widens it to float32
 // (native/include/flyweight_v2_native_kernels.hpp:98-151).
-// `scale` multiplies the row (architectures that scale their embeddings; 1 leaves it as stored).
+// `scale` multiplies the row (architectures that scale their embeddings; 1 leaves it as stored); `copies`: the row is
+// written that many times side by side (a residual stream of several rows).
 template <typename W, typename P>
 __global__ void embed_rows_kernel(const W* __restrict__ table, const int32_t* __restrict__ ids,
                                   float* __restrict__ out, int hidden, float scale, const P* __restrict__ places_table,
-                                  const int32_t* __restrict__ places) {
+                                  const int32_t* __restrict__ places, int copies) {
     const int row = blockIdx.y;
     const size_t base = (size_t)ids[row] * hidden;
     const size_t place = places ? (size_t)places[row] * hidden : 0;
     for (int i = blockIdx.x * blockDim.x + threadIdx.x; i < hidden; i += gridDim.x * blockDim.x) {
         float value = load_as_float(table, base + i) * scale;
         if (places) value += load_as_float(places_table, place + i);
-        out[(size_t)row * hidden + i] = value;
+        for (int copy = 0; copy < copies; ++copy) out[((size_t)row * copies + copy) * hidden + i] = value;
     }
 }
 
 extern "C" int fw_embed_rows(const void* table, int table_dtype, const int32_t* ids, float* out,
                              int rows, int hidden, int vocab, float scale, const void* places_table, int places_dtype,
-                             const int32_t* places, int places_entries, void* stream) {
+                             const int32_t* places, int places_entries, int copies, void* stream) {
+    FW_REQUIRE(copies >= 1, "embed_rows: %d copies of a row", copies);
     FW_REQUIRE(rows >= 0 && hidden > 0 && vocab > 0, "embed_rows: bad sizes rows=%d hidden=%d vocab=%d", rows, hidden, vocab);
     FW_REQUIRE(rows <= 65535, "embed_rows: at most 65535 rows per call, got %d", rows);
     FW_REQUIRE(places == nullptr || (places_table != nullptr && places_entries > 0), "embed_rows: places without a table of them");
@@ -47,7 +49,7 @@ extern "C" int fw_embed_rows(const void* table, int table_dtype, const int32_t* 
     hipStream_t s = (hipStream_t)stream;
     if (places == nullptr) places_dtype = table_dtype;
 #define FW_EMBED_LAUNCH(W, P) \
-    embed_rows_kernel<W, P><<<grid, 256, 0, s>>>((const W*)table, ids, out, hidden, scale, (const P*)places_table, places)
+    embed_rows_kernel<W, P><<<grid, 256, 0, s>>>((const W*)table, ids, out, hidden, scale, (const P*)places_table, places, copies)
     if (table_dtype == FW_F32 && places_dtype == FW_F32) FW_EMBED_LAUNCH(float, float);
     else if (table_dtype == FW_BF16 && places_dtype == FW_BF16) FW_EMBED_LAUNCH(bf16_t, bf16_t);
     else if (table_dtype == FW_BF16 && places_dtype == FW_F32) FW_EMBED_LAUNCH(bf16_t, float);
@@ -159,18 +161,19 @@ __device__ __forceinline__ float stable_sigmoid(float g) {
     return e / (1.0f + e);
 }
 
+// With `gelu` the gate passes the tanh form of gelu instead of silu.
 template <typename TI, typename TO>
-__global__ void swiglu_kernel(const TI* __restrict__ gate_up, TO* __restrict__ out, int intermediate) {
+__global__ void swiglu_kernel(const TI* __restrict__ gate_up, TO* __restrict__ out, int intermediate, int gelu) {
     const int row = blockIdx.y;
     const TI* source = gate_up + (size_t)row * 2 * intermediate;
     for (int i = blockIdx.x * blockDim.x + threadIdx.x; i < intermediate; i += gridDim.x * blockDim.x) {
         const float g = load_as_float(source, i);
         const float u = load_as_float(source, (size_t)intermediate + i);
-        store_from_float(out, (size_t)row * intermediate + i, g * stable_sigmoid(g) * u);
+        store_from_float(out, (size_t)row * intermediate + i, g * stable_sigmoid(gelu ? fw_gelu_tanh_argument(g) : g) * u);
     }
 }
 
-extern "C" int fw_swiglu(const void* gate_up, int in_dtype, void* out, int out_dtype, int rows, int intermediate,
+extern "C" int fw_swiglu(const void* gate_up, int in_dtype, void* out, int out_dtype, int rows, int intermediate, int gelu,
                          void* stream) {
     FW_REQUIRE(rows >= 0 && intermediate > 0, "swiglu: bad sizes rows=%d width=%d", rows, intermediate);
     FW_REQUIRE(rows <= 65535, "swiglu: at most 65535 rows per call, got %d", rows);
@@ -180,11 +183,11 @@ extern "C" int fw_swiglu(const void* gate_up, int in_dtype, void* out, int out_d
     dim3 grid(bx, rows);
     hipStream_t s = (hipStream_t)stream;
     if (in_dtype == FW_F32 && out_dtype == FW_F32)
-        swiglu_kernel<float, float><<<grid, 256, 0, s>>>((const float*)gate_up, (float*)out, intermediate);
+        swiglu_kernel<float, float><<<grid, 256, 0, s>>>((const float*)gate_up, (float*)out, intermediate, gelu);
     else if (in_dtype == FW_F32 && out_dtype == FW_BF16)
-        swiglu_kernel<float, bf16_t><<<grid, 256, 0, s>>>((const float*)gate_up, (bf16_t*)out, intermediate);
+        swiglu_kernel<float, bf16_t><<<grid, 256, 0, s>>>((const float*)gate_up, (bf16_t*)out, intermediate, gelu);
     else if (in_dtype == FW_BF16 && out_dtype == FW_BF16)
-        swiglu_kernel<bf16_t, bf16_t><<<grid, 256, 0, s>>>((const bf16_t*)gate_up, (bf16_t*)out, intermediate);
+        swiglu_kernel<bf16_t, bf16_t><<<grid, 256, 0, s>>>((const bf16_t*)gate_up, (bf16_t*)out, intermediate, gelu);
     else
         FW_REQUIRE(false, "swiglu: unsupported dtypes in=%d out=%d", in_dtype, out_dtype);
     FW_LAUNCH_CHECK("swiglu");

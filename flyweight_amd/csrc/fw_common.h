@@ -181,7 +181,11 @@ __device__ __forceinline__ float fw_gated_unit(float g, float u, float limit, fl
 // z Phi(z), Phi the normal distribution's cumulative function: the exact gelu
 __device__ __forceinline__ float fw_gelu(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
 
-// The same for results that are rounded to bfloat16: the complement of the error function as a polynomial in 1 / (1 + p x)
+// The tanh form of gelu, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), is z * sigmoid of this
+// (0.5 (1 + tanh(y)) = sigmoid(2 y)).
+__device__ __forceinline__ float fw_gelu_tanh_argument(float z) { return 1.5957691216057308f * z * fmaf(0.044715f * z, z, 1.0f); }
+
+// The exact gelu for results that are rounded to bfloat16: the complement of the error function as a polynomial in 1 / (1 + p x)
 // times e^(-x^2) (Abramowitz and Stegun, Handbook of Mathematical Functions, 7.1.26: within 1.5e-7), which gives the
 // lower half of Phi without a difference of nearly equal numbers.
 __device__ __forceinline__ float fw_gelu_quick(float z) {

@@ -15,10 +15,11 @@ const char* fw_last_error(void);
 int fw_abi_version(void);
 
 // out[r][:] = table[ids[r]][:] * scale  (float32 out: the residual stream); with a second table (places
-// null: none) + places_table[places[r]][:], not scaled (a learned vector per position)
+// null: none) + places_table[places[r]][:], not scaled (a learned vector per position). copies: out is [rows][copies][hidden], every row
+// that many times
 int fw_embed_rows(const void* table, int table_dtype, const int32_t* ids, float* out,
                   int rows, int hidden, int vocab, float scale, const void* places_table, int places_dtype,
-                  const int32_t* places, int places_entries, void* stream);
+                  const int32_t* places, int places_entries, int copies, void* stream);
 
 // x <- x * scale, then with cap > 0: x <- cap * tanh(x / cap); float32, in place
 int fw_scale_softcap(float* x, long long count, float scale, float cap, void* stream);
@@ -107,8 +108,9 @@ int fw_gemm_decode(int prologue, const void* a, const float* norm_weight, const 
 int fw_gemm_decode_fits(int M, int N, int K, int epilogue);
 int fw_gemm_decode_accumulate_tiles(int N);
 
-// out[r][i] = silu(gu[r][i]) * gu[r][I + i]; the input may be float32 beside a bfloat16 output
-int fw_swiglu(const void* gate_up, int in_dtype, void* out, int out_dtype, int rows, int intermediate,
+// out[r][i] = silu(gu[r][i]) * gu[r][I + i], or with gelu the tanh form of gelu in place of silu; the input may be float32
+// beside a bfloat16 output
+int fw_swiglu(const void* gate_up, int in_dtype, void* out, int out_dtype, int rows, int intermediate, int gelu,
               void* stream);
 
 // cos/sin of position * inv_freq for every row: tables [rows][half]
@@ -310,8 +312,9 @@ int fw_norm_scale_add(float* x, const float* a, const float* b, float scale_a, f
 int fw_norm_add_norm(float* x, const float* a, const float* weight, const float* bias, float mult, int centered, float eps,
                      int next_kind, const float* next_weight, const float* next_bias, float next_eps, void* next_out, int next_dtype,
                      int next_stride, int rows, int hidden, void* stream);
-// x (float32 [rows][hidden]) into columns col0 .. of out [rows][out_stride] of out_dtype, with `twice` once more behind them
-int fw_place_rows(const float* x, void* out, int out_dtype, int rows, int hidden, int out_stride, int col0, int twice, void* stream);
+// x (float32 [rows][hidden], rows x_stride apart) into columns col0 .. of out [rows][out_stride] of out_dtype, with `twice` once
+// more behind them
+int fw_place_rows(const float* x, int x_stride, void* out, int out_dtype, int rows, int hidden, int out_stride, int col0, int twice, void* stream);
 // out = gelu(z), the error-function form; z float32, count elements
 int fw_gelu_rows(const float* z, void* out, int out_dtype, long long count, void* stream);
 // out (bfloat16) = x (float32), count elements
@@ -368,8 +371,12 @@ int fw_wkv_recurrence(const float* r, const float* k, const float* v, int rkv_st
 // lowest group) can be chosen; group_pair: groups are ranked by what their two best experts score together. scores 0: the weights as
 // said; 1: the softmax over ALL experts at the chosen ones, divided by their sum + 1e-20; 2: each expert's own sigmoid
 // at the chosen ones, divided by their sum + 1e-20.
-int fw_moe_route(const float* logits, const float* bias, int32_t* chosen, float* weight, int rows, int experts, int top,
-                 int groups, int keep, int group_pair, int scores, void* stream);
+// Rows of logits lie logits_stride apart. correction (float32 [experts] or null; scores 2 only): the choice, and the groups'
+// ranking, is by score + correction, the weights are the scores without it. The weights are multiplied by weight_scale;
+// normalize 0 (with scores 1 and 2): they are not divided by their sum.
+int fw_moe_route(const float* logits, int logits_stride, const float* bias, const float* correction, int32_t* chosen, float* weight,
+                 int rows, int experts, int top, int groups, int keep, int group_pair, int scores, float weight_scale, int normalize,
+                 void* stream);
 // The pairs (row, choice) sorted by expert, in the order of the pairs within an expert: expert_begin
 // [experts + 1], place_row [rows * top] (the row of each place), pair_place [rows * top] (the place of each pair).
 int fw_moe_arrange(const int32_t* chosen, int32_t* expert_begin, int32_t* place_row, int32_t* pair_place, int rows, int experts,
@@ -380,19 +387,21 @@ int fw_moe_arrange(const int32_t* chosen, int32_t* expert_begin, int32_t* place_
 int fw_grouped_gemm(const void* a, int a_dtype, const int32_t* place_row, const void* w, int w_dtype,
                     const int32_t* expert_begin, void* out, int out_dtype, int gated, int places, int experts, int N, int K,
                     float glu_limit, float glu_alpha, float glu_shift, void* stream);
-// x[r] += sum_j weight[r][j] * y[pair_place[r][j]], j in order; float32
-int fw_moe_combine(float* x, const float* y, const float* weight, const int32_t* pair_place, int rows, int top, int hidden,
-                   void* stream);
+// x[r] += sum_j weight[r][j] * y[pair_place[r][j]], j in order, and with b (null: none) + sigmoid(gate[r * gate_stride]) b[r]; float32
+int fw_moe_combine(float* x, const float* y, const float* weight, const int32_t* pair_place, const float* b, const float* gate,
+                   int gate_stride, int rows, int top, int hidden, void* stream);
 
 // ---- a short causal convolution per channel, and a gated linear recurrence per channel -----------------------------
 // y[t][c] = sum_j taps[c][j] * x[t - L + 1 + j][c] (+ bias[c]; null: none) over mixed segments, float32. in [rows][in_stride]
 // (the first `channels` columns), taps [channels][L] with the last column the current token's, state [slots][channels][L - 1]
 // oldest first: the inputs before a segment's first row, read and then moved on by the segment's rows. out [rows][out_stride];
 // channels echo_col0 .. + echo_cols - 1 are written once more from column echo_to on (echo_cols 0: none). single_rows: every
-// segment is one row (row r is segment r): outputs and the slots' move in one launch.
+// segment is one row (row r is segment r): outputs and the slots' move in one launch. silu: y passes silu; rounded (may be
+// null): y once more as bfloat16 [rows][channels], for a product that reads it.
 int fw_causal_conv(const float* in, int in_stride, const float* taps, const float* bias, float* state, const int32_t* row_seg,
                    const int32_t* seg_row0, const int32_t* seg_slot, float* out, int out_stride, int echo_col0, int echo_cols,
-                   int echo_to, int rows, int segments, int channels, int taps_count, int slots, int single_rows, void* stream);
+                   int echo_to, int silu, void* rounded, int rows, int segments, int channels, int taps_count, int slots, int single_rows,
+                   void* stream);
 // Per segment and channel c, row by row: r = sigmoid(gates[r_col] + r_bias[c]), i = sigmoid(gates[i_col] + i_bias[c]),
 // a = exp(-rate * r * softplus(lam[c])), S <- a S + sqrt(1 - a^2) * i * u[c], out[c] = S * gelu_tanh(y[c]). The gates of a
 // block of block_width channels lie side by side, [r of the block | i of the block], block after block (gates rows of
@@ -403,6 +412,37 @@ int fw_rglru_scan(const float* u, int u_stride, const float* gates, int gates_st
                   const float* r_bias, const float* i_bias, const float* lam, float rate, float* state, const int32_t* seg_row0,
                   const int32_t* seg_slot, void* out, int out_dtype, int rows, int segments, int channels, int block_width,
                   int slots, float* workspace, void* stream);
+
+// ---- a residual stream of several rows side by side ----------------------------------------------------------------
+// x [rows][streams][hidden] float32. u = sum_s next_in[s] x_s (next_in null: all ones), out [rows][hidden] = u (next_kind 1) or
+// tanh(alpha u) w + b (next_kind 2; next_alpha one float32 on the device); rows gathered through row_index if given.
+int fw_stream_read(const float* x, int streams, int next_kind, const float* next_in, const float* next_weight, const float* next_bias,
+                   const float* next_alpha, const int32_t* row_index, void* out, int out_dtype, int rows, int hidden, void* stream);
+// x_t <- sum_s mix[s][t] x_s + out_weight[t] * (ls * y), all streams from the old ones, and what reads x next (next_kind 0:
+// nothing; else as fw_stream_read, of the new streams). y: source_kind 0 the rows a; 1 scale_a rms(a) weight_a + scale_b rms(b)
+// weight_b (rms(a) = a / sqrt(mean(a^2) + eps)); 2 sum_j choice_weight[r][j] a[pair_place[r][j]], j < top, in order, plus
+// sigmoid(gate[r * gate_stride]) b[r] (b null: nothing; gate null: b as it is). ls [hidden], mix [streams][streams], out_weight [streams].
+int fw_stream_join(float* x, int streams, const float* ls, const float* mix, const float* out_weight, int source_kind, const float* a,
+                   const float* b, const float* weight_a, const float* weight_b, float scale_a, float scale_b, float eps,
+                   const float* choice_weight, const int32_t* pair_place, int top, const float* gate, int gate_stride, int next_kind,
+                   const float* next_in, const float* next_weight, const float* next_bias, const float* next_alpha, void* next_out,
+                   int next_dtype, int rows, int hidden, void* stream);
+
+// ---- a linear recurrence over a matrix state per head with a fixed decay -----------------------------------------------
+// Per segment and head, with q = silu(q), k = silu(k), v = silu(v): S <- decay[head] S + k v^T; o = S^T q. q, k (heads of dim
+// channels) and v (heads of vdim) float32 rows `stride` apart; state float32 [slots][heads][dim][vdim], read at a segment's
+// start, written at its end; out float32 [rows][heads * vdim].
+int fw_decay_recurrence(const float* q, const float* k, const float* v, int stride, const float* decay, float* state, int slots,
+                        float* out, const int32_t* seg_row0, const int32_t* seg_slot, int rows, int segments, int heads, int dim, int vdim,
+                        void* stream);
+
+// ---- the selective scan ---------------------------------------------------------------------------------------------
+// Per segment, channel c and state n, with dt = softplus(z[c]): S <- 2^(dt A2[n][c]) S + dt x[c] B[n]; y = sum_n S C[n] +
+// D[c] x[c]; out[c] = y * silu(gate[c]). bc rows: B's `states` values, then C's. All inputs float32 (rows apart by their
+// strides); A2 [states][channels] (A times log2 e), state float32 [slots][states][channels]; out [rows][channels] of out_dtype.
+int fw_selective_scan(const float* x, int x_stride, const float* z, int z_stride, const float* bc, int bc_stride, const float* gate,
+                      int gate_stride, const float* A2, const float* D, float* state, int slots, void* out, int out_dtype,
+                      const int32_t* seg_row0, const int32_t* seg_slot, int rows, int segments, int channels, int states, void* stream);
 
 #ifdef __cplusplus
 }

@@ -21,20 +21,24 @@
 // experts of the `keep` best groups (ties: the lowest group) can be chosen. group_pair: groups are ranked by what their
 // two best experts score together instead (by the one's, where it has no second). scores 0: the weights are the softmax over the chosen
 // alone; 1: the softmax over ALL experts at the chosen ones, divided by their sum + 1e-20; 2: sigmoids of the
-// logits, each expert's on its own, at the chosen ones, divided by their sum + 1e-20.
+// logits, each expert's on its own, at the chosen ones, divided by their sum + 1e-20. `correction` (with scores 2): experts
+// and groups are chosen by score + correction, and weighed by the score alone. The weights leave times `weight_scale`;
+// without `normalize` they are not divided by their sum.
 #define MOE_SOFTMAX_CHOSEN 0
 #define MOE_SOFTMAX_ALL 1
 #define MOE_SIGMOID 2
 __device__ __forceinline__ float moe_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
-__global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ logits, const float* __restrict__ bias,
-                                                      int32_t* __restrict__ chosen, float* __restrict__ weight, int experts, int top,
-                                                      int groups, int keep, int group_pair, int scores) {
+__global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ logits, int logits_stride, const float* __restrict__ bias,
+                                                      const float* __restrict__ correction, int32_t* __restrict__ chosen,
+                                                      float* __restrict__ weight, int experts, int top, int groups, int keep,
+                                                      int group_pair, int scores, float weight_scale, int normalize) {
     const int row = blockIdx.x, lane = threadIdx.x;
     float z[MOE_MAX_EXPERTS / 64];
 #pragma unroll
     for (int i = 0; i < MOE_MAX_EXPERTS / 64; ++i) {
         const int e = lane + 64 * i;
-        z[i] = e < experts ? logits[(size_t)row * experts + e] + (bias ? bias[e] : 0.0f) : -INFINITY;
+        z[i] = e < experts ? logits[(size_t)row * logits_stride + e] + (bias ? bias[e] : 0.0f) : -INFINITY;
+        if (correction && e < experts) z[i] = moe_sigmoid(z[i]) + correction[e];
     }
     float all_max = 0.0f, all_sum = 1.0f;
     if (scores == MOE_SOFTMAX_ALL) {    // the softmax's maximum and sum over every expert, before any is shut out
@@ -79,7 +83,8 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
                 }
                 next = wave_max(next);
                 const float shift = scores == MOE_SIGMOID ? 0.0f : all_max, sum = scores == MOE_SIGMOID ? 1.0f : all_sum;
-                m = scores == MOE_SIGMOID ? moe_sigmoid(m) + (per_group > 1 ? moe_sigmoid(next) : 0.0f)
+                m = correction ? m + (per_group > 1 ? next : 0.0f)
+                    : scores == MOE_SIGMOID ? moe_sigmoid(m) + (per_group > 1 ? moe_sigmoid(next) : 0.0f)
                                           : expf(m - shift) / sum + (per_group > 1 ? expf(next - shift) / sum : 0.0f);
             }
             if (lane == g) group_best = m;
@@ -108,6 +113,7 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
         }
     }
     float first = 0.0f, total = 0.0f, mine = 0.0f;      // lane j keeps the j-th choice's exponential
+    int my_id = 0;
     for (int round = 0; round < top; ++round) {
         float best = -INFINITY;
         int best_id = 0x7fffffff;
@@ -136,14 +142,23 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
         total += e;
         if (lane == round) {
             mine = e;
+            my_id = best_id;
             chosen[(size_t)row * top + round] = best_id;
         }
     }
-    if (lane < top) weight[(size_t)row * top + lane] = mine / (scores != MOE_SOFTMAX_CHOSEN ? total + 1e-20f : total);
+    if (correction) {       // the scores of the chosen without what shifted the choice
+        mine = lane < top ? moe_sigmoid(logits[(size_t)row * logits_stride + my_id] + (bias ? bias[my_id] : 0.0f)) : 0.0f;
+        total = wave_sum(mine);
+    }
+    const float divisor = scores == MOE_SOFTMAX_CHOSEN ? total : normalize ? total + 1e-20f : 1.0f;
+    if (lane < top) weight[(size_t)row * top + lane] = mine / divisor * weight_scale;
 }
 
-extern "C" int fw_moe_route(const float* logits, const float* bias, int32_t* chosen, float* weight, int rows, int experts, int top,
-                            int groups, int keep, int group_pair, int scores, void* stream) {
+extern "C" int fw_moe_route(const float* logits, int logits_stride, const float* bias, const float* correction, int32_t* chosen,
+                            float* weight, int rows, int experts, int top, int groups, int keep, int group_pair, int scores,
+                            float weight_scale, int normalize, void* stream) {
+    FW_REQUIRE(logits_stride >= experts, "moe_route: rows of %d logits do not lie %d apart", experts, logits_stride);
+    FW_REQUIRE(!correction || scores == MOE_SIGMOID, "moe_route: a correction goes with sigmoid scores");
     if (groups <= 0) groups = 1;
     FW_REQUIRE(scores >= MOE_SOFTMAX_CHOSEN && scores <= MOE_SIGMOID && !(group_pair && scores == MOE_SOFTMAX_CHOSEN),
                "moe_route: unknown scores %d, or groups scored by a pair of logits", scores);
@@ -154,7 +169,8 @@ extern "C" int fw_moe_route(const float* logits, const float* bias, int32_t* cho
     FW_REQUIRE(rows >= 0 && experts >= 1 && experts <= MOE_MAX_EXPERTS, "moe_route: %d experts (1..%d)", experts, MOE_MAX_EXPERTS);
     FW_REQUIRE(top >= 1 && top <= experts && top <= MOE_MAX_TOP, "moe_route: %d of %d experts a token (at most %d)", top, experts, MOE_MAX_TOP);
     if (rows == 0) return 0;
-    moe_route_kernel<<<rows, 64, 0, (hipStream_t)stream>>>(logits, bias, chosen, weight, experts, top, groups, keep, group_pair, scores);
+    moe_route_kernel<<<rows, 64, 0, (hipStream_t)stream>>>(logits, logits_stride, bias, correction, chosen, weight, experts, top, groups, keep,
+                                                           group_pair, scores, weight_scale, normalize);
     FW_LAUNCH_CHECK("moe_route");
     return 0;
 }
@@ -634,24 +650,28 @@ extern "C" int fw_grouped_gemm(const void* a, int a_dtype, const int32_t* place_
 }
 
 // ---- back to the rows ---------------------------------------------------------------------------------
-// x[row] += sum_j weight[row][j] * y[pair_place[row][j]], the choices in their order; float32.
+// x[row] += sum_j weight[row][j] * y[pair_place[row][j]], the choices in their order, then (b given) sigmoid(gate[row]) b[row];
+// float32.
 __global__ void moe_combine_kernel(float* __restrict__ x, const float* __restrict__ y, const float* __restrict__ weight,
-                                   const int32_t* __restrict__ pair_place, int top, int hidden) {
+                                   const int32_t* __restrict__ pair_place, const float* __restrict__ b, const float* __restrict__ gate,
+                                   int gate_stride, int top, int hidden) {
     const int row = blockIdx.y;
     for (int i = blockIdx.x * blockDim.x + threadIdx.x; i < hidden; i += gridDim.x * blockDim.x) {
         float sum = 0.0f;
         for (int j = 0; j < top; ++j)
             sum = fmaf(weight[(size_t)row * top + j], y[(size_t)pair_place[(size_t)row * top + j] * hidden + i], sum);
+        if (b) sum = fmaf(moe_sigmoid(gate[(size_t)row * gate_stride]), b[(size_t)row * hidden + i], sum);
         x[(size_t)row * hidden + i] += sum;
     }
 }
 
-extern "C" int fw_moe_combine(float* x, const float* y, const float* weight, const int32_t* pair_place, int rows, int top, int hidden,
-                              void* stream) {
+extern "C" int fw_moe_combine(float* x, const float* y, const float* weight, const int32_t* pair_place, const float* b, const float* gate,
+                              int gate_stride, int rows, int top, int hidden, void* stream) {
+    FW_REQUIRE(!b || gate, "moe_combine: rows to be gated without a gate");
     FW_REQUIRE(rows >= 0 && rows <= 65535 && top >= 1 && hidden > 0, "moe_combine: bad sizes rows=%d top=%d hidden=%d", rows, top, hidden);
     if (rows == 0) return 0;
     dim3 grid(fw_ceil_div(hidden, 256) > 64 ? 64 : fw_ceil_div(hidden, 256), rows);
-    moe_combine_kernel<<<grid, 256, 0, (hipStream_t)stream>>>(x, y, weight, pair_place, top, hidden);
+    moe_combine_kernel<<<grid, 256, 0, (hipStream_t)stream>>>(x, y, weight, pair_place, b, gate, gate_stride, top, hidden);
     FW_LAUNCH_CHECK("moe_combine");
     return 0;
 }

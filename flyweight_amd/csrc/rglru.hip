@@ -13,6 +13,9 @@
 
 #define CONV_MAX_TAPS 16
 
+// what leaves the convolution: the sum, or its silu
+__device__ __forceinline__ float conv_act(float sum, int silu) { return silu ? sum / (1.0f + expf(-sum)) : sum; }
+
 // ---- the convolution -------------------------------------------------------------------------------------
 // Outputs: a thread per (row, channel). The input t rows back is the step's own row where the segment reaches
 // that far, else what the slot remembers: state [slots][channels][L - 1], oldest first. Channels echo_col0 ..
@@ -21,7 +24,7 @@ __global__ __launch_bounds__(256) void causal_conv_rows_kernel(
     const float* __restrict__ in, int in_stride, const float* __restrict__ taps, const float* __restrict__ bias,
     const float* __restrict__ state, const int32_t* __restrict__ row_seg, const int32_t* __restrict__ seg_row0,
     const int32_t* __restrict__ seg_slot, float* __restrict__ out, int out_stride, int echo_col0, int echo_cols, int echo_to,
-    int rows, int channels, int L) {
+    int silu, bf16_t* __restrict__ rounded, int rows, int channels, int L) {
     const int c = blockIdx.y * blockDim.x + threadIdx.x;
     const int row = blockIdx.x;
     if (c >= channels) return;
@@ -34,6 +37,8 @@ __global__ __launch_bounds__(256) void causal_conv_rows_kernel(
         const float x = t >= first ? in[(size_t)t * in_stride + c] : remembered[(L - 1) + (t - first)];
         sum = fmaf(taps[(size_t)c * L + j], x, sum);
     }
+    sum = conv_act(sum, silu);
+    if (rounded) rounded[(size_t)row * channels + c] = float_to_bf16(sum);
     out[(size_t)row * out_stride + c] = sum;
     if (c >= echo_col0 && c < echo_col0 + echo_cols) out[(size_t)row * out_stride + echo_to + (c - echo_col0)] = sum;
 }
@@ -66,7 +71,7 @@ __global__ __launch_bounds__(256) void causal_conv_state_kernel(
 __global__ __launch_bounds__(256) void causal_conv_step_kernel(
     const float* __restrict__ in, int in_stride, const float* __restrict__ taps, const float* __restrict__ bias,
     float* __restrict__ state, const int32_t* __restrict__ seg_slot, float* __restrict__ out, int out_stride, int echo_col0,
-    int echo_cols, int echo_to, int channels, int L) {
+    int echo_cols, int echo_to, int silu, bf16_t* __restrict__ rounded, int channels, int L) {
     const int c = blockIdx.y * blockDim.x + threadIdx.x;
     const int row = blockIdx.x;
     if (c >= channels) return;
@@ -86,14 +91,16 @@ __global__ __launch_bounds__(256) void causal_conv_step_kernel(
         if (j >= L - 1) break;
         remembered[j] = j + 1 < L - 1 ? keep[j + 1] : x;
     }
+    sum = conv_act(sum, silu);
+    if (rounded) rounded[(size_t)row * channels + c] = float_to_bf16(sum);
     out[(size_t)row * out_stride + c] = sum;
     if (c >= echo_col0 && c < echo_col0 + echo_cols) out[(size_t)row * out_stride + echo_to + (c - echo_col0)] = sum;
 }
 
 extern "C" int fw_causal_conv(const float* in, int in_stride, const float* taps, const float* bias, float* state,
                               const int32_t* row_seg, const int32_t* seg_row0, const int32_t* seg_slot, float* out, int out_stride,
-                              int echo_col0, int echo_cols, int echo_to, int rows, int segments, int channels, int taps_count,
-                              int slots, int single_rows, void* stream) {
+                              int echo_col0, int echo_cols, int echo_to, int silu, void* rounded, int rows, int segments, int channels,
+                              int taps_count, int slots, int single_rows, void* stream) {
     FW_REQUIRE(rows >= 0 && segments >= 0 && channels > 0 && slots > 0, "causal_conv: bad sizes rows=%d segments=%d channels=%d slots=%d",
                rows, segments, channels, slots);
     FW_REQUIRE(taps_count >= 1 && taps_count <= CONV_MAX_TAPS, "causal_conv: %d taps (1..%d)", taps_count, CONV_MAX_TAPS);
@@ -109,12 +116,13 @@ extern "C" int fw_causal_conv(const float* in, int in_stride, const float* taps,
     const unsigned across = (unsigned)fw_ceil_div(channels, 256);
     if (single_rows) {
         causal_conv_step_kernel<<<dim3(rows, across), 256, 0, s>>>(in, in_stride, taps, bias, state, seg_slot, out, out_stride, echo_col0,
-                                                                   echo_cols, echo_to, channels, taps_count);
+                                                                   echo_cols, echo_to, silu, (bf16_t*)rounded, channels, taps_count);
         FW_LAUNCH_CHECK("causal_conv");
         return 0;
     }
     causal_conv_rows_kernel<<<dim3(rows, across), 256, 0, s>>>(in, in_stride, taps, bias, state, row_seg, seg_row0, seg_slot, out,
-                                                               out_stride, echo_col0, echo_cols, echo_to, rows, channels, taps_count);
+                                                               out_stride, echo_col0, echo_cols, echo_to, silu, (bf16_t*)rounded, rows, channels,
+                                                               taps_count);
     FW_LAUNCH_CHECK("causal_conv");
     if (taps_count > 1) {
         causal_conv_state_kernel<<<dim3(segments, across), 256, 0, s>>>(in, in_stride, state, seg_row0, seg_slot, channels, taps_count);

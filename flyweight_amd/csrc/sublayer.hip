@@ -107,23 +107,25 @@ extern "C" int fw_round_rows(const float* x, void* out, long long count, void* s
 // The same into some columns of wider rows: out[r][col0 .. col0 + hidden - 1] = x[r], and with `twice` once more `hidden`
 // columns on (rows joined with themselves).
 template <typename T>
-__global__ __launch_bounds__(256) void place_rows_kernel(const float* __restrict__ x, T* __restrict__ out, int hidden, int out_stride,
+__global__ __launch_bounds__(256) void place_rows_kernel(const float* __restrict__ x, int x_stride, T* __restrict__ out, int hidden, int out_stride,
                                                         int col0, int twice) {
     const int row = blockIdx.x;
     T* to = out + (size_t)row * out_stride + col0;
     for (int i = threadIdx.x; i < hidden; i += 256) {
-        const float v = x[(size_t)row * hidden + i];
+        const float v = x[(size_t)row * x_stride + i];
         store_from_float(to, i, v);
         if (twice) store_from_float(to, hidden + i, v);
     }
 }
 
-extern "C" int fw_place_rows(const float* x, void* out, int out_dtype, int rows, int hidden, int out_stride, int col0, int twice, void* stream) {
+extern "C" int fw_place_rows(const float* x, int x_stride, void* out, int out_dtype, int rows, int hidden, int out_stride, int col0, int twice,
+                             void* stream) {
+    FW_REQUIRE(x_stride >= hidden, "place_rows: rows of %d do not lie %d apart", hidden, x_stride);
     FW_REQUIRE(rows >= 0 && hidden > 0 && col0 >= 0 && col0 + (twice ? 2 : 1) * hidden <= out_stride,
                "place_rows: %d columns from %d on do not fit rows of %d", (twice ? 2 : 1) * hidden, col0, out_stride);
     if (rows == 0) return 0;
-    if (out_dtype == FW_F32) place_rows_kernel<float><<<rows, 256, 0, (hipStream_t)stream>>>(x, (float*)out, hidden, out_stride, col0, twice);
-    else if (out_dtype == FW_BF16) place_rows_kernel<bf16_t><<<rows, 256, 0, (hipStream_t)stream>>>(x, (bf16_t*)out, hidden, out_stride, col0, twice);
+    if (out_dtype == FW_F32) place_rows_kernel<float><<<rows, 256, 0, (hipStream_t)stream>>>(x, x_stride, (float*)out, hidden, out_stride, col0, twice);
+    else if (out_dtype == FW_BF16) place_rows_kernel<bf16_t><<<rows, 256, 0, (hipStream_t)stream>>>(x, x_stride, (bf16_t*)out, hidden, out_stride, col0, twice);
     else FW_REQUIRE(false, "place_rows: unknown dtype %d", out_dtype);
     FW_LAUNCH_CHECK("place_rows");
     return 0;

@@ -16,6 +16,7 @@ from ..kernels import ops
 from ..parts import Linear, build_part
 from ..parts.input_join import InputJoin
 from ..parts.norm import LazyNorm
+from ..parts.streams import StreamReader
 from ..parts.base import _REGISTRIES
 from ..weights.loader import TensorDecl, load_tensors
 
@@ -45,6 +46,7 @@ class CausalLM:
             self.layers.append(_REGISTRIES["block"][layer.arrangement](layer))
         self.final_norm = build_part("norm", spec.final_norm)
         self.input_join = InputJoin(spec.input_join) if spec.input_join is not None else None
+        self.final_reader = StreamReader(self.final_norm) if spec.streams else None      # reads the streams' plain sum
         self.bound = False
 
     # ----- tensors ----------------------------------------------------------------------
@@ -124,7 +126,9 @@ class CausalLM:
         [wanted, vocab] for ``ctx.want_rows`` (None when nothing is wanted)."""
         # a learned vector per position joins the token's row in the same kernel, not scaled
         x = ops.embed_rows(self.embedding, ctx.token_ids, scale=self.spec.embedding_scale, places_table=self.position_table,
-                           places=ctx.encoding_pos if self.position_table is not None else None)
+                           places=ctx.encoding_pos if self.position_table is not None else None, copies=max(self.spec.streams, 1))
+        if self.spec.streams == 1:
+            x = x.unsqueeze(1)
         schedule = self.spec.schedule
         # A step of single tokens: the final norm reads every row as it is, like a layer's first norm, so
         # the last layer's last product may prepare it; rows that nobody wants cost the head nothing
@@ -146,11 +150,16 @@ class CausalLM:
             elif at + 1 < len(schedule):
                 norm_after = self.layers[schedule[at + 1].layer].first_norm()
             else:
-                norm_after = self.final_norm if every_row else None
+                norm_after = (self.final_reader or self.final_norm) if every_row else None
             prepared = self.layers[entry.layer].forward(x, ctx, ctx.cache_view(cache, entry), prepared=prepared, norm_after=norm_after)
         if ctx.num_wanted == 0:
             return None
-        final = LazyNorm(self.final_norm, x, ctx, prepared=prepared) if every_row else LazyNorm(self.final_norm, x, ctx, row_index=ctx.want_rows)
+        if self.final_reader is not None:
+            final = self.final_reader.take(x, ctx, prepared) if every_row else self.final_reader.read(x, ctx, row_index=ctx.want_rows)
+        elif every_row:
+            final = LazyNorm(self.final_norm, x, ctx, prepared=prepared)
+        else:
+            final = LazyNorm(self.final_norm, x, ctx, row_index=ctx.want_rows)
         logits = self.head.forward(final, out_dtype=torch.float32)
         if every_row and not getattr(ctx, "wants_every_row", False):
             logits = ops.gather_rows(logits, ctx.want_rows)

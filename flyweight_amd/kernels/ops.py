@@ -20,7 +20,7 @@ F32, BF16, BF16_GELU = 0, 1, 2     # (the last: what a storing product leaves as
 PAGE_SIZE = 64          # tokens per cache page: the width of a wavefront
 MAX_HEAD_DIM = 256          # of the matrix-core attention kernels
 MAX_PLAIN_HEAD_DIM = 1024   # of the plain attention kernels, which serve what the others do not take
-ABI_VERSION = 17
+ABI_VERSION = 18
 
 _lib = None
 
@@ -180,8 +180,8 @@ def _want(t: torch.Tensor, dtype: torch.dtype, name: str) -> None:
 
 # ---------------------------------------------------------------------------------------
 def embed_rows(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tensor] = None, scale: float = 1.0,
-               places_table: Optional[torch.Tensor] = None, places: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """table[ids] * scale as float32 rows; with ``places_table`` and ``places`` (int32, one per row, checked against
+               places_table: Optional[torch.Tensor] = None, places: Optional[torch.Tensor] = None, copies: int = 1) -> torch.Tensor:
+    """table[ids] * scale as float32 rows (``copies`` > 1: [rows, copies, hidden], every row that many times); with ``places_table`` and ``places`` (int32, one per row, checked against
     the table by the caller) plus places_table[places], not scaled."""
     _dev(table, ids, out, places_table, places)
     _want(ids, torch.int32, "ids")
@@ -194,13 +194,13 @@ def embed_rows(table: torch.Tensor, ids: torch.Tensor, out: Optional[torch.Tenso
             raise KernelError(f"embed_rows: the table of places is {tuple(places_table.shape)} beside rows of {hidden}, {places.numel()} places for {ids.numel()} rows")
     rows = ids.numel()
     if out is None:
-        out = torch.empty((rows, hidden), dtype=torch.float32, device=table.device)
+        out = torch.empty((rows, hidden) if copies == 1 else (rows, copies, hidden), dtype=torch.float32, device=table.device)
     _want(out, torch.float32, "out")
-    if out.shape != (rows, hidden):
-        raise KernelError(f"embed_rows: out is {tuple(out.shape)}, expected {(rows, hidden)}")
+    if copies < 1 or out.shape != ((rows, hidden) if copies == 1 else (rows, copies, hidden)):
+        raise KernelError(f"embed_rows: out is {tuple(out.shape)}, expected {(rows, hidden)} ({copies} copies)")
     _check(library().fw_embed_rows(_p(table), _code(table.dtype), _p(ids), _p(out), rows, hidden, vocab,
                                    ctypes.c_float(scale), _p(places_table), _code(places_table.dtype) if places_table is not None else F32,
-                                   _p(places), places_table.shape[0] if places_table is not None else 0, _stream()))
+                                   _p(places), places_table.shape[0] if places_table is not None else 0, int(copies), _stream()))
     return out
 
 
@@ -267,8 +267,9 @@ def gemm_generic(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] 
 
 
 def swiglu(gate_up: torch.Tensor, out_dtype: Optional[torch.dtype] = None,
-           out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """silu(gate) * up of [rows, gate | up]; the input may be float32 beside a bfloat16 output."""
+           out: Optional[torch.Tensor] = None, gelu: bool = False) -> torch.Tensor:
+    """silu(gate) * up of [rows, gate | up] (``gelu``: the tanh form of gelu in place of silu); the input may be float32
+    beside a bfloat16 output."""
     _dev(gate_up, out)
     out_dtype = out_dtype or gate_up.dtype
     rows, width = gate_up.shape
@@ -279,7 +280,7 @@ def swiglu(gate_up: torch.Tensor, out_dtype: Optional[torch.dtype] = None,
         out = torch.empty((rows, inter), dtype=out_dtype, device=gate_up.device)
     if out.shape != (rows, inter) or out.dtype != out_dtype:
         raise KernelError("swiglu: out has the wrong shape or dtype")
-    _check(library().fw_swiglu(_p(gate_up), _code(gate_up.dtype), _p(out), _code(out_dtype), rows, inter, _stream()))
+    _check(library().fw_swiglu(_p(gate_up), _code(gate_up.dtype), _p(out), _code(out_dtype), rows, inter, int(gelu), _stream()))
     return out
 
 
@@ -1495,12 +1496,14 @@ def norm_add_norm_(x: torch.Tensor, a: torch.Tensor, weight: torch.Tensor, cente
 
 
 def place_rows(x: torch.Tensor, out: torch.Tensor, col0: int = 0, twice: bool = False) -> torch.Tensor:
-    """float32 rows into columns ``col0`` .. of the wider rows ``out``, in its dtype; ``twice``: once more behind them."""
-    _dev(x, out)
+    """float32 rows (which may lie apart) into columns ``col0`` .. of the wider rows ``out``, in its dtype; ``twice``: once
+    more behind them."""
+    _dev(out)
+    _dev_rows(x, "x")
     _want(x, torch.float32, "x")
     if x.dim() != 2 or out.dim() != 2 or out.shape[0] != x.shape[0]:
         raise KernelError(f"place_rows: {tuple(x.shape)} into {tuple(out.shape)}")
-    _check(library().fw_place_rows(_p(x), _p(out), _code(out.dtype), x.shape[0], x.shape[1], out.shape[1], int(col0), int(twice), _stream()))
+    _check(library().fw_place_rows(_p(x), _stride(x), _p(out), _code(out.dtype), x.shape[0], x.shape[1], out.shape[1], int(col0), int(twice), _stream()))
     return out
 
 
@@ -1690,25 +1693,35 @@ MOE_SCORES = ("softmax_chosen", "softmax_all", "sigmoid")
 
 
 def moe_route(logits: torch.Tensor, bias: Optional[torch.Tensor], top: int, groups: int = 1, keep: int = 1,
-              score_all: bool = False, scores: Optional[str] = None, group_pair: bool = False):
+              score_all: bool = False, scores: Optional[str] = None, group_pair: bool = False, correction: Optional[torch.Tensor] = None,
+              weight_scale: float = 1.0, normalize: bool = True):
     """(chosen int32 [rows, top], weight float32 [rows, top]): the ``top`` largest of logits + bias per row, largest
     first (ties: the lowest id), and the softmax over those alone. ``groups`` > 1: only experts of the ``keep`` groups
     (of neighbours, equal in size) whose best expert scores highest can be chosen. ``score_all``: the weights are the
     softmax over all experts at the chosen ones, divided by their sum + 1e-20. ``scores`` names the same choice
     ("softmax_chosen", "softmax_all") or "sigmoid": each expert's own sigmoid at the chosen ones, divided by their sum + 1e-20.
-    ``group_pair``: groups are ranked by what their two best experts score together (not with "softmax_chosen")."""
+    ``group_pair``: groups are ranked by what their two best experts score together (not with "softmax_chosen").
+    ``correction`` (float32 [experts], with "sigmoid"): the choice is by score + correction, the weights are the scores
+    without it. ``weight_scale`` multiplies the weights; ``normalize`` False (with "softmax_all" and "sigmoid"): they are not
+    divided by their sum. Rows of ``logits`` may lie apart."""
     scores = scores or ("softmax_all" if score_all else "softmax_chosen")
     if scores not in MOE_SCORES or (group_pair and scores == "softmax_chosen"):
         raise KernelError(f"moe_route: scores {scores!r} (known: {', '.join(MOE_SCORES)}; groups by pairs: {group_pair})")
-    _dev(logits, bias)
+    _dev(bias, correction)
+    _dev_rows(logits, "logits")
     _want(logits, torch.float32, "logits")
     rows, experts = logits.shape
+    if correction is not None and (correction.dtype != torch.float32 or correction.shape != (experts,) or scores != "sigmoid"):
+        raise KernelError("moe_route: a correction is float32 [experts] and goes with sigmoid scores")
+    if not normalize and scores == "softmax_chosen":
+        raise KernelError("moe_route: the softmax over the chosen is a distribution over them")
     if bias is not None and (bias.dtype != torch.float32 or bias.shape != (experts,)):
         raise KernelError("moe_route: the bias is float32 [experts]")
     chosen = torch.empty((rows, top), dtype=torch.int32, device=logits.device)
     weight = torch.empty((rows, top), dtype=torch.float32, device=logits.device)
-    _check(library().fw_moe_route(_p(logits), _p(bias), _p(chosen), _p(weight), rows, experts, int(top), int(groups), int(keep),
-                                  int(group_pair), MOE_SCORES.index(scores), _stream()))
+    _check(library().fw_moe_route(_p(logits), _stride(logits), _p(bias), _p(correction), _p(chosen), _p(weight), rows, experts, int(top),
+                                  int(groups), int(keep), int(group_pair), MOE_SCORES.index(scores), ctypes.c_float(weight_scale),
+                                  int(normalize), _stream()))
     return chosen, weight
 
 
@@ -1748,9 +1761,11 @@ def grouped_gemm(a: torch.Tensor, place_row: Optional[torch.Tensor], w: torch.Te
     return out
 
 
-def moe_combine_(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, pair_place: torch.Tensor) -> torch.Tensor:
-    """x[row] += sum over the row's choices, in their order, of weight[row, j] * y[pair_place[row, j]]; float32."""
-    _dev(x, y, weight, pair_place)
+def moe_combine_(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, pair_place: torch.Tensor, shared: Optional[torch.Tensor] = None,
+                 gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x[row] += sum over the row's choices, in their order, of weight[row, j] * y[pair_place[row, j]], plus with ``shared``
+    [rows, hidden] and ``gate`` [rows, 1] (rows may lie apart) sigmoid(gate) * shared; float32."""
+    _dev(x, y, weight, pair_place, shared)
     for name, t in (("x", x), ("y", y), ("weight", weight)):
         _want(t, torch.float32, name)
     _want(pair_place, torch.int32, "pair_place")
@@ -1758,19 +1773,26 @@ def moe_combine_(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, pair_pl
     top = weight.shape[1]
     if weight.shape != (rows, top) or pair_place.shape != (rows, top) or y.shape != (rows * top, hidden):
         raise KernelError(f"moe_combine: x {tuple(x.shape)}, y {tuple(y.shape)}, weight {tuple(weight.shape)}, places {tuple(pair_place.shape)}")
-    _check(library().fw_moe_combine(_p(x), _p(y), _p(weight), _p(pair_place), rows, top, hidden, _stream()))
+    if (shared is None) != (gate is None):
+        raise KernelError("moe_combine: rows to be gated and their gate come together")
+    if shared is not None:
+        _dev_rows(gate, "gate")
+        if shared.dtype != torch.float32 or shared.shape != (rows, hidden) or gate.dtype != torch.float32 or gate.shape != (rows, 1):
+            raise KernelError(f"moe_combine: shared rows {tuple(shared.shape)} and gate {tuple(gate.shape)} beside x {tuple(x.shape)}")
+    _check(library().fw_moe_combine(_p(x), _p(y), _p(weight), _p(pair_place), _p(shared), _p(gate), _stride(gate) if gate is not None else 0,
+                                    rows, top, hidden, _stream()))
     return x
 
 
 # ---- a short causal convolution per channel, and a gated linear recurrence per channel ---------------------------------
 def causal_conv(x: torch.Tensor, taps: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor, row_seg: torch.Tensor,
                 seg_row0: torch.Tensor, seg_slot: torch.Tensor, segments: int, single_rows: bool = False,
-                echo: Optional[tuple] = None) -> torch.Tensor:
+                echo: Optional[tuple] = None, silu: bool = False, rounded: bool = False):
     """y[t, c] = sum_j taps[c, j] * x[t - L + 1 + j, c] (+ bias[c]) over the step's segments, float32. ``x`` float32
     [rows, channels] (rows may lie apart), ``taps`` [channels, L] with the last column the current token's, ``state``
     float32 [slots, channels, L - 1]: the inputs before each segment's first row, read and moved on. ``echo`` = (first
     channel, count): those channels are written once more behind the others (the output is then that much wider).
-    ``single_rows``: every segment is one row."""
+    ``single_rows``: every segment is one row. ``silu``: y passes silu. ``rounded``: y is returned twice, (float32, bfloat16)."""
     _dev(taps, bias, state, row_seg, seg_row0, seg_slot)
     _dev_rows(x, "x")
     for name, t in (("x", x), ("taps", taps), ("state", state)):
@@ -1789,11 +1811,12 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, bias: Optional[torch.Tensor
     if count and not (0 <= first and first + count <= channels):
         raise KernelError(f"causal_conv: channels {first}..{first + count} of {channels}")
     out = torch.empty((rows, channels + count), dtype=torch.float32, device=x.device)
+    short = torch.empty((rows, channels), dtype=torch.bfloat16, device=x.device) if rounded else None
     stride = x.stride(0) if rows > 1 else max(channels, x.stride(0))
     _check(library().fw_causal_conv(_p(x), stride, _p(taps), _p(bias), _p(state), _p(row_seg), _p(seg_row0), _p(seg_slot), _p(out),
-                                    channels + count, int(first), int(count), channels, rows, int(segments), channels, L,
+                                    channels + count, int(first), int(count), channels, int(silu), _p(short), rows, int(segments), channels, L,
                                     state.shape[0], int(bool(single_rows)), _stream()))
-    return out
+    return (out, short) if rounded else out
 
 
 SCAN_LONG = 256     # rows of a segment beyond which the recurrence walks it in chunks side by side
@@ -1830,4 +1853,166 @@ def rglru_scan(u: torch.Tensor, gates: torch.Tensor, y: torch.Tensor, r_bias: to
     _check(library().fw_rglru_scan(_p(u), stride(u), _p(gates), 2 * channels, _p(y), stride(y), _p(r_bias), _p(i_bias), _p(lam),
                                    ctypes.c_float(rate), _p(state), _p(seg_row0), _p(seg_slot), _p(out), _code(out_dtype), rows,
                                    int(segments), channels, int(block_width), state.shape[0], _p(workspace), _stream()))
+    return out
+
+
+# ---- a residual stream of several rows side by side ----------------------------------------------------------------
+NEXT_SUM, NEXT_TANH = 1, 2
+SOURCE_ROWS, SOURCE_BRANCHES, SOURCE_CHOSEN = 0, 1, 2
+MAX_STREAMS = 32
+
+
+def _reader(kind: int, streams: int, hidden: int, reader_in: Optional[torch.Tensor], weight: Optional[torch.Tensor],
+            bias: Optional[torch.Tensor], alpha: Optional[torch.Tensor]) -> tuple:
+    for name, t, shape in (("reader_in", reader_in, (streams,)), ("weight", weight, (hidden,)), ("bias", bias, (hidden,))):
+        if t is not None:
+            _want(t, torch.float32, name)
+            if t.shape != shape:
+                raise KernelError(f"streams: {name} is {tuple(t.shape)}, expected {shape}")
+    if kind == NEXT_TANH and (weight is None or bias is None or alpha is None or alpha.dtype != torch.float32 or alpha.numel() != 1):
+        raise KernelError("streams: the tanh norm has a weight, a bias and one float32 alpha")
+    return int(kind), _p(reader_in), _p(weight), _p(bias), _p(alpha)
+
+
+def stream_read(x: torch.Tensor, reader_in: Optional[torch.Tensor], out_dtype: torch.dtype, *, kind: int = NEXT_SUM,
+                weight: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None, alpha: Optional[torch.Tensor] = None,
+                row_index: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """u = sum_s reader_in[s] x_s of the streams ``x`` float32 [rows, streams, hidden] (``reader_in`` None: their plain sum),
+    as it is (``NEXT_SUM``) or through the norm tanh(alpha u) weight + bias (``NEXT_TANH``); rows gathered through
+    ``row_index`` if given."""
+    _dev(x, reader_in, weight, bias, alpha, row_index)
+    _want(x, torch.float32, "x")
+    if x.dim() != 3 or kind not in (NEXT_SUM, NEXT_TANH):
+        raise KernelError(f"stream_read: the streams are {tuple(x.shape)}, kind {kind}")
+    rows, streams, hidden = x.shape
+    if row_index is not None:
+        _want(row_index, torch.int32, "row_index")
+        rows = row_index.numel()
+    out = torch.empty((rows, hidden), dtype=out_dtype, device=x.device)
+    _check(library().fw_stream_read(_p(x), streams, *_reader(kind, streams, hidden, reader_in, weight, bias, alpha), _p(row_index), _p(out),
+                                    _code(out_dtype), rows, hidden, _stream()))
+    return out
+
+
+def stream_join_(x: torch.Tensor, ls: torch.Tensor, mix: torch.Tensor, out_weight: torch.Tensor, a: torch.Tensor, *,
+                 branches: Optional[tuple] = None, chosen: Optional[tuple] = None, next_kind: int = NEXT_NOTHING,
+                 next_in: Optional[torch.Tensor] = None, next_weight: Optional[torch.Tensor] = None,
+                 next_bias: Optional[torch.Tensor] = None, next_alpha: Optional[torch.Tensor] = None,
+                 next_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
+    """In place on the streams ``x`` float32 [rows, streams, hidden]: x_t <- sum_s mix[s, t] x_s + out_weight[t] * (ls * y).
+    y is ``a`` [rows, hidden]; with ``branches`` = (b, weight_a, weight_b, scale_a, scale_b, eps) it is scale_a rms(a) weight_a +
+    scale_b rms(b) weight_b; with ``chosen`` = (choice_weight, pair_place, b or None, gate or None) it is the sum of the rows of
+    ``a`` [places, hidden] that each row chose, in order, plus sigmoid(gate) b (``gate`` float32, one number a row, rows may lie
+    apart; b [rows, hidden]). ``next_kind`` NEXT_SUM or NEXT_TANH: what reads the streams next (see ``stream_read``) is formed in
+    the same kernel and returned in ``next_dtype``."""
+    _dev(x, ls, mix, out_weight, a, next_in, next_weight, next_bias, next_alpha)
+    for name, t in (("x", x), ("ls", ls), ("mix", mix), ("out_weight", out_weight), ("a", a)):
+        _want(t, torch.float32, name)
+    if x.dim() != 3:
+        raise KernelError(f"stream_join: the streams are {tuple(x.shape)}, expected [rows, streams, hidden]")
+    rows, streams, hidden = x.shape
+    if ls.shape != (hidden,) or mix.shape != (streams, streams) or out_weight.shape != (streams,) or next_kind not in (NEXT_NOTHING, NEXT_SUM, NEXT_TANH):
+        raise KernelError(f"stream_join: streams {tuple(x.shape)}, scales {tuple(ls.shape)}, mix {tuple(mix.shape)}, kind {next_kind}")
+    source, b, weight_a, weight_b, scale_a, scale_b, eps = SOURCE_ROWS, None, None, None, 1.0, 1.0, 0.0
+    choice_weight, pair_place, top, gate = None, None, 0, None
+    places = rows
+    if branches is not None:
+        source = SOURCE_BRANCHES
+        b, weight_a, weight_b, scale_a, scale_b, eps = branches
+        for name, t, shape in (("b", b, (rows, hidden)), ("weight_a", weight_a, (hidden,)), ("weight_b", weight_b, (hidden,))):
+            _dev(t)
+            if t is None or t.dtype != torch.float32 or t.shape != shape:
+                raise KernelError(f"stream_join: {name} must be float32 {shape}")
+    elif chosen is not None:
+        source = SOURCE_CHOSEN
+        choice_weight, pair_place, b, gate = chosen
+        _dev(choice_weight, pair_place, b)
+        _want(choice_weight, torch.float32, "choice_weight")
+        _want(pair_place, torch.int32, "pair_place")
+        top = choice_weight.shape[1]
+        places = rows * top
+        if choice_weight.shape != (rows, top) or pair_place.shape != (rows, top):
+            raise KernelError(f"stream_join: weights {tuple(choice_weight.shape)} and places {tuple(pair_place.shape)} of {rows} rows")
+        if b is not None and (b.dtype != torch.float32 or b.shape != (rows, hidden)):
+            raise KernelError(f"stream_join: b is {tuple(b.shape)}, expected float32 {(rows, hidden)}")
+        if gate is not None:
+            _dev_rows(gate, "gate")
+            if b is None or gate.dtype != torch.float32 or gate.shape != (rows, 1):
+                raise KernelError(f"stream_join: a gate is one float32 number a row beside rows to gate, found {tuple(gate.shape)}")
+    if a.shape != (places, hidden):
+        raise KernelError(f"stream_join: a is {tuple(a.shape)}, expected {(places, hidden)}")
+    out = torch.empty((rows, hidden), dtype=next_dtype or torch.float32, device=x.device) if next_kind != NEXT_NOTHING else None
+    _check(library().fw_stream_join(
+        _p(x), streams, _p(ls), _p(mix), _p(out_weight), source, _p(a), _p(b), _p(weight_a), _p(weight_b), ctypes.c_float(scale_a),
+        ctypes.c_float(scale_b), ctypes.c_float(eps), _p(choice_weight), _p(pair_place), int(top), _p(gate),
+        _stride(gate) if gate is not None else 0, *_reader(next_kind, streams, hidden, next_in, next_weight, next_bias, next_alpha), _p(out),
+        _code(out.dtype) if out is not None else F32, rows, hidden, _stream()))
+    return out
+
+
+# ---- a linear recurrence over a matrix state per head with a fixed decay -------------------------------------------------
+def _segments(name: str, segments: int, seg_row0: torch.Tensor, seg_slot: torch.Tensor) -> None:
+    _dev(seg_row0, seg_slot)
+    for which, t, n in (("seg_row0", seg_row0, segments + 1), ("seg_slot", seg_slot, segments)):
+        _want(t, torch.int32, which)
+        if t.numel() < n:
+            raise KernelError(f"{name}: {which} holds {t.numel()} entries, needs {n}")
+
+
+MAX_DECAY_DIM = 256      # key channels of a head
+
+
+def decay_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, seg_row0: torch.Tensor,
+                     seg_slot: torch.Tensor, segments: int, heads: int, dim: int, vdim: int) -> torch.Tensor:
+    """Per head S <- decay S + silu(k) silu(v)^T, o = S^T silu(q) over each segment's rows in order. ``q``, ``k`` float32
+    [rows, heads dim] and ``v`` [rows, heads vdim] with one row stride (views of wider rows will do); ``decay`` float32 [heads];
+    ``state`` float32 [slots, heads, dim, vdim] is read and moved on. Returns float32 [rows, heads vdim]."""
+    _dev(decay, state)
+    _segments("decay_recurrence", segments, seg_row0, seg_slot)
+    rows = q.shape[0]
+    for name, t, width in (("q", q, heads * dim), ("k", k, heads * dim), ("v", v, heads * vdim)):
+        _dev_rows(t, name)
+        _want(t, torch.float32, name)
+        if t.shape != (rows, width):
+            raise KernelError(f"decay_recurrence: {name} is {tuple(t.shape)}, expected {(rows, width)}")
+    if rows > 1 and not (q.stride(0) == k.stride(0) == v.stride(0)):
+        raise KernelError("decay_recurrence: q, k and v have one row stride")
+    stride = max(_stride(q), _stride(k), _stride(v))
+    for name, t, shape in (("decay", decay, (heads,)), ("state", state[0], (heads, dim, vdim))):
+        _want(t, torch.float32, name)
+        if t.shape != shape:
+            raise KernelError(f"decay_recurrence: {name} is {tuple(t.shape)}, expected {shape}")
+    out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=q.device)
+    _check(library().fw_decay_recurrence(_p(q), _p(k), _p(v), stride, _p(decay), _p(state), state.shape[0], _p(out), _p(seg_row0),
+                                         _p(seg_slot), rows, int(segments), heads, dim, vdim, _stream()))
+    return out
+
+
+# ---- the selective scan ---------------------------------------------------------------------------------------------
+MAX_SCAN_STATES = 128
+
+
+def selective_scan(x: torch.Tensor, z: torch.Tensor, bc: torch.Tensor, gate: torch.Tensor, A2: torch.Tensor, D: torch.Tensor,
+                   state: torch.Tensor, seg_row0: torch.Tensor, seg_slot: torch.Tensor, segments: int, out_dtype: torch.dtype) -> torch.Tensor:
+    """Per channel c and state n, with dt = softplus(z): S <- 2^(dt A2[n, c]) S + dt x B[n], y = sum_n S C[n] + D x, out = y *
+    silu(gate), over each segment's rows in order. ``x``, ``z``, ``gate`` float32 [rows, channels], ``bc`` float32 [rows, 2 states]
+    (B, then C); rows may lie apart. ``A2`` [states, channels] and ``D`` [channels] float32; ``state`` float32 [slots, states,
+    channels] is read and moved on. Returns [rows, channels] of ``out_dtype``."""
+    _dev(A2, D, state)
+    _segments("selective_scan", segments, seg_row0, seg_slot)
+    rows, channels = x.shape
+    states = A2.shape[0]
+    for name, t, shape in (("x", x, (rows, channels)), ("z", z, (rows, channels)), ("bc", bc, (rows, 2 * states)), ("gate", gate, (rows, channels))):
+        _dev_rows(t, name)
+        _want(t, torch.float32, name)
+        if t.shape != shape:
+            raise KernelError(f"selective_scan: {name} is {tuple(t.shape)}, expected {shape}")
+    for name, t, shape in (("A2", A2, (states, channels)), ("D", D, (channels,)), ("state", state[0], (states, channels))):
+        _want(t, torch.float32, name)
+        if t.shape != shape:
+            raise KernelError(f"selective_scan: {name} is {tuple(t.shape)}, expected {shape}")
+    out = torch.empty((rows, channels), dtype=out_dtype, device=x.device)
+    _check(library().fw_selective_scan(_p(x), _stride(x), _p(z), _stride(z), _p(bc), _stride(bc), _p(gate), _stride(gate), _p(A2), _p(D), _p(state),
+                                       state.shape[0], _p(out), _code(out_dtype), _p(seg_row0), _p(seg_slot), rows, int(segments), channels,
+                                       states, _stream()))
     return out

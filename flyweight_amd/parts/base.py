@@ -20,7 +20,7 @@ struct (native/src/v2_runtime.cpp:395-560,4177-4184).
 
 from __future__ import annotations
 
-from typing import Callable, Dict, Mapping, Optional, Type
+from typing import Callable, Dict, Mapping, NamedTuple, Optional, Type
 
 import torch
 
@@ -69,6 +69,16 @@ class Part:
         place), ``batch`` has this replay's ``host_row_pos`` and ``host_seg_slot``. When several
         steps run back to back on the device this is called before the first of them only.
         The default leaves the arrays as they were built."""
+
+
+class SublayerOutput(NamedTuple):
+    """A sublayer's output as a kernel that joins it to the residual stream takes it (``joined_output`` of a part that
+    leaves more to that kernel than rows to add): float32 ``rows``; with ``branches`` = (b, weight_a, weight_b, scale_a,
+    scale_b, eps) scale_a rms(rows) weight_a + scale_b rms(b) weight_b; with ``chosen`` = (weight, place, b, gate) the weighted
+    sum of the ``rows`` each row chose, plus sigmoid(gate) b."""
+    rows: torch.Tensor
+    branches: Optional[tuple] = None
+    chosen: Optional[tuple] = None
 
 
 class Norm(Part):

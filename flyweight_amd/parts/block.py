@@ -16,15 +16,19 @@ x also forms what reads x next (the next norm's output, or x rounded, also in it
 
 ``parallel_residual``: with h = norm1(x), x <- x + (mixer(h) + ffn(h)): one norm, and both sublayers read its
 output. The feed-forward may be absent.
+
+``stream_residual``: x is several rows side by side that a sublayer reads as one weighted sum and writes to all (see
+``parts/streams.py``). The feed-forward may be absent.
 """
 
 from __future__ import annotations
 
 from ..config.spec import ConfigError
 from ..kernels import ops
-from .base import Block, build_part, register_block
+from .base import Block, SublayerOutput, build_part, register_block
 from .input_join import JoinedRows
 from .norm import LazyNorm, NormedRows
+from .streams import StreamConnection, StreamReader, StreamRows
 from .token_input import TokenInput
 
 
@@ -256,3 +260,58 @@ class ParallelResidualBlock(Block):
         if self.ffn is not None:
             self.ffn.forward(normed, x, ctx)
         return None
+
+
+@register_block("stream_residual")
+class StreamResidualBlock(Block):
+    """``LayerSpec.params``: ``mixer_connection`` and ``ffn_connection`` (PartSpecs of :class:`StreamConnection`). ``x`` is float32
+    [rows, streams, hidden]. What a sublayer leaves (``joined_output``, or rows of its ``output``) joins the streams in the kernel
+    that also forms what reads them next, the layer after this one included (``norm_after``: its :class:`StreamReader`)."""
+
+    def __init__(self, spec):
+        self.spec = spec
+        self.mixer_norm = build_part("norm", spec.mixer_norm)
+        self.mixer = build_part("mixer", spec.mixer)
+        self.mixer_connection = StreamConnection(spec.params["mixer_connection"])
+        self.ffn = build_part("ffn", spec.ffn) if spec.ffn is not None else None
+        self.ffn_norm = build_part("norm", spec.ffn_norm) if spec.ffn is not None else None
+        self.ffn_connection = StreamConnection(spec.params["ffn_connection"]) if spec.ffn is not None else None
+        self.mixer_reader = StreamReader(self.mixer_norm)
+        self.ffn_reader = StreamReader(self.ffn_norm) if spec.ffn is not None else None
+        for part in (self.mixer, self.ffn):
+            if part is not None and not hasattr(part, "joined_output") and not hasattr(part, "output"):
+                raise ConfigError(f"part '{part.spec.kind}' cannot give its output apart from the residual stream")
+
+    def parts(self):
+        return tuple(part for part in (self.mixer_norm, self.mixer, self.mixer_connection, self.ffn_norm, self.ffn, self.ffn_connection)
+                     if part is not None)
+
+    def bind(self, tensors, dtype, device) -> None:
+        super().bind(tensors, dtype, device)
+        self.mixer_reader.weights = self.mixer_connection.weights_in
+        if self.ffn is not None:
+            self.ffn_reader.weights = self.ffn_connection.weights_in
+
+    def first_norm(self):
+        return self.mixer_reader
+
+    def cache_need(self):
+        return self.mixer.cache_need()
+
+    @property
+    def graph_safe(self) -> bool:
+        position = getattr(self.mixer, "position", None)
+        return all(part.graph_safe for part in self.parts()) and (position is None or position.graph_safe)
+
+    @staticmethod
+    def _output(part, *args) -> SublayerOutput:
+        return part.joined_output(*args) if hasattr(part, "joined_output") else SublayerOutput(part.output(*args))
+
+    def forward(self, x, ctx, cache, prepared=None, norm_after=None):
+        """``x`` is updated in place."""
+        after = norm_after if isinstance(norm_after, StreamReader) else None
+        h = self.mixer_reader.take(x, ctx, prepared)
+        h = self.mixer_connection.join(x, self._output(self.mixer, h, ctx, cache), self.ffn_reader if self.ffn is not None else after, ctx)
+        if self.ffn is not None:
+            h = self.ffn_connection.join(x, self._output(self.ffn, h, ctx), after, ctx)
+        return None if after is None else StreamRows(after, h)

@@ -136,8 +136,11 @@ class Linear:
         ops.gemm(a, self.weight, self.bias, accumulate_into=residual, w_tiled=self.tiled)
         return None
 
-    def swiglu(self, a: Input) -> torch.Tensor:
-        """The weight holds gate rows then up rows: silu(a . gate^T) * (a . up^T)."""
+    def swiglu(self, a: Input, gelu: bool = False) -> torch.Tensor:
+        """The weight holds gate rows then up rows: silu(a . gate^T) * (a . up^T); ``gelu``: the tanh form of gelu in
+        place of silu."""
+        if gelu:
+            return ops.swiglu(self.forward(a, out_dtype=torch.float32), out_dtype=a.dtype, gelu=True)
         if self.bias is None and self._medium(a):
             return ops.gemm_medium(self._rows_of(a), self.weight, ops.EPILOGUE_SWIGLU, w_tiled=self.tiled, **self._prepared_arguments(a))
         if self.bias is None and self._fused(a, self.out_features // 2, ops.EPILOGUE_SWIGLU):

@@ -15,7 +15,10 @@ expert's, and only experts of the ``keep`` best groups can be chosen; ``group_sc
 two best experts score together instead. ``router_scores`` "sigmoid": every expert scores sigmoid(z) on its own, and the
 chosen scores divided by their sum (+ 1e-20) are the weights. ``unit`` "clamped" with ``limit`` (and ``alpha``,
 ``shift``): an expert is W_down (g sigmoid(alpha g) (u + shift)) with g = min(W_gate h, limit), u = clamp(W_up h, -limit,
-limit); the shared unit is then of the same form with ``shared_limit``. Registered as ``moe_swiglu`` and ``moe_glu``.
+limit); the shared unit is then of the same form with ``shared_limit``.
+``router_correction`` (with sigmoid scores): a vector per expert that is added to the scores for the choice alone.
+``weight_scale`` multiplies the weights, ``normalize`` False leaves them undivided. ``shared_gate``: the shared unit's output is
+multiplied by sigmoid(W_sg h), one number per token. Registered as ``moe_swiglu`` and ``moe_glu``.
 """
 
 from __future__ import annotations
@@ -27,12 +30,12 @@ import torch
 from ..config.spec import ConfigError, PartSpec
 from ..kernels import ops
 from ..weights.loader import TensorDecl
-from .base import FeedForward, build_part, register_feed_forward
+from .base import FeedForward, SublayerOutput, build_part, register_feed_forward
 from .linear import Linear
 from .norm import LazyNorm
 
 _DEFAULT_NAMES = {"router": "router", "router_bias": "router.b", "expert": "e{index}.", "gate": "gate", "up": "up", "down": "down",
-                  "shared": "shared."}
+                  "shared": "shared.", "shared_gate": "shared.sg", "correction": "correction"}
 
 
 @register_feed_forward("moe_glu")
@@ -54,7 +57,15 @@ class MoeSwiGLU(FeedForward):
         self.groups, self.keep_groups = (int(n) for n in (spec.get("router_groups") or (1, 1)))
         self.clamped = spec.get("unit", "swiglu") == "clamped"
         self.glu = (float(spec["limit"]), float(spec.get("alpha", 1.702)), float(spec.get("shift", 1.0))) if self.clamped else None
+        self.has_correction = bool(spec.get("router_correction", False))
+        self.weight_scale = float(spec.get("weight_scale", 1.0))
+        self.normalize = bool(spec.get("normalize", True))
+        self.shared_gate = bool(spec.get("shared_gate", False))
         self.names = {**_DEFAULT_NAMES, **dict(spec.get("names", {}))}
+        if (self.has_correction and self.scores != "sigmoid") or (not self.normalize and self.scores == "softmax_chosen"):
+            raise ConfigError("a correction of the choice goes with sigmoid scores; weights that are a softmax over the chosen are a distribution")
+        if self.shared_gate and not self.shared_intermediate:
+            raise ConfigError("a gate on the shared unit needs a shared unit")
         if self.scores not in ops.MOE_SCORES or spec.get("unit", "swiglu") not in ("swiglu", "clamped"):
             raise ConfigError(f"a mixture's router scores are one of {', '.join(ops.MOE_SCORES)}, its units 'swiglu' or 'clamped'")
         if spec.get("group_score", "best") not in ("best", "pair") or (self.group_pair and self.scores == "softmax_chosen"):
@@ -88,6 +99,10 @@ class MoeSwiGLU(FeedForward):
         declared = {self.prefix + self.names["router"]: TensorDecl((self.experts, D))}
         if self.router_bias:
             declared[self.prefix + self.names["router_bias"]] = TensorDecl((self.experts,), "vector", "bias")
+        if self.has_correction:
+            declared[self.prefix + self.names["correction"]] = TensorDecl((self.experts,), "vector", "bias")
+        if self.shared_gate:
+            declared[self.prefix + self.names["shared_gate"]] = TensorDecl((1, D))
         for index in range(self.experts):
             declared[self._expert(index, "gate")] = TensorDecl((F, D))
             declared[self._expert(index, "up")] = TensorDecl((F, D))
@@ -98,7 +113,13 @@ class MoeSwiGLU(FeedForward):
 
     def bind(self, tensors, dtype, device) -> None:
         super().bind(tensors, dtype, device)
-        self.router = Linear(tensors[self.prefix + self.names["router"]])
+        router = tensors[self.prefix + self.names["router"]]
+        if self.shared_gate:        # one more row of the router's product, behind the experts' (rows of zeros fill it up)
+            gate = tensors[self.prefix + self.names["shared_gate"]].to(router.dtype)
+            fill = torch.zeros((-(self.experts + 1) % 8, self.hidden), dtype=router.dtype, device=router.device)
+            router = torch.cat([router, gate, fill], dim=0)
+        self.router = Linear(router)
+        self.correction = tensors[self.prefix + self.names["correction"]] if self.has_correction else None
         self.bias = tensors[self.prefix + self.names["router_bias"]] if self.router_bias else None
         self.gate_up = torch.stack([torch.cat([tensors[self._expert(e, "gate")], tensors[self._expert(e, "up")]], dim=0)
                                     for e in range(self.experts)]).contiguous()
@@ -119,18 +140,50 @@ class MoeSwiGLU(FeedForward):
     def chosen_flops_per_token(self) -> int:
         return 2 * self.top * 3 * self.hidden * self.intermediate
 
+    def _logits(self, h: torch.Tensor):
+        """(the router's logits [rows, experts], the shared unit's gate [rows, 1] before its sigmoid or None)."""
+        logits = self.router.forward(h, out_dtype=torch.float32)
+        if not self.shared_gate:
+            return logits, None
+        return logits[:, :self.experts], logits[:, self.experts:self.experts + 1]
+
+    def _choose(self, logits: torch.Tensor):
+        return ops.moe_route(logits, self.bias, self.top, self.groups, self.keep_groups, scores=self.scores, group_pair=self.group_pair,
+                             correction=self.correction, weight_scale=self.weight_scale, normalize=self.normalize)
+
     def route(self, h: torch.Tensor):
         """(chosen [rows, top], weight [rows, top]) of the rows ``h``."""
-        logits = self.router.forward(h, out_dtype=torch.float32)
-        return ops.moe_route(logits, self.bias, self.top, self.groups, self.keep_groups, scores=self.scores, group_pair=self.group_pair)
+        return self._choose(self._logits(h)[0])
 
-    def forward(self, h, residual, ctx):
-        rows = (h.tensor() if isinstance(h, LazyNorm) else h)
-        chosen, weight = self.route(rows)
+    def _experts_output(self, rows: torch.Tensor):
+        """(the chosen experts' outputs by place, the choices' weights, the pairs' places, the shared unit's gate or None)."""
+        logits, gate = self._logits(rows)
+        chosen, weight = self._choose(logits)
         begin, place_row, pair_place = ops.moe_arrange(chosen, self.experts)
         places = rows.shape[0] * self.top
         hidden = ops.grouped_gemm(rows, place_row, self.gate_up, begin, places, gated=True, out_dtype=rows.dtype, glu=self.glu)
-        outputs = ops.grouped_gemm(hidden, None, self.down, begin, places, gated=False, out_dtype=torch.float32)
+        return ops.grouped_gemm(hidden, None, self.down, begin, places, gated=False, out_dtype=torch.float32), weight, pair_place, gate
+
+    def _shared_output(self, h, rows, ctx):
+        if self.shared is None:
+            return None
+        if hasattr(self.shared, "output"):
+            return self.shared.output(rows, ctx)
+        ((output, _),) = self.shared.output_terms(rows, ctx)
+        return output
+
+    def joined_output(self, h, ctx) -> SublayerOutput:
+        """The output for a kernel that joins it to the residual stream: the experts' rows are summed there."""
+        rows = (h.tensor() if isinstance(h, LazyNorm) else h)
+        outputs, weight, pair_place, gate = self._experts_output(rows)
+        return SublayerOutput(outputs, chosen=(weight, pair_place, self._shared_output(h, rows, ctx), gate))
+
+    def forward(self, h, residual, ctx):
+        rows = (h.tensor() if isinstance(h, LazyNorm) else h)
+        outputs, weight, pair_place, gate = self._experts_output(rows)
+        if gate is not None:
+            ops.moe_combine_(residual, outputs, weight, pair_place, shared=self._shared_output(h, rows, ctx), gate=gate)
+            return None
         ops.moe_combine_(residual, outputs, weight, pair_place)
         if self.shared is not None:
             return self.shared.forward(h if getattr(self.shared, "accepts_lazy_norm", False) else rows, residual, ctx)

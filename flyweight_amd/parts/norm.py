@@ -1,7 +1,8 @@
 """RMS norm: y = x * rsqrt(mean(x^2) + eps) * w, sums in float32; the weight multiplies
 directly (native/include/flyweight_v2_qwen_kernels.hpp:425-447 with one_centered = 0).
 Layer norm: the row's mean is taken off first, y = (x - m) * rsqrt(mean((x - m)^2) + eps) * w, plus a bias vector where
-the design has one."""
+the design has one.
+The tanh norm takes no statistics of the row: y = tanh(alpha x) w + b, alpha one number."""
 
 from __future__ import annotations
 
@@ -144,3 +145,37 @@ class LayerNorm(Norm):
 
     def forward(self, x: torch.Tensor, ctx, row_index: Optional[torch.Tensor] = None) -> torch.Tensor:
         return ops.layernorm_rows(x, self.weight, self.eps, self.dtype, row_index=row_index, bias=self.bias)
+
+
+@register_norm("tanh")
+class TanhNorm(Norm):
+    """tanh(alpha x) * w + b per channel (Dynamic Tanh: Zhu, Chen, He, LeCun and Liu, "Transformers without Normalization"). The
+    scalar and the bias are the tensors of the weight's name with ".alpha" and ".b" behind it. A kernel that works on some
+    channels of a row alone can apply it (``tanh_parameters``)."""
+    graph_safe = True
+
+    def __init__(self, spec):
+        super().__init__(spec)
+        self.size = int(spec["size"])
+
+    @property
+    def tensor_name(self) -> str:
+        return self.spec.get("tensor") or self.prefix + "weight"
+
+    def tensors(self) -> Dict[str, TensorDecl]:
+        return {self.tensor_name: TensorDecl((self.size,), role="vector", init="norm"),
+                self.tensor_name + ".b": TensorDecl((self.size,), role="vector", init="bias"),
+                self.tensor_name + ".alpha": TensorDecl((), role="vector", init="norm")}
+
+    def bind(self, tensors, dtype, device) -> None:
+        super().bind(tensors, dtype, device)
+        self.weight = tensors[self.tensor_name]
+        self.bias = tensors[self.tensor_name + ".b"]
+        self.alpha = tensors[self.tensor_name + ".alpha"]
+
+    def tanh_parameters(self):
+        return self.weight, self.bias, self.alpha
+
+    def forward(self, x: torch.Tensor, ctx, row_index: Optional[torch.Tensor] = None) -> torch.Tensor:
+        return ops.stream_read(x.unsqueeze(1), None, self.dtype, kind=ops.NEXT_TANH, weight=self.weight, bias=self.bias, alpha=self.alpha,
+                               row_index=row_index)

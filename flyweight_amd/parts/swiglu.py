@@ -1,6 +1,6 @@
 """SwiGLU feed-forward: f = W_down (silu(W_gate h) * (W_up h)), no biases
 (native/src/v2_runtime.cpp:28797-28805; silu_mul native/include/flyweight_v2_qwen_kernels.hpp:1209-1223).
-Gate and up are one operand of 2I rows, so h is read once."""
+Gate and up are one operand of 2I rows, so h is read once. ``activation`` "gelu_tanh": the tanh form of gelu in place of silu."""
 
 from __future__ import annotations
 
@@ -29,6 +29,10 @@ class SwiGLU(FeedForward):
         self.names = {**_DEFAULT_NAMES, **dict(spec.get("names", {}))}
         # what follows a tensor's name in the checkpoint: ".weight" unless the layout has none
         self.weight_suffix = spec.get("weight_suffix", ".weight")
+        activation = spec.get("activation", "silu")
+        if activation not in ("silu", "gelu_tanh"):
+            raise ConfigError(f"a gated unit's activation is 'silu' or 'gelu_tanh', not {activation!r}")
+        self.gelu = activation == "gelu_tanh"
 
     def _name(self, which: str) -> str:
         return f"{self.prefix}{self.names[which]}{self.weight_suffix}"
@@ -50,9 +54,9 @@ class SwiGLU(FeedForward):
 
     def forward(self, h, residual, ctx):
         # the activation is formed from float32 sums and rounded once
-        return self.down.accumulate(self.gate_up.swiglu(h), residual, then=getattr(ctx, "upcoming_norm", None))
+        return self.down.accumulate(self.gate_up.swiglu(h, gelu=self.gelu), residual, then=getattr(ctx, "upcoming_norm", None))
 
     def output(self, h, ctx) -> torch.Tensor:
         """The feed-forward's output as float32 rows of its own (for arrangements that do something to
         it before it joins the residual stream)."""
-        return self.down.forward(self.gate_up.swiglu(h), out_dtype=torch.float32)
+        return self.down.forward(self.gate_up.swiglu(h, gelu=self.gelu), out_dtype=torch.float32)

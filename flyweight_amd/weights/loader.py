@@ -30,7 +30,7 @@ class TensorDecl:
 
     shape: Tuple[int, ...]
     role: str = "matrix"
-    init: str = "matrix"        # matrix | norm | conv | bias | zeros
+    init: str = "matrix"        # matrix | norm | conv | bias | zeros | share (equal shares of one) | unit (the unit matrix)
 
 
 class WeightError(ValueError):

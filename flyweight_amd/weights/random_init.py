@@ -36,6 +36,13 @@ def _std(decl: TensorDecl, scale: str) -> float:
     return {"conv": 0.5, "bias": 0.1}[decl.init]
 
 
+def _fixed(decl: TensorDecl) -> torch.Tensor:
+    """Tensors that are not drawn: zeros, equal shares that add up to one, the unit matrix."""
+    if decl.init == "share":
+        return torch.full(decl.shape, 1.0 / max(decl.shape[-1], 1), dtype=torch.float32)
+    return torch.eye(decl.shape[0], dtype=torch.float32) if decl.init == "unit" else torch.zeros(decl.shape, dtype=torch.float32)
+
+
 def random_tensors(declared: Mapping[str, TensorDecl], seed: int,
                    matrix_dtype: torch.dtype = torch.bfloat16, scale: str = "small") -> Dict[str, torch.Tensor]:
     generator = torch.Generator(device="cpu")
@@ -48,8 +55,8 @@ def random_tensors(declared: Mapping[str, TensorDecl], seed: int,
             continue
         if decl.init == "norm":
             value = 1.0 + (torch.rand(decl.shape, generator=generator, dtype=torch.float32) * 0.2 - 0.1)
-        elif decl.init == "zeros":
-            value = torch.zeros(decl.shape, dtype=torch.float32)
+        elif decl.init in ("zeros", "share", "unit"):
+            value = _fixed(decl)
         else:
             value = torch.randn(decl.shape, generator=generator, dtype=torch.float32) * _std(decl, scale)
         tensors[name] = value.to(matrix_dtype) if decl.role == "matrix" else value
@@ -82,8 +89,8 @@ def random_tensors_on_device(declared: Mapping[str, TensorDecl], seed: int, devi
             tensors[name] = torch.zeros(decl.shape, dtype=torch.int32, device=device)
         elif decl.init == "norm":
             tensors[name] = 0.9 + 0.2 * torch.rand(decl.shape, generator=generator, dtype=torch.float32, device=device)
-        elif decl.init == "zeros":
-            tensors[name] = torch.zeros(decl.shape, dtype=torch.float32, device=device)
+        elif decl.init in ("zeros", "share", "unit"):
+            tensors[name] = _fixed(decl).to(device)
         else:
             value = torch.randn(decl.shape, generator=generator, dtype=torch.float32, device=device) * _std(decl, scale)
             tensors[name] = value.to(run_dtype) if decl.role == "matrix" else value
