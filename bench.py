@@ -217,6 +217,35 @@ def zaluvik_configs(size: dict):
     return zaluvik, telapel_configs(size)[0]
 
 
+# Fevolorn (a residual stream of four rows; lightning attention, or windowed attention beside a selective scan; a dense unit
+# or a mixture of experts with a gated shared unit; the second layer runs twice) at the two sizes of DALERAX_SIZES, beside the
+# engine's two closest existing models: a Dalerax of as many layer runs, the same width, vocabulary, experts and window (a
+# linear recurrence of as many key channels, experts and a shared unit), and that Dalerax's Koketar (two mixers side by side).
+FEVOLORN_SIZES = {
+    "w1024": dict(DALERAX_SIZES["w1024"], streams=4, l_heads=8, l_dim=128, l_vdim=128, inner=2048, state=16, dt_rank=64),
+    "w2048": dict(DALERAX_SIZES["w2048"], streams=4, l_heads=16, l_dim=128, l_vdim=128, inner=4096, state=16, dt_rank=128),
+}
+
+
+def fevolorn_configs(size: dict):
+    """(Fevolorn configuration, Dalerax and Koketar configurations of equal size)."""
+    from flyweight_amd.config import config_from_dict
+    moe = {"kind": "moe", "router": {"experts": size["experts"], "top": size["top"], "scale": 1.5}, "expert": {"ff": size["expert_ff"]},
+           "shared": {"ff": size["shared_ff"]}}
+    lightning = {"heads": size["l_heads"], "dim": size["l_dim"], "vdim": size["l_vdim"],
+                 "decay": [1.0 - 2.0 ** (-2.0 - 6.0 * h / size["l_heads"]) for h in range(size["l_heads"])]}
+    parallel = {"left": {"heads": size["heads"], "kv_heads": size["kv_heads"], "dim": size["dim"], "vdim": size["vdim"],
+                         "scale": size["dim"] ** -0.5, "mask": {"size": size["window"]}},
+                "right": {"inner": size["inner"], "state": size["state"], "dt_rank": size["dt_rank"], "conv": size["conv"]}}
+    layers = [{"type": "lightning", "mixer": lightning, "mlp": {"kind": "dense", "ff": size["ff"]}},
+              {"type": "parallel", "mixer": parallel, "mlp": moe},
+              {"type": "lightning", "mixer": lightning, "mlp": moe}]
+    fevolorn = config_from_dict({"architecture": "Fevolorn", "vocab": size["vocab"], "width": size["width"], "streams": size["streams"],
+                                 "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0}, "layers": layers,
+                                 "loop": {"start": 1, "stop": 2, "times": 2}})
+    return (fevolorn,) + dalerax_configs(size)
+
+
 def kernel_times(torch, run) -> dict:
     """Entry point of the kernel library -> microseconds of GPU time per call, over one call of ``run``
     (launched kernel by kernel, every call bracketed by two events)."""
@@ -589,11 +618,12 @@ def main() -> int:
     parser.add_argument("--only", choices=("decode", "prefill"), help="run one phase and print no JSON (for profiling)")
     parser.add_argument("--drawn", action="store_true", help="with --only decode: the requests draw their tokens "
                         "(temperature 0.8, top_k 40, top_p 0.95, min_p 0.05) instead of taking the most likely one")
-    parser.add_argument("--workload", choices=("headline",) + tuple(WORKLOADS) + ("koketar", "vavelorn", "dalerax", "telapel", "zaluvik"), default="headline",
+    parser.add_argument("--workload", choices=("headline",) + tuple(WORKLOADS) + ("koketar", "vavelorn", "dalerax", "telapel", "zaluvik", "fevolorn"), default="headline",
                         help="headline: the LFM2-1.2B decode and prefill figures; long-context, mixed: a whole serving run; "
                              "koketar: prefill and decode of Koketar beside LFM2 at equal sizes, kernel by kernel; "
                              "vavelorn: the same of Vavelorn beside Koketar; dalerax: the same of Dalerax beside Koketar; "
-                             "telapel: the same of Telapel beside Dalerax; zaluvik: the same of Zaluvik beside Telapel")
+                             "telapel: the same of Telapel beside Dalerax; zaluvik: the same of Zaluvik beside Telapel; "
+                             "fevolorn: the same of Fevolorn beside Dalerax and Koketar")
     parser.add_argument("--requests", type=int, help="requests of a serving workload (default: as the workload names)")
     args = parser.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
@@ -607,8 +637,11 @@ def main() -> int:
     from flyweight_amd import Model
     from flyweight_amd.config import config_from_dict
 
-    if args.workload in ("koketar", "vavelorn", "dalerax", "telapel", "zaluvik"):
-        if args.workload == "zaluvik":
+    if args.workload in ("koketar", "vavelorn", "dalerax", "telapel", "zaluvik", "fevolorn"):
+        if args.workload == "fevolorn":
+            record = koketar_run(torch, args, families=("fevolorn", "dalerax", "koketar"), sizes=FEVOLORN_SIZES, configs_of=fevolorn_configs,
+                                 title="Fevolorn", beside="Fevolorn beside Dalerax and Koketar at equal width, layer runs, vocabulary and window")
+        elif args.workload == "zaluvik":
             record = koketar_run(torch, args, families=("zaluvik", "telapel"), sizes=ZALUVIK_SIZES, configs_of=zaluvik_configs,
                                  title="Zaluvik", beside="Zaluvik beside Telapel at equal width, layer runs, vocabulary, latent, experts and windows")
         elif args.workload == "telapel":

@@ -373,6 +373,48 @@ __global__ __launch_bounds__(64) void gated_head_norm_kernel(const float* __rest
     }
 }
 
+// The same for wide heads (all of a row's heads normed together are one): a workgroup per (row, head), everything the row needs
+// asked for at once where it fits in registers.
+#define GHN_HELD 16
+template <typename TG, typename T, int N>
+__global__ __launch_bounds__(256) void gated_head_norm_wide_kernel(const float* __restrict__ o, const TG* __restrict__ gate, int gate_stride,
+                                                                 const float* __restrict__ weight, T* __restrict__ out, int heads, int vdim,
+                                                                 float eps, int gate_silu, int weight_per_head) {
+    __shared__ float scratch[4];
+    const int row = blockIdx.x, head = blockIdx.y;
+    const float* source = o + ((size_t)row * heads + head) * vdim;
+    const size_t gate0 = (size_t)row * gate_stride + (size_t)head * vdim;
+    T* to = out + ((size_t)row * heads + head) * vdim;
+    if (weight_per_head) weight += (size_t)head * vdim;
+    float sum = 0.0f;
+    if constexpr (N > 0) {
+        float held[N], scale[N], z[N];
+#pragma unroll
+        for (int u = 0; u < N; ++u) {
+            const int j = threadIdx.x + 256 * u < vdim ? threadIdx.x + 256 * u : vdim - 1;
+            held[u] = source[j];
+            scale[u] = weight[j];
+            z[u] = load_as_float(gate, gate0 + j);
+        }
+#pragma unroll
+        for (int u = 0; u < N; ++u)
+            if (threadIdx.x + 256 * u < vdim) sum = fmaf(held[u], held[u], sum);
+        const float inv = 1.0f / sqrtf(block_sum_by_lds(sum, scratch) / (float)vdim + eps);
+#pragma unroll
+        for (int u = 0; u < N; ++u) {
+            const int j = threadIdx.x + 256 * u;
+            if (j < vdim) store_from_float(to, j, held[u] * inv * scale[u] * (gate_silu ? z[u] * fw_sigmoid(z[u]) : fw_sigmoid(z[u])));
+        }
+    } else {
+        for (int j = threadIdx.x; j < vdim; j += 256) sum = fmaf(source[j], source[j], sum);
+        const float inv = 1.0f / sqrtf(block_sum_by_lds(sum, scratch) / (float)vdim + eps);
+        for (int j = threadIdx.x; j < vdim; j += 256) {
+            const float z = load_as_float(gate, gate0 + j);
+            store_from_float(to, j, source[j] * inv * weight[j] * (gate_silu ? z * fw_sigmoid(z) : fw_sigmoid(z)));
+        }
+    }
+}
+
 extern "C" int fw_gated_head_norm(const float* o, const void* gate, int gate_dtype, int gate_stride, const float* weight,
                                   int weight_per_head, void* out, int out_dtype, int rows, int heads, int vdim, float eps, int gate_silu, void* stream) {
     FW_REQUIRE(rows >= 0 && heads > 0 && heads <= 65535 && vdim > 0, "gated_head_norm: bad sizes rows=%d heads=%d vdim=%d", rows, heads, vdim);
@@ -380,13 +422,24 @@ extern "C" int fw_gated_head_norm(const float* o, const void* gate, int gate_dty
     if (rows == 0) return 0;
     dim3 grid(rows, heads);
     hipStream_t s = (hipStream_t)stream;
-#define FW_GHN_LAUNCH(TG, T) \
-    gated_head_norm_kernel<TG, T><<<grid, 64, 0, s>>>(o, (const TG*)gate, gate_stride, weight, (T*)out, heads, vdim, eps, gate_silu, weight_per_head)
-    if (gate_dtype == FW_F32 && out_dtype == FW_F32) FW_GHN_LAUNCH(float, float);
-    else if (gate_dtype == FW_F32 && out_dtype == FW_BF16) FW_GHN_LAUNCH(float, bf16_t);
-    else if (gate_dtype == FW_BF16 && out_dtype == FW_BF16) FW_GHN_LAUNCH(bf16_t, bf16_t);
+#define FW_GHN_WIDE(TG, T, N)                                                                                                       \
+    gated_head_norm_wide_kernel<TG, T, N><<<grid, 256, 0, s>>>(o, (const TG*)gate, gate_stride, weight, (T*)out, heads, vdim, eps, gate_silu, \
+                                                               weight_per_head)
+#define FW_GHN_LAUNCH(TG, T)                                                                                                        \
+    {                                                                                                                               \
+        if (vdim <= 256) gated_head_norm_kernel<TG, T><<<grid, 64, 0, s>>>(o, (const TG*)gate, gate_stride, weight, (T*)out, heads, vdim, eps, \
+                                                                           gate_silu, weight_per_head);                             \
+        else if (vdim <= 256 * 4) FW_GHN_WIDE(TG, T, 4);                                                                            \
+        else if (vdim <= 256 * 8) FW_GHN_WIDE(TG, T, 8);                                                                            \
+        else if (vdim <= 256 * GHN_HELD) FW_GHN_WIDE(TG, T, GHN_HELD);                                                              \
+        else FW_GHN_WIDE(TG, T, 0);                                                                                                 \
+    }
+    if (gate_dtype == FW_F32 && out_dtype == FW_F32) FW_GHN_LAUNCH(float, float)
+    else if (gate_dtype == FW_F32 && out_dtype == FW_BF16) FW_GHN_LAUNCH(float, bf16_t)
+    else if (gate_dtype == FW_BF16 && out_dtype == FW_BF16) FW_GHN_LAUNCH(bf16_t, bf16_t)
     else FW_REQUIRE(false, "gated_head_norm: unsupported dtypes gate=%d out=%d", gate_dtype, out_dtype);
 #undef FW_GHN_LAUNCH
+#undef FW_GHN_WIDE
     FW_LAUNCH_CHECK("gated_head_norm");
     return 0;
 }

@@ -429,20 +429,37 @@ int fw_stream_join(float* x, int streams, const float* ls, const float* mix, con
                    int next_dtype, int rows, int hidden, void* stream);
 
 // ---- a linear recurrence over a matrix state per head with a fixed decay -----------------------------------------------
-// Per segment and head, with q = silu(q), k = silu(k), v = silu(v): S <- decay[head] S + k v^T; o = S^T q. q, k (heads of dim
-// channels) and v (heads of vdim) float32 rows `stride` apart; state float32 [slots][heads][dim][vdim], read at a segment's
-// start, written at its end; out float32 [rows][heads * vdim].
-int fw_decay_recurrence(const float* q, const float* k, const float* v, int stride, const float* decay, float* state, int slots,
+// Per segment and head, with q = silu(q), k = silu(k), v = silu(v): S <- decay S + k v^T; o = S^T q. q, k (heads of dim
+// channels) and v (heads of vdim) float32 rows `stride` apart; powers [heads][chunk + 1]: decay^0 .. decay^chunk of every head,
+// chunk = fw_decay_chunk_rows(); state float32 [slots][heads][dim][vdim], read at a segment's start, written at its end; out
+// float32 [rows][heads * vdim]. Segments of more than long_rows rows can be walked in chunks side by side on the matrix cores
+// (float32; the sums differ from the walk in order by rounding alone): chunk_seg / chunk_row0 [chunks] name every such
+// segment's chunks, side by side and in order, seg_chunk0 [segments + 1] where each segment's begin (an empty range for a short
+// one), workspace holds chunks * heads * dim * vdim floats. chunks 0: everything in order.
+int fw_decay_chunk_rows(void);
+int fw_decay_recurrence(const float* q, const float* k, const float* v, int stride, const float* powers, float* state, int slots,
                         float* out, const int32_t* seg_row0, const int32_t* seg_slot, int rows, int segments, int heads, int dim, int vdim,
-                        void* stream);
+                        const int32_t* chunk_seg, const int32_t* chunk_row0, const int32_t* seg_chunk0, int chunks, int long_rows,
+                        float* workspace, void* stream);
 
 // ---- the selective scan ---------------------------------------------------------------------------------------------
 // Per segment, channel c and state n, with dt = softplus(z[c]): S <- 2^(dt A2[n][c]) S + dt x[c] B[n]; y = sum_n S C[n] +
 // D[c] x[c]; out[c] = y * silu(gate[c]). bc rows: B's `states` values, then C's. All inputs float32 (rows apart by their
 // strides); A2 [states][channels] (A times log2 e), state float32 [slots][states][channels]; out [rows][channels] of out_dtype.
+// Chunks of fw_scan_chunk_rows() rows as for fw_decay_recurrence; workspace: chunks * (states + 1) * channels floats.
+int fw_scan_chunk_rows(void);
 int fw_selective_scan(const float* x, int x_stride, const float* z, int z_stride, const float* bc, int bc_stride, const float* gate,
                       int gate_stride, const float* A2, const float* D, float* state, int slots, void* out, int out_dtype,
-                      const int32_t* seg_row0, const int32_t* seg_slot, int rows, int segments, int channels, int states, void* stream);
+                      const int32_t* seg_row0, const int32_t* seg_slot, int rows, int segments, int channels, int states,
+                      const int32_t* chunk_seg, const int32_t* chunk_row0, const int32_t* seg_chunk0, int chunks, int long_rows,
+                      float* workspace, void* stream);
+// The same for segments of one row each (row r is segment r), with the map in front of the step sizes: z[c] = sum_j low[j]
+// w[j][c] + bias[c]. low rows: `rank` numbers, then B's `states` values, then C's. w float32 [rank][channels], or bfloat16 with
+// two neighbouring ranks of a channel side by side, [rank / 2][channels][2] (rank even).
+int fw_selective_scan_low_rank(const float* x, int x_stride, const float* low, int low_stride, int rank, const void* w, int w_dtype,
+                               const float* bias, const float* gate, int gate_stride, const float* A2, const float* D, float* state,
+                               int slots, void* out, int out_dtype, const int32_t* seg_slot, int rows, int channels, int states,
+                               void* stream);
 
 #ifdef __cplusplus
 }

@@ -43,6 +43,52 @@ __global__ __launch_bounds__(256) void causal_conv_rows_kernel(
     if (c >= echo_col0 && c < echo_col0 + echo_cols) out[(size_t)row * out_stride + echo_to + (c - echo_col0)] = sum;
 }
 
+// The same for few taps and many rows: a thread walks CONV_RUN rows of one channel, each input read once for all the taps that
+// meet it. Rows belong to segments as they may: which one is the same for all threads of a workgroup.
+#define CONV_RUN 16
+template <int L>
+__global__ __launch_bounds__(256) void causal_conv_run_kernel(
+    const float* __restrict__ in, int in_stride, const float* __restrict__ taps, const float* __restrict__ bias,
+    const float* __restrict__ state, const int32_t* __restrict__ row_seg, const int32_t* __restrict__ seg_row0,
+    const int32_t* __restrict__ seg_slot, float* __restrict__ out, int out_stride, int silu, bf16_t* __restrict__ rounded, int rows,
+    int channels) {
+    const int c = blockIdx.y * blockDim.x + threadIdx.x;
+    const int row0 = blockIdx.x * CONV_RUN;
+    if (c >= channels) return;
+    float x[CONV_RUN + L - 1], tap[L];
+#pragma unroll
+    for (int i = 0; i < CONV_RUN + L - 1; ++i) {
+        int t = row0 - (L - 1) + i;
+        t = t < 0 ? 0 : (t < rows ? t : rows - 1);
+        x[i] = in[(size_t)t * in_stride + c];
+    }
+#pragma unroll
+    for (int j = 0; j < L; ++j) tap[j] = taps[(size_t)c * L + j];
+    const float start = bias ? bias[c] : 0.0f;
+#pragma unroll
+    for (int u = 0; u < CONV_RUN; ++u) {
+        const int row = row0 + u;
+        if (row >= rows) break;
+        const int seg = row_seg[row];
+        const int back = row - seg_row0[seg];           // rows of this step ahead of it
+        float sum = start;
+        if (back >= L - 1) {
+#pragma unroll
+            for (int j = 0; j < L; ++j) sum = fmaf(tap[j], x[u + j], sum);
+        } else {
+            const float* remembered = state + ((size_t)seg_slot[seg] * channels + c) * (L - 1);
+#pragma unroll
+            for (int j = 0; j < L; ++j) {
+                const int ago = L - 1 - j;
+                sum = fmaf(tap[j], ago <= back ? x[u + j] : remembered[j + back], sum);
+            }
+        }
+        sum = conv_act(sum, silu);
+        out[(size_t)row * out_stride + c] = sum;
+        if (rounded) rounded[(size_t)row * channels + c] = float_to_bf16(sum);
+    }
+}
+
 // The slots move on: a thread per (segment, channel) reads what it needs (the segment's last L - 1 inputs, of
 // which the slot's own newest ones stand in for rows the segment does not have) and then writes.
 __global__ __launch_bounds__(256) void causal_conv_state_kernel(
@@ -120,9 +166,18 @@ extern "C" int fw_causal_conv(const float* in, int in_stride, const float* taps,
         FW_LAUNCH_CHECK("causal_conv");
         return 0;
     }
-    causal_conv_rows_kernel<<<dim3(rows, across), 256, 0, s>>>(in, in_stride, taps, bias, state, row_seg, seg_row0, seg_slot, out,
-                                                               out_stride, echo_col0, echo_cols, echo_to, silu, (bf16_t*)rounded, rows, channels,
-                                                               taps_count);
+    const dim3 runs(fw_ceil_div(rows, CONV_RUN), across);
+#define FW_CONV_RUN(L)                                                                                                                      \
+    causal_conv_run_kernel<L><<<runs, 256, 0, s>>>(in, in_stride, taps, bias, state, row_seg, seg_row0, seg_slot, out, out_stride, silu, \
+                                                   (bf16_t*)rounded, rows, channels)
+    const bool by_runs = echo_cols == 0 && taps_count >= 2 && taps_count <= 4 && rows >= 256;
+    if (by_runs && taps_count == 2) FW_CONV_RUN(2);
+    else if (by_runs && taps_count == 3) FW_CONV_RUN(3);
+    else if (by_runs) FW_CONV_RUN(4);
+    else
+        causal_conv_rows_kernel<<<dim3(rows, across), 256, 0, s>>>(in, in_stride, taps, bias, state, row_seg, seg_row0, seg_slot, out, out_stride,
+                                                                   echo_col0, echo_cols, echo_to, silu, (bf16_t*)rounded, rows, channels, taps_count);
+#undef FW_CONV_RUN
     FW_LAUNCH_CHECK("causal_conv");
     if (taps_count > 1) {
         causal_conv_state_kernel<<<dim3(segments, across), 256, 0, s>>>(in, in_stride, state, seg_row0, seg_slot, channels, taps_count);

@@ -1962,12 +1962,39 @@ def _segments(name: str, segments: int, seg_row0: torch.Tensor, seg_slot: torch.
 MAX_DECAY_DIM = 256      # key channels of a head
 
 
-def decay_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, seg_row0: torch.Tensor,
-                     seg_slot: torch.Tensor, segments: int, heads: int, dim: int, vdim: int) -> torch.Tensor:
+def _chunks(name: str, chunks: Optional[tuple], segments: int):
+    """(chunk_seg, chunk_row0, seg_chunk0, rows from which a segment is walked in chunks) -> the arguments of a launch, their
+    number."""
+    if chunks is None:
+        return (None, None, None), 0, 0
+    chunk_seg, chunk_row0, seg_chunk0, long_rows = chunks
+    _dev(chunk_seg, chunk_row0, seg_chunk0)
+    count = chunk_seg.numel()
+    for which, t, n in (("chunk_seg", chunk_seg, count), ("chunk_row0", chunk_row0, count), ("seg_chunk0", seg_chunk0, segments + 1)):
+        _want(t, torch.int32, which)
+        if t.numel() < n:
+            raise KernelError(f"{name}: {which} holds {t.numel()} entries, needs {n}")
+    return (chunk_seg, chunk_row0, seg_chunk0), count, int(long_rows)
+
+
+DECAY_CHUNK = 64        # rows of a chunk, as the kernels have them
+
+
+def decay_powers(decays, device) -> torch.Tensor:
+    """decay^0 .. decay^chunk of every head, formed in float64: float32 [heads, chunk + 1]."""
+    if library().fw_decay_chunk_rows() != DECAY_CHUNK or library().fw_scan_chunk_rows() != DECAY_CHUNK:
+        raise KernelError("the kernel library's chunks are of another length")
+    exponents = torch.arange(DECAY_CHUNK + 1, dtype=torch.float64)
+    return torch.pow(torch.as_tensor(decays, dtype=torch.float64)[:, None], exponents[None, :]).to(dtype=torch.float32, device=device)
+
+
+def decay_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, powers: torch.Tensor, state: torch.Tensor, seg_row0: torch.Tensor,
+                     seg_slot: torch.Tensor, segments: int, heads: int, dim: int, vdim: int, chunks: Optional[tuple] = None) -> torch.Tensor:
     """Per head S <- decay S + silu(k) silu(v)^T, o = S^T silu(q) over each segment's rows in order. ``q``, ``k`` float32
-    [rows, heads dim] and ``v`` [rows, heads vdim] with one row stride (views of wider rows will do); ``decay`` float32 [heads];
-    ``state`` float32 [slots, heads, dim, vdim] is read and moved on. Returns float32 [rows, heads vdim]."""
-    _dev(decay, state)
+    [rows, heads dim] and ``v`` [rows, heads vdim] with one row stride (views of wider rows will do); ``powers``: see
+    ``decay_powers``; ``state`` float32 [slots, heads, dim, vdim] is read and moved on. ``chunks`` (chunk_seg, chunk_row0, seg_chunk0,
+    long_rows): segments of more than long_rows rows are walked in these chunks side by side. Returns float32 [rows, heads vdim]."""
+    _dev(powers, state)
     _segments("decay_recurrence", segments, seg_row0, seg_slot)
     rows = q.shape[0]
     for name, t, width in (("q", q, heads * dim), ("k", k, heads * dim), ("v", v, heads * vdim)):
@@ -1978,13 +2005,16 @@ def decay_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: t
     if rows > 1 and not (q.stride(0) == k.stride(0) == v.stride(0)):
         raise KernelError("decay_recurrence: q, k and v have one row stride")
     stride = max(_stride(q), _stride(k), _stride(v))
-    for name, t, shape in (("decay", decay, (heads,)), ("state", state[0], (heads, dim, vdim))):
+    for name, t, shape in (("powers", powers, (heads, DECAY_CHUNK + 1)), ("state", state[0], (heads, dim, vdim))):
         _want(t, torch.float32, name)
         if t.shape != shape:
             raise KernelError(f"decay_recurrence: {name} is {tuple(t.shape)}, expected {shape}")
     out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=q.device)
-    _check(library().fw_decay_recurrence(_p(q), _p(k), _p(v), stride, _p(decay), _p(state), state.shape[0], _p(out), _p(seg_row0),
-                                         _p(seg_slot), rows, int(segments), heads, dim, vdim, _stream()))
+    places, count, long_rows = _chunks("decay_recurrence", chunks, segments)
+    workspace = torch.empty((count, heads, dim, vdim), dtype=torch.float32, device=q.device) if count else None
+    _check(library().fw_decay_recurrence(_p(q), _p(k), _p(v), stride, _p(powers), _p(state), state.shape[0], _p(out), _p(seg_row0),
+                                         _p(seg_slot), rows, int(segments), heads, dim, vdim, *(_p(t) for t in places), count, long_rows,
+                                         _p(workspace), _stream()))
     return out
 
 
@@ -1993,11 +2023,12 @@ MAX_SCAN_STATES = 128
 
 
 def selective_scan(x: torch.Tensor, z: torch.Tensor, bc: torch.Tensor, gate: torch.Tensor, A2: torch.Tensor, D: torch.Tensor,
-                   state: torch.Tensor, seg_row0: torch.Tensor, seg_slot: torch.Tensor, segments: int, out_dtype: torch.dtype) -> torch.Tensor:
+                   state: torch.Tensor, seg_row0: torch.Tensor, seg_slot: torch.Tensor, segments: int, out_dtype: torch.dtype,
+                   chunks: Optional[tuple] = None) -> torch.Tensor:
     """Per channel c and state n, with dt = softplus(z): S <- 2^(dt A2[n, c]) S + dt x B[n], y = sum_n S C[n] + D x, out = y *
     silu(gate), over each segment's rows in order. ``x``, ``z``, ``gate`` float32 [rows, channels], ``bc`` float32 [rows, 2 states]
     (B, then C); rows may lie apart. ``A2`` [states, channels] and ``D`` [channels] float32; ``state`` float32 [slots, states,
-    channels] is read and moved on. Returns [rows, channels] of ``out_dtype``."""
+    channels] is read and moved on. ``chunks``: as for ``decay_recurrence``. Returns [rows, channels] of ``out_dtype``."""
     _dev(A2, D, state)
     _segments("selective_scan", segments, seg_row0, seg_slot)
     rows, channels = x.shape
@@ -2012,7 +2043,46 @@ def selective_scan(x: torch.Tensor, z: torch.Tensor, bc: torch.Tensor, gate: tor
         if t.shape != shape:
             raise KernelError(f"selective_scan: {name} is {tuple(t.shape)}, expected {shape}")
     out = torch.empty((rows, channels), dtype=out_dtype, device=x.device)
+    places, count, long_rows = _chunks("selective_scan", chunks, segments)
+    workspace = torch.empty((count, states + 1, channels), dtype=torch.float32, device=x.device) if count else None
     _check(library().fw_selective_scan(_p(x), _stride(x), _p(z), _stride(z), _p(bc), _stride(bc), _p(gate), _stride(gate), _p(A2), _p(D), _p(state),
                                        state.shape[0], _p(out), _code(out_dtype), _p(seg_row0), _p(seg_slot), rows, int(segments), channels,
-                                       states, _stream()))
+                                       states, *(_p(t) for t in places), count, long_rows, _p(workspace), _stream()))
+    return out
+
+
+def low_rank_weights(w: torch.Tensor) -> torch.Tensor:
+    """A map [channels, rank] as ``selective_scan_low_rank`` reads it: [rank, channels], or of bfloat16 [rank / 2, channels, 2]."""
+    channels, rank = w.shape
+    if w.dtype == torch.bfloat16 and rank % 2 == 0:
+        return w.view(channels, rank // 2, 2).permute(1, 0, 2).contiguous()
+    return w.to(torch.float32).t().contiguous()
+
+
+def selective_scan_low_rank(x: torch.Tensor, low: torch.Tensor, w: torch.Tensor, bias: torch.Tensor, gate: torch.Tensor, A2: torch.Tensor,
+                            D: torch.Tensor, state: torch.Tensor, seg_slot: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """``selective_scan`` over segments of one row each (row r is segment r), with the map in front of the step sizes: z = low[:,
+    :rank] . W^T + bias. ``low`` float32 [rows, rank + 2 states] (the low part, B, C; rows may lie apart); ``w`` from
+    ``low_rank_weights``."""
+    _dev(A2, D, state, w, bias, seg_slot)
+    _want(seg_slot, torch.int32, "seg_slot")
+    rows, channels = x.shape
+    states = A2.shape[0]
+    rank = w.shape[0] * (2 if w.dim() == 3 else 1)
+    for name, t, shape in (("x", x, (rows, channels)), ("low", low, (rows, rank + 2 * states)), ("gate", gate, (rows, channels))):
+        _dev_rows(t, name)
+        _want(t, torch.float32, name)
+        if t.shape != shape:
+            raise KernelError(f"selective_scan_low_rank: {name} is {tuple(t.shape)}, expected {shape}")
+    for name, t, shape in (("A2", A2, (states, channels)), ("D", D, (channels,)), ("bias", bias, (channels,)), ("state", state[0], (states, channels))):
+        _want(t, torch.float32, name)
+        if t.shape != shape:
+            raise KernelError(f"selective_scan_low_rank: {name} is {tuple(t.shape)}, expected {shape}")
+    if w.shape != ((rank // 2, channels, 2) if w.dim() == 3 else (rank, channels)) or w.dtype != (torch.bfloat16 if w.dim() == 3 else torch.float32) \
+            or seg_slot.numel() < rows:
+        raise KernelError(f"selective_scan_low_rank: w is {tuple(w.shape)} {w.dtype}, {seg_slot.numel()} slots for {rows} rows")
+    out = torch.empty((rows, channels), dtype=out_dtype, device=x.device)
+    _check(library().fw_selective_scan_low_rank(_p(x), _stride(x), _p(low), _stride(low), rank, _p(w), _code(w.dtype), _p(bias), _p(gate),
+                                                _stride(gate), _p(A2), _p(D), _p(state), state.shape[0], _p(out), _code(out_dtype),
+                                                _p(seg_slot), rows, channels, states, _stream()))
     return out

@@ -20,13 +20,14 @@ from ..config.spec import ConfigError
 from ..kernels import ops
 from ..weights.loader import TensorDecl
 from .base import Mixer, register_mixer
+from .chunks import RecurrenceChunks
 from .linear import Linear
 
 _DEFAULT_NAMES = {"q": "q", "k": "k", "v": "v", "g": "g", "norm": "norm", "o": "o"}
 
 
 @register_mixer("lightning")
-class LightningAttention(Mixer):
+class LightningAttention(RecurrenceChunks, Mixer):
     graph_safe = True
 
     def __init__(self, spec):
@@ -65,14 +66,14 @@ class LightningAttention(Mixer):
         self.in_proj = Linear(torch.cat([tensors[self._name(n)] for n in ("q", "k", "v", "g")], dim=0))
         self.out = Linear(tensors[self._name("o")])
         self.norm_weight = tensors[self._name("norm")]
-        self.decay = torch.tensor(self.decays, dtype=torch.float64).to(dtype=torch.float32, device=device)
+        self.powers = ops.decay_powers(self.decays, device)
 
     def heads_output(self, h, ctx, cache) -> torch.Tensor:
         """The heads' normed and gated read-outs [rows, heads * vdim] in the activation dtype; the request's state moves on."""
         proj = self.in_proj.forward(h, out_dtype=torch.float32)
         qk, vw = self.heads * self.dim, self.heads * self.vdim
-        o = ops.decay_recurrence(proj[:, :qk], proj[:, qk:2 * qk], proj[:, 2 * qk:2 * qk + vw], self.decay, cache["state"].state,
-                                 ctx.seg_row0, ctx.seg_slot, ctx.num_segments, self.heads, self.dim, self.vdim)
+        o = ops.decay_recurrence(proj[:, :qk], proj[:, qk:2 * qk], proj[:, 2 * qk:2 * qk + vw], self.powers, cache["state"].state,
+                                 ctx.seg_row0, ctx.seg_slot, ctx.num_segments, self.heads, self.dim, self.vdim, **self.chunk_arguments(ctx))
         return ops.gated_head_norm(o, proj[:, 2 * qk + vw:], self.norm_weight, 1, vw, self.eps, self.dtype)
 
     def output(self, h, ctx, cache) -> torch.Tensor:

@@ -8,7 +8,7 @@ from S = 0:
 
 and out = W_o (y * silu(z)). A request's slot keeps S (float32 [state, inner]) and the convolution's last taps - 1 inputs.
 The convolution, the step sizes, the decays and the state are float32 in either run dtype; x is rounded for W_x, the low
-part for W_dt, and y * silu(z) for W_o.
+part for W_dt (not in steps of a few single rows, whose scan forms that map itself), and y * silu(z) for W_o.
 """
 
 from __future__ import annotations
@@ -23,6 +23,7 @@ from ..config.spec import ConfigError
 from ..kernels import ops
 from ..weights.loader import TensorDecl
 from .base import Mixer, register_mixer
+from .chunks import RecurrenceChunks
 from .linear import Linear
 
 _DEFAULT_NAMES = {"in": "in", "conv": "conv", "conv_bias": "conv.b", "x": "x", "dt": "dt", "dt_bias": "dt.b", "A_log": "A_log", "D": "D",
@@ -30,8 +31,10 @@ _DEFAULT_NAMES = {"in": "in", "conv": "conv", "conv_bias": "conv.b", "x": "x", "
 
 
 @register_mixer("mamba")
-class Mamba(Mixer):
+class Mamba(RecurrenceChunks, Mixer):
     graph_safe = True
+    # up to so many single rows the scan forms the step sizes' map itself: two launches fewer, but every row reads the map
+    LOW_RANK_ROWS = 16
 
     def __init__(self, spec):
         super().__init__(spec)
@@ -59,6 +62,10 @@ class Mamba(Mixer):
         """The convolution, and per channel and state the decay's exponential and product, the write and the read."""
         return rows * self.inner * (2 * self.taps_count + 7 * self.states + 8)
 
+    def gathered_tensors(self):
+        """The step sizes' map in its second layout: a step reads one of the two (counted once)."""
+        return (self.low_rank,)
+
     def tensors(self) -> Dict[str, TensorDecl]:
         D, C, N, R = self.hidden, self.inner, self.states, self.rank
         return {
@@ -76,6 +83,8 @@ class Mamba(Mixer):
         self.in_proj = Linear(t["in"])
         self.x_proj = Linear(t["x"])
         self.dt_proj = Linear(t["dt"], t["dt_bias"])
+        self.low_rank = ops.low_rank_weights(t["dt"])
+        self.dt_bias = t["dt_bias"]
         self.out = Linear(t["o"])
         self.taps, self.conv_bias, self.D = t["conv"], t["conv_bias"], t["D"]
         # exp(dt A) is taken as 2^(dt A log2 e); a state's row holds all channels
@@ -98,11 +107,14 @@ class Mamba(Mixer):
                             ctx.seg_slot, ctx.num_segments, single_rows=ctx.all_decode, silu=True, rounded=short)
         x, rounded = x if short else (x, x)
         low = self.x_proj.forward(rounded, out_dtype=torch.float32)
+        if ctx.all_decode and ctx.num_rows <= self.LOW_RANK_ROWS:
+            return ops.selective_scan_low_rank(x, low, self.low_rank, self.dt_bias, both[:, self.inner:], self.A2, self.D, cache["state"].state,
+                                               ctx.seg_slot, self.dtype)
         rank = torch.empty((low.shape[0], self.rank), dtype=self.dtype, device=low.device)
         ops.place_rows(low[:, :self.rank], rank)
         z = self.dt_proj.forward(rank, out_dtype=torch.float32)
         return ops.selective_scan(x, z, low[:, self.rank:], both[:, self.inner:], self.A2, self.D, cache["state"].state, ctx.seg_row0,
-                                  ctx.seg_slot, ctx.num_segments, self.dtype)
+                                  ctx.seg_slot, ctx.num_segments, self.dtype, **self.chunk_arguments(ctx))
 
     def output(self, h, ctx, cache) -> torch.Tensor:
         return self.out.forward(self.scanned(h, ctx, cache), out_dtype=torch.float32)
