@@ -95,8 +95,6 @@ __global__ __launch_bounds__(256) void decay_recurrence_step_kernel(
 typedef __attribute__((ext_vector_type(16))) float dr_f32x16;
 typedef __attribute__((ext_vector_type(4))) float dr_f32x4;
 
-__device__ __forceinline__ float dr_silu_quick(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
-
 __device__ __forceinline__ dr_f32x16 dr_zero() {
     dr_f32x16 acc;
 #pragma unroll
@@ -123,7 +121,7 @@ __global__ __launch_bounds__(256, 2) void decay_chunk_sum_kernel(const float* __
         const int token = i / dp, c = i % dp;
         const bool there = token < tokens && c < dim;
         const float z = k[(size_t)(row0 + (there ? token : 0)) * stride + (size_t)head * dim + (there ? c : 0)];
-        lds[i] = there ? dr_silu_quick(z) * p[tokens - 1 - token] : 0.0f;
+        lds[i] = there ? dr_silu(z) * p[tokens - 1 - token] : 0.0f;
     }
     __syncthreads();
     float* to = local + ((size_t)chunk * heads + head) * dim * vdim;
@@ -137,7 +135,7 @@ __global__ __launch_bounds__(256, 2) void decay_chunk_sum_kernel(const float* __
             value[t] = from[(size_t)(token < tokens ? token : tokens - 1) * stride];
         }
 #pragma unroll
-        for (int t = 0; t < DR_CHUNK / 2; ++t) value[t] = dr_silu_quick(value[t]);      // (a row past the chunk's end meets k = 0)
+        for (int t = 0; t < DR_CHUNK / 2; ++t) value[t] = dr_silu(value[t]);      // (a row past the chunk's end meets k = 0)
         for (int key0 = 0; key0 < dp; key0 += 128) {
             const int tiles = (dp - key0) / 32 < 4 ? (dp - key0) / 32 : 4;
             dr_f32x16 acc[4];
@@ -216,8 +214,8 @@ __global__ __launch_bounds__(256, 2) void decay_chunk_read_kernel(const float* _
         const bool there = token < tokens && c < dim;
         const size_t at = (size_t)(row0 + (there ? token : 0)) * stride + (size_t)head * dim + (there ? c : 0);
         const float zq = q[at], zk = k[at];
-        lq[token * pitch + c] = there ? dr_silu_quick(zq) : 0.0f;
-        lk[token * pitch + c] = there ? dr_silu_quick(zk) : 0.0f;
+        lq[token * pitch + c] = there ? dr_silu(zq) : 0.0f;
+        lk[token * pitch + c] = there ? dr_silu(zk) : 0.0f;
     }
     __syncthreads();
     // scores: a 32 x 32 tile a wave; the tile above the diagonal is zero
@@ -274,7 +272,7 @@ __global__ __launch_bounds__(256, 2) void decay_chunk_read_kernel(const float* _
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const int token = t + 4 * half + e;
-                b[e] = dr_silu_quick(from[(size_t)(token < tokens ? token : tokens - 1) * stride]);     // (its scores are zero)
+                b[e] = dr_silu(from[(size_t)(token < tokens ? token : tokens - 1) * stride]);     // (its scores are zero)
             }
             const dr_f32x4 a1 = *reinterpret_cast<const dr_f32x4*>(ls + (32 + within) * SCORES + t + 4 * half);
             if (t < 32) {

@@ -15,13 +15,13 @@
 // softplus(x) = ln(1 + e^x). The logarithm of the rounded u = 1 + e is corrected by e / (u - 1), which is exact to the last
 // digits however small e is; beyond 20 e^-x no longer shows.
 __device__ __forceinline__ float ss_softplus(float x) {
-    const float e = __builtin_amdgcn_exp2f(x * 1.4426950408889634f);
+    const float e = expf(x);
     const float u = 1.0f + e, d = u - 1.0f;
     const float ln = __builtin_amdgcn_logf(u) * 0.69314718055994531f;
-    const float corrected = d == 0.0f ? e : ln * (e * __builtin_amdgcn_rcpf(d));
+    const float corrected = d == 0.0f ? e : ln * (e / d);
     return x > 20.0f ? x : corrected;
 }
-__device__ __forceinline__ float ss_silu(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)); }
+__device__ __forceinline__ float ss_silu(float z) { return z / (1.0f + expf(-z)); }
 
 // A run of rows row0 .. row0 + count - 1 for one channel a lane: S moves on; with OUT the outputs are formed, else the steps' sum
 // is. All lanes of the workgroup (one wave) call it together: they share the staged B and C.
