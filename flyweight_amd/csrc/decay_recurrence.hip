@@ -95,6 +95,36 @@ __global__ __launch_bounds__(256) void decay_recurrence_step_kernel(
 typedef __attribute__((ext_vector_type(16))) float dr_f32x16;
 typedef __attribute__((ext_vector_type(4))) float dr_f32x4;
 
+__device__ __forceinline__ float dr_silu_quick(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
+
+// Copies a chunk's rows of one head's q and k (or k alone: q null) into LDS rows `pitch` apart, silu applied; what lies past the
+// chunk's last row, and past dim up to `width`, is zero. 256 threads; eight elements of each are asked for before any is used.
+template <bool BOTH>
+__device__ __forceinline__ void dr_stage(const float* __restrict__ q, const float* __restrict__ k, int stride, int tokens, int dim, int width,
+                                         int pitch, float* lq, float* lk, const float* weight) {
+    const int shift = width <= 32 ? 5 : width <= 64 ? 6 : width <= 128 ? 7 : 8;     // columns are numbered in a power of two
+    for (int base = threadIdx.x; base < (DR_CHUNK << shift); base += 256 * 8) {
+        float zq[8], zk[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int i = base + 256 * u;
+            const int token = i >> shift, c = i & ((1 << shift) - 1);
+            const int at = (token < tokens ? token : tokens - 1) * stride + (c < dim ? c : dim - 1);
+            if (BOTH) zq[u] = q[at];
+            zk[u] = k[at];
+        }
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int i = base + 256 * u;
+            const int token = i >> shift, c = i & ((1 << shift) - 1);
+            if (token >= DR_CHUNK || c >= width) continue;
+            const bool there = token < tokens && c < dim;
+            if (BOTH) lq[token * pitch + c] = there ? dr_silu_quick(zq[u]) : 0.0f;
+            lk[token * pitch + c] = there ? dr_silu_quick(zk[u]) * (weight ? weight[tokens - 1 - token] : 1.0f) : 0.0f;
+        }
+    }
+}
+
 __device__ __forceinline__ dr_f32x16 dr_zero() {
     dr_f32x16 acc;
 #pragma unroll
@@ -117,12 +147,7 @@ __global__ __launch_bounds__(256, 2) void decay_chunk_sum_kernel(const float* __
     const int dp = (dim + 31) & ~31;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, half = lane >> 5, column = lane & 31;
     const float* p = powers + head * (DR_CHUNK + 1);
-    for (int i = threadIdx.x; i < DR_CHUNK * dp; i += 256) {
-        const int token = i / dp, c = i % dp;
-        const bool there = token < tokens && c < dim;
-        const float z = k[(size_t)(row0 + (there ? token : 0)) * stride + (size_t)head * dim + (there ? c : 0)];
-        lds[i] = there ? dr_silu(z) * p[tokens - 1 - token] : 0.0f;
-    }
+    dr_stage<false>(nullptr, k + (size_t)row0 * stride + (size_t)head * dim, stride, tokens, dim, dp, dp, nullptr, lds, p);
     __syncthreads();
     float* to = local + ((size_t)chunk * heads + head) * dim * vdim;
     for (int col0 = wave * 32; col0 < vdim; col0 += 128) {
@@ -135,7 +160,7 @@ __global__ __launch_bounds__(256, 2) void decay_chunk_sum_kernel(const float* __
             value[t] = from[(size_t)(token < tokens ? token : tokens - 1) * stride];
         }
 #pragma unroll
-        for (int t = 0; t < DR_CHUNK / 2; ++t) value[t] = dr_silu(value[t]);      // (a row past the chunk's end meets k = 0)
+        for (int t = 0; t < DR_CHUNK / 2; ++t) value[t] = dr_silu_quick(value[t]);      // (a row past the chunk's end meets k = 0)
         for (int key0 = 0; key0 < dp; key0 += 128) {
             const int tiles = (dp - key0) / 32 < 4 ? (dp - key0) / 32 : 4;
             dr_f32x16 acc[4];
@@ -209,14 +234,8 @@ __global__ __launch_bounds__(256, 2) void decay_chunk_read_kernel(const float* _
     float* lk = lds + DR_CHUNK * pitch;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, half = lane >> 5, within = lane & 31;
     const float* p = powers + head * (DR_CHUNK + 1);
-    for (int i = threadIdx.x; i < DR_CHUNK * dp; i += 256) {
-        const int token = i / dp, c = i % dp;
-        const bool there = token < tokens && c < dim;
-        const size_t at = (size_t)(row0 + (there ? token : 0)) * stride + (size_t)head * dim + (there ? c : 0);
-        const float zq = q[at], zk = k[at];
-        lq[token * pitch + c] = there ? dr_silu(zq) : 0.0f;
-        lk[token * pitch + c] = there ? dr_silu(zk) : 0.0f;
-    }
+    const size_t at = (size_t)row0 * stride + (size_t)head * dim;
+    dr_stage<true>(q + at, k + at, stride, tokens, dim, dp, pitch, lq, lk, nullptr);
     __syncthreads();
     // scores: a 32 x 32 tile a wave; the tile above the diagonal is zero
     const int ti = wave >> 1, tj = wave & 1;
@@ -272,7 +291,7 @@ __global__ __launch_bounds__(256, 2) void decay_chunk_read_kernel(const float* _
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 const int token = t + 4 * half + e;
-                b[e] = dr_silu(from[(size_t)(token < tokens ? token : tokens - 1) * stride]);     // (its scores are zero)
+                b[e] = dr_silu_quick(from[(size_t)(token < tokens ? token : tokens - 1) * stride]);     // (its scores are zero)
             }
             const dr_f32x4 a1 = *reinterpret_cast<const dr_f32x4*>(ls + (32 + within) * SCORES + t + 4 * half);
             if (t < 32) {
@@ -299,26 +318,29 @@ extern "C" int fw_decay_chunk_rows(void) { return DR_CHUNK; }
 extern "C" int fw_decay_recurrence(const float* q, const float* k, const float* v, int stride, const float* powers, float* state, int slots,
                                    float* out, const int32_t* seg_row0, const int32_t* seg_slot, int rows, int segments, int heads, int dim,
                                    int vdim, const int32_t* chunk_seg, const int32_t* chunk_row0, const int32_t* seg_chunk0, int chunks,
-                                   int long_rows, float* workspace, void* stream) {
+                                   int long_rows, int all_long, float* workspace, void* stream) {
     FW_REQUIRE(rows >= 0 && segments >= 0 && heads > 0 && heads <= 65535 && slots > 0, "decay_recurrence: bad sizes rows=%d segments=%d heads=%d",
                rows, segments, heads);
     FW_REQUIRE(dim >= 1 && dim <= 256 && vdim >= 1 && vdim <= 65536, "decay_recurrence: heads of %d (1..256) and %d channels", dim, vdim);
+    FW_REQUIRE(stride <= 1 << 24, "decay_recurrence: rows of %d values", stride);
     FW_REQUIRE(stride >= heads * dim && stride >= heads * vdim, "decay_recurrence: rows of %d values do not hold %d heads of %d / %d", stride, heads, dim, vdim);
     FW_REQUIRE(chunks >= 0 && (chunks == 0 || (chunk_seg && chunk_row0 && seg_chunk0 && workspace && long_rows > 0)),
                "decay_recurrence: chunks come with their places, a workspace and the length from which they are used");
     if (rows == 0 || segments == 0) return 0;
     hipStream_t s = (hipStream_t)stream;
     const dim3 grid(segments, heads, fw_ceil_div(vdim, 64));
-#define FW_DECAY_LAUNCH(RPT)                                                                                                         \
-    decay_recurrence_step_kernel<RPT><<<grid, 256, 0, s>>>(q, k, v, stride, powers, state, out, seg_row0, seg_slot, heads, dim, vdim, \
-                                                           chunks > 0 ? long_rows : 0)
-    if (dim <= 16) FW_DECAY_LAUNCH(4);
-    else if (dim <= 32) FW_DECAY_LAUNCH(8);
-    else if (dim <= 64) FW_DECAY_LAUNCH(16);
-    else if (dim <= 128) FW_DECAY_LAUNCH(32);
-    else FW_DECAY_LAUNCH(64);
+    if (chunks == 0 || !all_long) {
+#define FW_DECAY_LAUNCH(RPT)                                                                                                             \
+        decay_recurrence_step_kernel<RPT><<<grid, 256, 0, s>>>(q, k, v, stride, powers, state, out, seg_row0, seg_slot, heads, dim, vdim, \
+                                                               chunks > 0 ? long_rows : 0)
+        if (dim <= 16) FW_DECAY_LAUNCH(4);
+        else if (dim <= 32) FW_DECAY_LAUNCH(8);
+        else if (dim <= 64) FW_DECAY_LAUNCH(16);
+        else if (dim <= 128) FW_DECAY_LAUNCH(32);
+        else FW_DECAY_LAUNCH(64);
 #undef FW_DECAY_LAUNCH
-    FW_LAUNCH_CHECK("decay_recurrence");
+        FW_LAUNCH_CHECK("decay_recurrence");
+    }
     if (chunks == 0) return 0;
     const int sum_bytes = DR_CHUNK * ((dim + 31) & ~31) * 4;
     const int read_width = ((dim + 7) & ~7) + 4;

@@ -37,6 +37,21 @@ __global__ void embed_rows_kernel(const W* __restrict__ table, const int32_t* __
     }
 }
 
+// Four values a thread, for rows that are written several times over (the kernel is bound by its stores then).
+__global__ __launch_bounds__(256) void embed_copies_kernel(const bf16_t* __restrict__ table, const int32_t* __restrict__ ids, float* __restrict__ out,
+                                                           int hidden, float scale, int copies) {
+    typedef __attribute__((ext_vector_type(4))) float f32x4;
+    typedef __attribute__((ext_vector_type(2))) uint32_t u32x2;
+    const int row = blockIdx.y;
+    const u32x2* source = reinterpret_cast<const u32x2*>(table + (size_t)ids[row] * hidden);
+    for (int i = blockIdx.x * blockDim.x + threadIdx.x; i < hidden / 4; i += gridDim.x * blockDim.x) {
+        const u32x2 v = source[i];
+        const f32x4 value = {bf16_bits_to_float(v[0] & 0xffffu) * scale, bf16_bits_to_float(v[0] >> 16) * scale,
+                             bf16_bits_to_float(v[1] & 0xffffu) * scale, bf16_bits_to_float(v[1] >> 16) * scale};
+        for (int copy = 0; copy < copies; ++copy) reinterpret_cast<f32x4*>(out + ((size_t)row * copies + copy) * hidden)[i] = value;
+    }
+}
+
 extern "C" int fw_embed_rows(const void* table, int table_dtype, const int32_t* ids, float* out,
                              int rows, int hidden, int vocab, float scale, const void* places_table, int places_dtype,
                              const int32_t* places, int places_entries, int copies, void* stream) {
@@ -47,6 +62,12 @@ extern "C" int fw_embed_rows(const void* table, int table_dtype, const int32_t* 
     if (rows == 0) return 0;
     dim3 grid(fw_ceil_div(hidden, 256) > 64 ? 64 : fw_ceil_div(hidden, 256), rows);
     hipStream_t s = (hipStream_t)stream;
+    if (places == nullptr && copies > 1 && table_dtype == FW_BF16 && hidden % 4 == 0 && (uintptr_t)table % 8 == 0 && (uintptr_t)out % 16 == 0) {
+        const dim3 by_four(fw_ceil_div(hidden, 1024) > 64 ? 64 : fw_ceil_div(hidden, 1024), rows);
+        embed_copies_kernel<<<by_four, 256, 0, s>>>((const bf16_t*)table, ids, out, hidden, scale, copies);
+        FW_LAUNCH_CHECK("embed_rows");
+        return 0;
+    }
     if (places == nullptr) places_dtype = table_dtype;
 #define FW_EMBED_LAUNCH(W, P) \
     embed_rows_kernel<W, P><<<grid, 256, 0, s>>>((const W*)table, ids, out, hidden, scale, (const P*)places_table, places, copies)

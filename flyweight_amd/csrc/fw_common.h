@@ -165,12 +165,19 @@ __device__ __forceinline__ float block_sum_by_lds(float v, float* scratch) {
     return ((scratch[0] + scratch[1]) + scratch[2]) + scratch[3];
 }
 
-// A gated unit behind a product that holds gate and up of one feature: silu(g) * u (limit <= 0), or
+// The tanh form of gelu, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), is z * sigmoid of this
+// (0.5 (1 + tanh(y)) = sigmoid(2 y)).
+__device__ __forceinline__ float fw_gelu_tanh_argument(float z) { return 1.5957691216057308f * z * fmaf(0.044715f * z, z, 1.0f); }
+// ... for results that are rounded to bfloat16
+__device__ __forceinline__ float fw_gelu_tanh_quick(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-fw_gelu_tanh_argument(z))); }
+
+// A gated unit behind a product that holds gate and up of one feature: silu(g) * u (limit 0), gelu_tanh(g) * u (limit < 0), or
 // with clamped halves g' = min(g, limit), u' = clamp(u, -limit, limit): g' * sigmoid(alpha g') * (u' + shift).
 // `silu` is the product's own form of silu(g) * u, so that the plain unit's results stay what they were.
 template <typename Silu>
 __device__ __forceinline__ float fw_gated_unit(float g, float u, float limit, float alpha, float shift, Silu silu) {
-    if (limit <= 0.0f) return silu(g) * u;
+    if (limit < 0.0f) return fw_gelu_tanh_quick(g) * u;
+    if (limit == 0.0f) return silu(g) * u;
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
     const float z = alpha * g;
@@ -180,10 +187,6 @@ __device__ __forceinline__ float fw_gated_unit(float g, float u, float limit, fl
 
 // z Phi(z), Phi the normal distribution's cumulative function: the exact gelu
 __device__ __forceinline__ float fw_gelu(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
-
-// The tanh form of gelu, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), is z * sigmoid of this
-// (0.5 (1 + tanh(y)) = sigmoid(2 y)).
-__device__ __forceinline__ float fw_gelu_tanh_argument(float z) { return 1.5957691216057308f * z * fmaf(0.044715f * z, z, 1.0f); }
 
 // The exact gelu for results that are rounded to bfloat16: the complement of the error function as a polynomial in 1 / (1 + p x)
 // times e^(-x^2) (Abramowitz and Stegun, Handbook of Mathematical Functions, 7.1.26: within 1.5e-7), which gives the
@@ -212,6 +215,23 @@ template <> __device__ __forceinline__ void store_from_float<gelu_bf16_t>(gelu_b
 // what a store of this output type does to a float32 sum before it is rounded (for stores that pack several values)
 template <typename T> __device__ __forceinline__ float fw_before_store(float v) { return v; }
 template <> __device__ __forceinline__ float fw_before_store<gelu_bf16_t>(float v) { return fw_gelu_quick(v); }
+
+// The gated product (gate rows, then up rows) with this output type (dtype code FW_BF16_GEGLU) stores gelu_tanh(gate) * up in
+// bfloat16 in place of silu(gate) * up.
+#define FW_BF16_GEGLU 3
+struct geglu_bf16_t {
+    uint16_t bits;
+};
+template <> __device__ __forceinline__ void store_from_float<geglu_bf16_t>(geglu_bf16_t* p, size_t i, float v) { p[i].bits = float_to_bf16_bits(v); }
+template <> __device__ __forceinline__ float load_as_float<geglu_bf16_t>(const geglu_bf16_t* p, size_t i) { return bf16_bits_to_float(p[i].bits); }
+// what the gate passes, by the output's type; `silu` is the product's own form of silu
+template <typename T, typename Silu> struct fw_gate {
+    static __device__ __forceinline__ float of(float g, Silu silu) { return silu(g); }
+};
+template <typename Silu> struct fw_gate<geglu_bf16_t, Silu> {
+    static __device__ __forceinline__ float of(float g, Silu) { return fw_gelu_tanh_quick(g); }
+};
+template <typename T, typename Silu> __device__ __forceinline__ float fw_gate_of(float g, Silu silu) { return fw_gate<T, Silu>::of(g, silu); }
 
 // The first key that a row at position `pos` may see: with a window the last `window` keys (itself
 // among them), with a chunk only the keys of its own chunk (chunks counted from position 0 of the

@@ -39,7 +39,7 @@ int fw_gemm_generic(const void* a, int a_dtype, const void* w, int w_dtype, cons
 // multiple of 8. mode 0: out = a . w^T (+ bias) stored as out_dtype (also 2, here and in every storing product below:
 // gelu(a . w^T (+ bias)), the error-function form, in bfloat16); mode 1: out (float32) +=
 // a . w^T (+ bias); mode 2 (SwiGLU): w is [2N][K], gate rows then up rows, out [M][N] bfloat16 =
-// silu(a . gate^T) * (a . up^T). fw_gemm_skinny streams w once for M <= 64 (decode);
+// silu(a . gate^T) * (a . up^T), or with out_dtype 3 gelu_tanh(a . gate^T) * (a . up^T). fw_gemm_skinny streams w once for M <= 64 (decode);
 // fw_gemm_mfma tiles both operands through LDS (prompts).
 int fw_gemm_skinny(const void* a, const void* w, const float* bias, void* out, int out_dtype, int mode,
                    int M, int N, int K, void* stream);
@@ -91,8 +91,8 @@ int fw_gemm_medium(const void* a, const void* w, int w_tiled, const float* bias,
 // [M][N] = x_new * w_next and next_squares [fw_gemm_decode_accumulate_tiles(N)][16], per-tile sums
 // of x_new^2 of every row. A later call takes them with prologue 2 (a = those activations,
 // squares/squares_tiles = those sums, eps) and applies the row's scale in its epilogue.
-// glu_limit / glu_alpha / glu_shift (here and in fw_gemm_medium, epilogue 2 only): with a limit <= 0 the
-// gated unit is SwiGLU, silu(gate) * up; with a positive one its halves are clamped, g = min(gate,
+// glu_limit / glu_alpha / glu_shift (here and in fw_gemm_medium, epilogue 2 only): with a limit of 0 the
+// gated unit is SwiGLU, silu(gate) * up; with a negative one gelu_tanh(gate) * up; with a positive one its halves are clamped, g = min(gate,
 // limit), u = clamp(up, -limit, limit), and out = g * sigmoid(alpha * g) * (u + shift).
 // w_tiled (here and in fw_gemm_medium): w is not row-major [rows][K] but lies in operand tiles,
 // [rows / 16][K / 32][4][16][8]: tile (i, j) holds rows 16 i .. 16 i + 15, columns 32 j .. 32 j + 31 as
@@ -435,12 +435,13 @@ int fw_stream_join(float* x, int streams, const float* ls, const float* mix, con
 // float32 [rows][heads * vdim]. Segments of more than long_rows rows can be walked in chunks side by side on the matrix cores
 // (float32; the sums differ from the walk in order by rounding alone): chunk_seg / chunk_row0 [chunks] name every such
 // segment's chunks, side by side and in order, seg_chunk0 [segments + 1] where each segment's begin (an empty range for a short
-// one), workspace holds chunks * heads * dim * vdim floats. chunks 0: everything in order.
+// one), workspace holds chunks * heads * dim * vdim floats. chunks 0: everything in order. all_long: the caller vouches that no
+// segment is short (nothing is then launched for those).
 int fw_decay_chunk_rows(void);
 int fw_decay_recurrence(const float* q, const float* k, const float* v, int stride, const float* powers, float* state, int slots,
                         float* out, const int32_t* seg_row0, const int32_t* seg_slot, int rows, int segments, int heads, int dim, int vdim,
                         const int32_t* chunk_seg, const int32_t* chunk_row0, const int32_t* seg_chunk0, int chunks, int long_rows,
-                        float* workspace, void* stream);
+                        int all_long, float* workspace, void* stream);
 
 // ---- the selective scan ---------------------------------------------------------------------------------------------
 // Per segment, channel c and state n, with dt = softplus(z[c]): S <- 2^(dt A2[n][c]) S + dt x[c] B[n]; y = sum_n S C[n] +
@@ -452,7 +453,7 @@ int fw_selective_scan(const float* x, int x_stride, const float* z, int z_stride
                       int gate_stride, const float* A2, const float* D, float* state, int slots, void* out, int out_dtype,
                       const int32_t* seg_row0, const int32_t* seg_slot, int rows, int segments, int channels, int states,
                       const int32_t* chunk_seg, const int32_t* chunk_row0, const int32_t* seg_chunk0, int chunks, int long_rows,
-                      float* workspace, void* stream);
+                      int all_long, float* workspace, void* stream);
 // The same for segments of one row each (row r is segment r), with the map in front of the step sizes: z[c] = sum_j low[j]
 // w[j][c] + bias[c]. low rows: `rank` numbers, then B's `states` values, then C's. w float32 [rank][channels], or bfloat16 with
 // two neighbouring ranks of a channel side by side, [rank / 2][channels][2] (rank even).

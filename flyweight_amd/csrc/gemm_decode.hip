@@ -64,7 +64,7 @@ struct DecodeGemmArgs {
     // pre-normed prologue
     const float* squares;           // [squares_tiles][16], left by the kernel above
     int squares_tiles;
-    // the gated unit of epilogue 2: limit <= 0: silu(gate) * up; else clamped halves (fw_gated_unit)
+    // the gated unit of epilogue 2: limit 0: silu(gate) * up; < 0: gelu_tanh(gate) * up; else clamped halves (fw_gated_unit)
     float glu_limit, glu_alpha, glu_shift;
 };
 

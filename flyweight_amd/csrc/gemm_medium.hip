@@ -56,7 +56,7 @@ struct MediumArgs {
     int squares_rows;
     float eps;
     int rotate;                     // workgroups start their walk over K at different chunks
-    // the gated unit of mode 2: limit <= 0: silu(gate) * up; else clamped halves (fw_gated_unit)
+    // the gated unit of mode 2: limit 0: silu(gate) * up; < 0: gelu_tanh(gate) * up; else clamped halves (fw_gated_unit)
     float glu_limit, glu_alpha, glu_shift;
 };
 

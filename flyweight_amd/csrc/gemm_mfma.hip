@@ -257,7 +257,7 @@ __global__ __launch_bounds__(256) void gemm_mfma_kernel(
             for (int r = 0; r < 16; ++r) {
                 const int m = m0 + wm * 64 + i * 32 + 8 * (r >> 2) + row_base + (r & 3);
                 if (m < M && n < N)
-                    store_from_float(out, (size_t)m * N + n, silu_fast(acc[i][0][r]) * acc[i][NJ - 1][r]);
+                    store_from_float(out, (size_t)m * N + n, fw_gate_of<TO>(acc[i][0][r], [](float g) { return silu_fast(g); }) * acc[i][NJ - 1][r]);
             }
         return;
     }
@@ -322,13 +322,14 @@ extern "C" int fw_gemm_mfma(const void* a, const void* w, const float* bias, voi
     FW_REQUIRE(M >= 1 && N > 0 && K > 0 && K % 8 == 0, "gemm_mfma: K (%d) must be a positive multiple of 8; M=%d N=%d", K, M, N);
     FW_REQUIRE(mode >= 0 && mode <= 2, "gemm_mfma: unknown mode %d", mode);
     FW_REQUIRE(mode != MF_ACCUMULATE || out_dtype == FW_F32, "gemm_mfma: accumulation needs a float32 destination");
-    FW_REQUIRE(mode != MF_SWIGLU || (out_dtype == FW_BF16 && bias == nullptr), "gemm_mfma: SwiGLU stores bfloat16 and takes no bias");
-    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == MF_STORE), "gemm_mfma: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(mode != MF_SWIGLU || ((out_dtype == FW_BF16 || out_dtype == FW_BF16_GEGLU) && bias == nullptr), "gemm_mfma: SwiGLU stores bfloat16 and takes no bias");
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == MF_STORE) || (out_dtype == FW_BF16_GEGLU && mode == MF_SWIGLU), "gemm_mfma: unknown out dtype %d", out_dtype);
     FW_REQUIRE(((uintptr_t)a % 16 == 0) && ((uintptr_t)w % 16 == 0), "gemm_mfma: operands must be 16-byte aligned");
     FW_REQUIRE((long long)fw_ceil_div(M, TM) * fw_ceil_div(N, TN / 2) < (1ll << 30), "gemm_mfma: too many tiles");
     hipStream_t s = (hipStream_t)stream;
     int status;
-    if (mode == MF_SWIGLU) status = launch<MF_SWIGLU, 128, bf16_t>(a, w, nullptr, out, M, N, K, s);
+    if (mode == MF_SWIGLU && out_dtype == FW_BF16_GEGLU) status = launch<MF_SWIGLU, 128, geglu_bf16_t>(a, w, nullptr, out, M, N, K, s);
+    else if (mode == MF_SWIGLU) status = launch<MF_SWIGLU, 128, bf16_t>(a, w, nullptr, out, M, N, K, s);
     else if (mode == MF_ACCUMULATE) status = launch_by_width<MF_ACCUMULATE, float>(a, w, bias, out, M, N, K, s);
     else if (out_dtype == FW_F32) status = launch_by_width<MF_STORE, float>(a, w, bias, out, M, N, K, s);
     else if (out_dtype == FW_BF16_GELU) status = launch_by_width<MF_STORE, gelu_bf16_t>(a, w, bias, out, M, N, K, s);
@@ -382,8 +383,8 @@ extern "C" int fw_gemm_mfma_split(const void* a, const void* w, const float* bia
     FW_REQUIRE(M >= 1 && N > 0 && K > 0 && K % 8 == 0, "gemm_mfma_split: K (%d) must be a positive multiple of 8; M=%d N=%d", K, M, N);
     FW_REQUIRE(mode >= 0 && mode <= 2, "gemm_mfma_split: unknown mode %d", mode);
     FW_REQUIRE(mode != MF_ACCUMULATE || out_dtype == FW_F32, "gemm_mfma_split: accumulation needs a float32 destination");
-    FW_REQUIRE(mode != MF_SWIGLU || (out_dtype == FW_BF16 && bias == nullptr), "gemm_mfma_split: SwiGLU stores bfloat16 and takes no bias");
-    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == MF_STORE), "gemm_mfma_split: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(mode != MF_SWIGLU || ((out_dtype == FW_BF16 || out_dtype == FW_BF16_GEGLU) && bias == nullptr), "gemm_mfma_split: SwiGLU stores bfloat16 and takes no bias");
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == MF_STORE) || (out_dtype == FW_BF16_GEGLU && mode == MF_SWIGLU), "gemm_mfma_split: unknown out dtype %d", out_dtype);
     FW_REQUIRE(((uintptr_t)a % 16 == 0) && ((uintptr_t)w % 16 == 0), "gemm_mfma_split: operands must be 16-byte aligned");
     FW_REQUIRE((long long)fw_ceil_div(M, TM) * fw_ceil_div(N, 64) < (1ll << 30), "gemm_mfma_split: too many tiles");
     const SplitPlan plan = split_plan(mode, M, N, K);
@@ -395,7 +396,9 @@ extern "C" int fw_gemm_mfma_split(const void* a, const void* w, const float* bia
     hipStream_t s = (hipStream_t)stream;
     float* partials = (float*)workspace;
     int status;
-    if (mode == MF_SWIGLU) status = launch<MF_SWIGLU, 128, bf16_t, true>(a, w, nullptr, out, M, N, K, s, plan.slices, plan.k_per_split, partials, counters);
+    if (mode == MF_SWIGLU && out_dtype == FW_BF16_GEGLU)
+        status = launch<MF_SWIGLU, 128, geglu_bf16_t, true>(a, w, nullptr, out, M, N, K, s, plan.slices, plan.k_per_split, partials, counters);
+    else if (mode == MF_SWIGLU) status = launch<MF_SWIGLU, 128, bf16_t, true>(a, w, nullptr, out, M, N, K, s, plan.slices, plan.k_per_split, partials, counters);
     else if (mode == MF_ACCUMULATE) status = launch<MF_ACCUMULATE, 64, float, true>(a, w, bias, out, M, N, K, s, plan.slices, plan.k_per_split, partials, counters);
     else if (out_dtype == FW_F32) status = launch<MF_STORE, 64, float, true>(a, w, bias, out, M, N, K, s, plan.slices, plan.k_per_split, partials, counters);
     else if (out_dtype == FW_BF16_GELU) status = launch<MF_STORE, 64, gelu_bf16_t, true>(a, w, bias, out, M, N, K, s, plan.slices, plan.k_per_split, partials, counters);

@@ -274,8 +274,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
                         for (int h = 0; h < 2; ++h) {
                             const int r = 4 * q + 2 * h;        // rows 8 q + 2 h and the one below, of row tile i
-                            const float upper = silu_quick(acc[i][j][r]) * acc[i][j + 2][r];
-                            const float lower = silu_quick(acc[i][j][r + 1]) * acc[i][j + 2][r + 1];
+                            const float upper = fw_gate_of<TO>(acc[i][j][r], [](float g) { return silu_quick(g); }) * acc[i][j + 2][r];
+                            const float lower = fw_gate_of<TO>(acc[i][j][r + 1], [](float g) { return silu_quick(g); }) * acc[i][j + 2][r + 1];
                             const float got = from_neighbour(odd ? upper : lower);
                             const uint32_t word = odd ? pack_bf16x2(got, lower) : pack_bf16x2(upper, got);
                             const int row = i * 32 + 8 * q + 2 * h + (odd ? 1 : 0);
@@ -293,7 +293,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
                     const int m = m0 + wm * (TM * 32) + i * 32 + 8 * (r >> 2) + row_base + (r & 3);
-                    if (m < M) store_from_float(out, (size_t)m * N + n, silu_quick(acc[i][j][r]) * acc[i][j + 2][r]);
+                    if (m < M) store_from_float(out, (size_t)m * N + n, fw_gate_of<TO>(acc[i][j][r], [](float g) { return silu_quick(g); }) * acc[i][j + 2][r]);
                 }
         }
         return;
@@ -433,14 +433,15 @@ extern "C" int fw_gemm_mfma_big(const void* a, const void* w, const float* bias,
     FW_REQUIRE(M >= 1 && N > 0 && K > 0 && K % BK == 0, "gemm_mfma_big: K (%d) must be a positive multiple of %d; M=%d N=%d", K, BK, M, N);
     FW_REQUIRE(mode >= 0 && mode <= 2, "gemm_mfma_big: unknown mode %d", mode);
     FW_REQUIRE(mode != MB_ACCUMULATE || out_dtype == FW_F32, "gemm_mfma_big: accumulation needs a float32 destination");
-    FW_REQUIRE(mode != MB_SWIGLU || (out_dtype == FW_BF16 && bias == nullptr), "gemm_mfma_big: SwiGLU stores bfloat16 and takes no bias");
-    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == MB_STORE), "gemm_mfma_big: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(mode != MB_SWIGLU || ((out_dtype == FW_BF16 || out_dtype == FW_BF16_GEGLU) && bias == nullptr), "gemm_mfma_big: SwiGLU stores bfloat16 and takes no bias");
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == MB_STORE) || (out_dtype == FW_BF16_GEGLU && mode == MB_SWIGLU), "gemm_mfma_big: unknown out dtype %d", out_dtype);
     FW_REQUIRE(((uintptr_t)a % 16 == 0) && ((uintptr_t)w % 16 == 0), "gemm_mfma_big: operands must be 16-byte aligned");
     FW_REQUIRE((long long)fw_ceil_div(M, BT / 2) * fw_ceil_div(N, BT / 2) < (1ll << 30), "gemm_mfma_big: too many tiles");
     hipStream_t s = (hipStream_t)stream;
     const BigPlan plan = big_plan(mode, M, N);
     int status;
-    if (mode == MB_SWIGLU) status = launch_big<MB_SWIGLU, bf16_t>(a, w, nullptr, out, M, N, K, s);
+    if (mode == MB_SWIGLU && out_dtype == FW_BF16_GEGLU) status = launch_big<MB_SWIGLU, geglu_bf16_t>(a, w, nullptr, out, M, N, K, s);
+    else if (mode == MB_SWIGLU) status = launch_big<MB_SWIGLU, bf16_t>(a, w, nullptr, out, M, N, K, s);
     else if (mode == MB_ACCUMULATE) status = launch_planned<MB_ACCUMULATE, float>(plan, a, w, bias, out, M, N, K, s);
     else if (out_dtype == FW_F32) status = launch_planned<MB_STORE, float>(plan, a, w, bias, out, M, N, K, s);
     else if (out_dtype == FW_BF16_GELU) status = launch_planned<MB_STORE, gelu_bf16_t>(plan, a, w, bias, out, M, N, K, s);

@@ -124,7 +124,7 @@ __global__ __launch_bounds__(SK_WAVES * 64) void gemm_skinny_kernel(
             if (n >= N) continue;
             float value = total[r];
             if (MODE == SK_SWIGLU) {
-                value = silu_f(value) * second[r];
+                value = fw_gate_of<TO>(value, [](float g) { return silu_f(g); }) * second[r];
             } else if (bias) {
                 value += bias[n];
             }
@@ -143,7 +143,10 @@ static void launch_mode(const void* a, const void* w, const float* bias, void* o
     const int threads = WAVES * 64;
     if (mode == SK_SWIGLU) {
         const int blocks = fw_ceil_div(N, 16);
-        gemm_skinny_kernel<MT, 2, WAVES, SK_SWIGLU, bf16_t><<<blocks, threads, 0, stream>>>(pa, pw, nullptr, (bf16_t*)out, M, N, K, up_offset);
+        if (out_dtype == FW_BF16_GEGLU)
+            gemm_skinny_kernel<MT, 2, WAVES, SK_SWIGLU, geglu_bf16_t><<<blocks, threads, 0, stream>>>(pa, pw, nullptr, (geglu_bf16_t*)out, M, N, K, up_offset);
+        else
+            gemm_skinny_kernel<MT, 2, WAVES, SK_SWIGLU, bf16_t><<<blocks, threads, 0, stream>>>(pa, pw, nullptr, (bf16_t*)out, M, N, K, up_offset);
         return;
     }
     const int blocks = fw_ceil_div(N, 16 * RT);
@@ -175,8 +178,8 @@ extern "C" int fw_gemm_skinny(const void* a, const void* w, const float* bias, v
     FW_REQUIRE(N > 0 && K > 0 && K % 8 == 0, "gemm_skinny: K (%d) must be a positive multiple of 8, N (%d) positive", K, N);
     FW_REQUIRE(mode >= 0 && mode <= 2, "gemm_skinny: unknown mode %d", mode);
     FW_REQUIRE(mode != SK_ACCUMULATE || out_dtype == FW_F32, "gemm_skinny: accumulation needs a float32 destination");
-    FW_REQUIRE(mode != SK_SWIGLU || (out_dtype == FW_BF16 && bias == nullptr), "gemm_skinny: SwiGLU stores bfloat16 and takes no bias");
-    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == SK_STORE), "gemm_skinny: unknown out dtype %d", out_dtype);
+    FW_REQUIRE(mode != SK_SWIGLU || ((out_dtype == FW_BF16 || out_dtype == FW_BF16_GEGLU) && bias == nullptr), "gemm_skinny: SwiGLU stores bfloat16 and takes no bias");
+    FW_REQUIRE(out_dtype == FW_F32 || out_dtype == FW_BF16 || (out_dtype == FW_BF16_GELU && mode == SK_STORE) || (out_dtype == FW_BF16_GEGLU && mode == SK_SWIGLU), "gemm_skinny: unknown out dtype %d", out_dtype);
     FW_REQUIRE(((uintptr_t)a % 16 == 0) && ((uintptr_t)w % 16 == 0), "gemm_skinny: operands must be 16-byte aligned");
     hipStream_t s = (hipStream_t)stream;
     switch ((M + 15) / 16) {

@@ -613,6 +613,7 @@ extern "C" int fw_grouped_gemm(const void* a, int a_dtype, const int32_t* place_
                                const int32_t* expert_begin, void* out, int out_dtype, int gated, int places, int experts, int N, int K,
                                float glu_limit, float glu_alpha, float glu_shift, void* stream) {
     const GatedUnit unit = {glu_limit, glu_alpha, glu_shift};
+    FW_REQUIRE(glu_limit >= 0.0f, "grouped_gemm: the experts' unit is silu or clamped");
     FW_REQUIRE(glu_limit <= 0.0f || gated, "grouped_gemm: a clamped unit goes with gate and up rows");
     FW_REQUIRE(places >= 0 && experts >= 1 && N > 0 && K > 0, "grouped_gemm: bad sizes places=%d experts=%d N=%d K=%d", places, experts, N, K);
     if (places == 0) return 0;

@@ -8,37 +8,46 @@
 #include "fw_kernels.h"
 
 #define SS_TOKENS 16            // tokens whose B and C are staged together
-#define SS_AHEAD 8              // tokens whose inputs are asked for together
 #define SS_CHUNK 64
 #define SS_MAX_STATE 128
 
 // softplus(x) = ln(1 + e^x). The logarithm of the rounded u = 1 + e is corrected by e / (u - 1), which is exact to the last
 // digits however small e is; beyond 20 e^-x no longer shows.
+// QUICK (the bfloat16 runs): the hardware's exponential and reciprocal, a few units in the last place of float32.
+template <bool QUICK>
 __device__ __forceinline__ float ss_softplus(float x) {
-    const float e = expf(x);
+    const float e = QUICK ? __expf(x) : expf(x);
     const float u = 1.0f + e, d = u - 1.0f;
     const float ln = __builtin_amdgcn_logf(u) * 0.69314718055994531f;
-    const float corrected = d == 0.0f ? e : ln * (e / d);
+    const float corrected = d == 0.0f ? e : ln * (QUICK ? e * __builtin_amdgcn_rcpf(d) : e / d);
     return x > 20.0f ? x : corrected;
 }
-__device__ __forceinline__ float ss_silu(float z) { return z / (1.0f + expf(-z)); }
+template <bool QUICK>
+__device__ __forceinline__ float ss_silu(float z) {
+    return QUICK ? z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)) : z / (1.0f + expf(-z));
+}
 
 // A run of rows row0 .. row0 + count - 1 for one channel a lane: S moves on; with OUT the outputs are formed, else the steps' sum
 // is. All lanes of the workgroup (one wave) call it together: they share the staged B and C.
-template <int N, bool OUT, typename TO>
+// EXACT: the model has N states, and B and C are read where they lie: the row is the same for all lanes, so they travel as
+// scalars and enter the arithmetic as such, with no trip through LDS.
+template <int N, bool EXACT, bool OUT, bool QUICK, typename TO>
 __device__ __forceinline__ float ss_run(float (&S)[N], const float (&a)[N], float d, const float* __restrict__ x, int x_stride,
                                         const float* __restrict__ z, int z_stride, const float* __restrict__ bc, int bc_stride,
                                         const float* __restrict__ gate, int gate_stride, TO* __restrict__ out, int row0, int count, int at,
                                         bool live, int channels, int states, float* staged) {
+    constexpr int SS_AHEAD = N <= 32 ? 8 : 2;           // tokens whose inputs are asked for together
     float total = 0.0f;
     for (int base = 0; base < count; base += SS_TOKENS) {
         const int tokens = count - base < SS_TOKENS ? count - base : SS_TOKENS;
-        __syncthreads();
-        for (int i = threadIdx.x; i < tokens * 2 * N; i += 64) {
-            const int token = i / (2 * N), j = i % (2 * N), n = j % N;
-            staged[i] = n < states ? bc[(size_t)(row0 + base + token) * bc_stride + (j < N ? n : states + n)] : 0.0f;
+        if (!EXACT) {
+            __syncthreads();
+            for (int i = threadIdx.x; i < tokens * 2 * N; i += 64) {
+                const int token = i / (2 * N), j = i % (2 * N), n = j % N;
+                staged[i] = n < states ? bc[(size_t)(row0 + base + token) * bc_stride + (j < N ? n : states + n)] : 0.0f;
+            }
+            __syncthreads();
         }
-        __syncthreads();
         for (int t0 = 0; t0 < tokens; t0 += SS_AHEAD) {
             float xs[SS_AHEAD], zs[SS_AHEAD], gs[SS_AHEAD];
 #pragma unroll
@@ -48,12 +57,10 @@ __device__ __forceinline__ float ss_run(float (&S)[N], const float (&a)[N], floa
                 zs[u] = z[row * z_stride + at];
                 gs[u] = OUT ? gate[row * gate_stride + at] : 0.0f;
             }
-#pragma unroll
-            for (int u = 0; u < SS_AHEAD; ++u) {
-                if (t0 + u >= tokens) break;
-                const float dt = ss_softplus(zs[u]);
+            auto token = [&](int u) {
+                const float dt = ss_softplus<QUICK>(zs[u]);
                 const float dx = dt * xs[u];
-                const float* B = staged + (t0 + u) * 2 * N;
+                const float* B = EXACT ? bc + (size_t)(row0 + base + t0 + u) * bc_stride : staged + (t0 + u) * 2 * N;
                 float y = 0.0f;
 #pragma unroll
                 for (int n = 0; n < N; ++n) {
@@ -62,9 +69,19 @@ __device__ __forceinline__ float ss_run(float (&S)[N], const float (&a)[N], floa
                 }
                 if (OUT) {
                     y = fmaf(d, xs[u], y);
-                    if (live) store_from_float(out, (size_t)(row0 + base + t0 + u) * channels + at, y * ss_silu(gs[u]));
+                    if (live) store_from_float(out, (size_t)(row0 + base + t0 + u) * channels + at, y * ss_silu<QUICK>(gs[u]));
                 } else {
                     total += dt;
+                }
+            };
+            if (t0 + SS_AHEAD <= tokens) {              // no branch between the tokens: what the next one needs is asked for ahead
+#pragma unroll
+                for (int u = 0; u < SS_AHEAD; ++u) token(u);
+            } else {
+#pragma unroll
+                for (int u = 0; u < SS_AHEAD; ++u) {
+                    if (t0 + u >= tokens) break;
+                    token(u);
                 }
             }
         }
@@ -75,12 +92,12 @@ __device__ __forceinline__ float ss_run(float (&S)[N], const float (&a)[N], floa
 // ---- in order ---------------------------------------------------------------------------------------------------
 // A thread per (segment, channel), its N states in registers (N: the template's size, the model's states of it used; the
 // others have A = B = C = 0 and stay zero). Segments of more than long_rows rows (> 0) are left to the chunked kernels.
-template <int N, typename TO>
+template <int N, bool EXACT, typename TO>
 __global__ __launch_bounds__(64) void selective_scan_step_kernel(
     const float* __restrict__ x, int x_stride, const float* __restrict__ z, int z_stride, const float* __restrict__ bc, int bc_stride,
     const float* __restrict__ gate, int gate_stride, const float* __restrict__ A2, const float* __restrict__ D, float* __restrict__ state,
     TO* __restrict__ out, const int32_t* __restrict__ seg_row0, const int32_t* __restrict__ seg_slot, int channels, int states, int long_rows) {
-    __shared__ __attribute__((aligned(16))) float staged[SS_TOKENS * 2 * N];
+    __shared__ __attribute__((aligned(16))) float staged[EXACT ? 4 : SS_TOKENS * 2 * N];
     const int seg = blockIdx.x;
     const int first = seg_row0[seg], count = seg_row0[seg + 1] - first;
     if (long_rows > 0 && count > long_rows) return;
@@ -94,7 +111,7 @@ __global__ __launch_bounds__(64) void selective_scan_step_kernel(
         S[n] = n < states ? mine[(size_t)n * channels] : 0.0f;
         a[n] = n < states ? A2[(size_t)n * channels + at] : 0.0f;
     }
-    ss_run<N, true, TO>(S, a, D[at], x, x_stride, z, z_stride, bc, bc_stride, gate, gate_stride, out, first, count, at, live, channels, states, staged);
+    ss_run<N, EXACT, true, sizeof(TO) == 2, TO>(S, a, D[at], x, x_stride, z, z_stride, bc, bc_stride, gate, gate_stride, out, first, count, at, live, channels, states, staged);
     if (live)
 #pragma unroll
         for (int n = 0; n < N; ++n)
@@ -106,12 +123,12 @@ __global__ __launch_bounds__(64) void selective_scan_step_kernel(
 // state (leaving its last state and the sum of its steps), the states ahead of the chunks (S_out = 2^(sum dt A') S_in + the
 // chunk's own, a thread per channel and state), and every chunk once more from its S_in, with the outputs.
 // local [chunk][n][channel], steps [chunk][channel].
-template <int N>
+template <int N, bool EXACT, bool QUICK>
 __global__ __launch_bounds__(64) void selective_scan_chunk_kernel(
     const float* __restrict__ x, int x_stride, const float* __restrict__ z, int z_stride, const float* __restrict__ bc, int bc_stride,
     const float* __restrict__ A2, float* __restrict__ local, float* __restrict__ steps, const int32_t* __restrict__ chunk_seg,
     const int32_t* __restrict__ chunk_row0, const int32_t* __restrict__ seg_row0, int channels, int states) {
-    __shared__ __attribute__((aligned(16))) float staged[SS_TOKENS * 2 * N];
+    __shared__ __attribute__((aligned(16))) float staged[EXACT ? 4 : SS_TOKENS * 2 * N];
     const int chunk = blockIdx.x;
     const int row0 = chunk_row0[chunk], end = seg_row0[chunk_seg[chunk] + 1];
     const int count = end - row0 < SS_CHUNK ? end - row0 : SS_CHUNK;
@@ -124,7 +141,7 @@ __global__ __launch_bounds__(64) void selective_scan_chunk_kernel(
         S[n] = 0.0f;
         a[n] = n < states ? A2[(size_t)n * channels + at] : 0.0f;
     }
-    const float total = ss_run<N, false, float>(S, a, 0.0f, x, x_stride, z, z_stride, bc, bc_stride, nullptr, 0, nullptr, row0, count, at, live,
+    const float total = ss_run<N, EXACT, false, QUICK, float>(S, a, 0.0f, x, x_stride, z, z_stride, bc, bc_stride, nullptr, 0, nullptr, row0, count, at, live,
                                                 channels, states, staged);
     if (!live) return;
     float* to = local + (size_t)chunk * states * channels + c;
@@ -167,13 +184,13 @@ __global__ __launch_bounds__(256) void selective_scan_state_kernel(const float* 
     *slot = S;
 }
 
-template <int N, typename TO>
+template <int N, bool EXACT, typename TO>
 __global__ __launch_bounds__(64) void selective_scan_finish_kernel(
     const float* __restrict__ x, int x_stride, const float* __restrict__ z, int z_stride, const float* __restrict__ bc, int bc_stride,
     const float* __restrict__ gate, int gate_stride, const float* __restrict__ A2, const float* __restrict__ D,
     const float* __restrict__ local, TO* __restrict__ out, const int32_t* __restrict__ chunk_seg, const int32_t* __restrict__ chunk_row0,
     const int32_t* __restrict__ seg_row0, int channels, int states) {
-    __shared__ __attribute__((aligned(16))) float staged[SS_TOKENS * 2 * N];
+    __shared__ __attribute__((aligned(16))) float staged[EXACT ? 4 : SS_TOKENS * 2 * N];
     const int chunk = blockIdx.x;
     const int row0 = chunk_row0[chunk], end = seg_row0[chunk_seg[chunk] + 1];
     const int count = end - row0 < SS_CHUNK ? end - row0 : SS_CHUNK;
@@ -187,7 +204,7 @@ __global__ __launch_bounds__(64) void selective_scan_finish_kernel(
         S[n] = n < states ? from[(size_t)n * channels] : 0.0f;
         a[n] = n < states ? A2[(size_t)n * channels + at] : 0.0f;
     }
-    ss_run<N, true, TO>(S, a, D[at], x, x_stride, z, z_stride, bc, bc_stride, gate, gate_stride, out, row0, count, at, live, channels, states, staged);
+    ss_run<N, EXACT, true, sizeof(TO) == 2, TO>(S, a, D[at], x, x_stride, z, z_stride, bc, bc_stride, gate, gate_stride, out, row0, count, at, live, channels, states, staged);
 }
 
 extern "C" int fw_scan_chunk_rows(void) { return SS_CHUNK; }
@@ -196,7 +213,7 @@ extern "C" int fw_selective_scan(const float* x, int x_stride, const float* z, i
                                  int gate_stride, const float* A2, const float* D, float* state, int slots, void* out, int out_dtype,
                                  const int32_t* seg_row0, const int32_t* seg_slot, int rows, int segments, int channels, int states,
                                  const int32_t* chunk_seg, const int32_t* chunk_row0, const int32_t* seg_chunk0, int chunks, int long_rows,
-                                 float* workspace, void* stream) {
+                                 int all_long, float* workspace, void* stream) {
     FW_REQUIRE(rows >= 0 && segments >= 0 && channels > 0 && slots > 0, "selective_scan: bad sizes rows=%d segments=%d channels=%d", rows, segments, channels);
     FW_REQUIRE(states >= 1 && states <= SS_MAX_STATE, "selective_scan: %d states a channel (1..%d)", states, SS_MAX_STATE);
     FW_REQUIRE((long long)channels * states < (1ll << 24), "selective_scan: too many channels (%d)", channels);
@@ -212,27 +229,34 @@ extern "C" int fw_selective_scan(const float* x, int x_stride, const float* z, i
     const dim3 by_state(segments, fw_ceil_div((long long)channels * states, 256));
     float* local = workspace;
     float* steps = workspace ? workspace + (size_t)chunks * states * channels : nullptr;
-#define FW_SCAN_OUT(N, TO)                                                                                                                   \
-    selective_scan_step_kernel<N, TO><<<grid, 64, 0, s>>>(x, x_stride, z, z_stride, bc, bc_stride, gate, gate_stride, A2, D, state,          \
-                                                          (TO*)out, seg_row0, seg_slot, channels, states, chunks > 0 ? long_rows : 0);       \
+#define FW_SCAN_OUT(N, EXACT, TO)                                                                                                            \
+    if (chunks == 0 || !all_long)                                                                                                            \
+        selective_scan_step_kernel<N, EXACT, TO><<<grid, 64, 0, s>>>(x, x_stride, z, z_stride, bc, bc_stride, gate, gate_stride, A2, D,      \
+                                                                     state, (TO*)out, seg_row0, seg_slot, channels, states,                  \
+                                                                     chunks > 0 ? long_rows : 0);                                            \
     if (chunks > 0) {                                                                                                                        \
-        selective_scan_chunk_kernel<N><<<by_chunk, 64, 0, s>>>(x, x_stride, z, z_stride, bc, bc_stride, A2, local, steps, chunk_seg,         \
-                                                               chunk_row0, seg_row0, channels, states);                                      \
+        selective_scan_chunk_kernel<N, EXACT, sizeof(TO) == 2><<<by_chunk, 64, 0, s>>>(x, x_stride, z, z_stride, bc, bc_stride, A2, local, steps, chunk_seg,  \
+                                                                      chunk_row0, seg_row0, channels, states);                               \
         selective_scan_state_kernel<<<by_state, 256, 0, s>>>(A2, local, steps, state, seg_chunk0, seg_slot, channels, states);               \
-        selective_scan_finish_kernel<N, TO><<<by_chunk, 64, 0, s>>>(x, x_stride, z, z_stride, bc, bc_stride, gate, gate_stride, A2, D, local, \
-                                                                    (TO*)out, chunk_seg, chunk_row0, seg_row0, channels, states);            \
+        selective_scan_finish_kernel<N, EXACT, TO><<<by_chunk, 64, 0, s>>>(x, x_stride, z, z_stride, bc, bc_stride, gate, gate_stride, A2,   \
+                                                                           D, local, (TO*)out, chunk_seg, chunk_row0, seg_row0, channels,    \
+                                                                           states);                                                          \
     }
-#define FW_SCAN_LAUNCH(N)                                 \
-    {                                                     \
-        if (out_dtype == FW_F32) { FW_SCAN_OUT(N, float) } \
-        else { FW_SCAN_OUT(N, bf16_t) }                   \
+#define FW_SCAN_LAUNCH(N, EXACT)                                 \
+    {                                                            \
+        if (out_dtype == FW_F32) { FW_SCAN_OUT(N, EXACT, float) } \
+        else { FW_SCAN_OUT(N, EXACT, bf16_t) }                   \
     }
-    if (states <= 8) FW_SCAN_LAUNCH(8)
-    else if (states <= 16) FW_SCAN_LAUNCH(16)
-    else if (states <= 24) FW_SCAN_LAUNCH(24)
-    else if (states <= 32) FW_SCAN_LAUNCH(32)
-    else if (states <= 64) FW_SCAN_LAUNCH(64)
-    else FW_SCAN_LAUNCH(128)
+    if (states == 8) FW_SCAN_LAUNCH(8, true)
+    else if (states == 16) FW_SCAN_LAUNCH(16, true)
+    else if (states == 32) FW_SCAN_LAUNCH(32, true)
+    else if (states == 64) FW_SCAN_LAUNCH(64, true)
+    else if (states <= 8) FW_SCAN_LAUNCH(8, false)
+    else if (states <= 16) FW_SCAN_LAUNCH(16, false)
+    else if (states <= 24) FW_SCAN_LAUNCH(24, false)
+    else if (states <= 32) FW_SCAN_LAUNCH(32, false)
+    else if (states <= 64) FW_SCAN_LAUNCH(64, false)
+    else FW_SCAN_LAUNCH(128, false)
 #undef FW_SCAN_LAUNCH
 #undef FW_SCAN_OUT
     FW_LAUNCH_CHECK("selective_scan");
@@ -293,7 +317,7 @@ __global__ __launch_bounds__(256) void selective_scan_low_rank_kernel(
     __syncthreads();
     if (part != 0) return;
     const float z = (((parts[lane] + parts[64 + lane]) + parts[128 + lane]) + parts[192 + lane]) + bias[at];
-    const float dt = ss_softplus(z), dx = dt * xx;
+    const float dt = ss_softplus<sizeof(TO) == 2>(z), dx = dt * xx;
     float y = 0.0f;
 #pragma unroll
     for (int n = 0; n < N; ++n) {
@@ -301,7 +325,7 @@ __global__ __launch_bounds__(256) void selective_scan_low_rank_kernel(
         y = fmaf(S[n], B[N + n], y);
     }
     if (!live) return;
-    store_from_float(out, (size_t)row * channels + c, fmaf(D[c], xx, y) * ss_silu(g));
+    store_from_float(out, (size_t)row * channels + c, fmaf(D[c], xx, y) * ss_silu<sizeof(TO) == 2>(g));
 #pragma unroll
     for (int n = 0; n < N; ++n)
         if (n < states) mine[(size_t)n * channels] = S[n];

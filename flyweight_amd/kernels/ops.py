@@ -16,7 +16,8 @@ import torch
 
 from . import build as _build
 
-F32, BF16, BF16_GELU = 0, 1, 2     # (the last: what a storing product leaves as gelu of its float32 sums)
+# (the last two: a storing product leaves gelu of its float32 sums; a gated product gelu_tanh(gate) * up)
+F32, BF16, BF16_GELU, BF16_GEGLU = 0, 1, 2, 3
 PAGE_SIZE = 64          # tokens per cache page: the width of a wavefront
 MAX_HEAD_DIM = 256          # of the matrix-core attention kernels
 MAX_PLAIN_HEAD_DIM = 1024   # of the plain attention kernels, which serve what the others do not take
@@ -520,7 +521,10 @@ def _fast_gemm(a: torch.Tensor, w: torch.Tensor, bias, target: torch.Tensor, out
     M, K = a.shape
     if SKINNY_MAX_ROWS < M <= MEDIUM_MAX_ROWS or (M <= SKINNY_MAX_ROWS and w.numel() >= MEDIUM_LARGE and K % 8 == 0):
         # also a few rows of a large W (a vocabulary's head: 65,536 x 2,048 at 8 rows 52 against 61 us)
-        gemm_medium_into(a, w, bias, target, out_code, mode, N, w_tiled=w_tiled)
+        if out_code == BF16_GEGLU:      # that product is told by its unit, not by the output's type
+            gemm_medium_into(a, w, bias, target, BF16, mode, N, w_tiled=w_tiled, glu=GEGLU)
+        else:
+            gemm_medium_into(a, w, bias, target, out_code, mode, N, w_tiled=w_tiled)
         return
     if M <= SKINNY_MAX_ROWS:
         entry = library().fw_gemm_skinny
@@ -809,8 +813,9 @@ def gemm(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None,
     return out
 
 
-def gemm_swiglu(a: torch.Tensor, w_gate_up: torch.Tensor, w_tiled: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """silu(a . gate^T) * (a . up^T) with w_gate_up = [gate rows; up rows]: [M, I] in a's dtype.
+def gemm_swiglu(a: torch.Tensor, w_gate_up: torch.Tensor, w_tiled: Optional[torch.Tensor] = None, gelu: bool = False) -> torch.Tensor:
+    """silu(a . gate^T) * (a . up^T) with w_gate_up = [gate rows; up rows]: [M, I] in a's dtype (``gelu``: the tanh form of gelu
+    in place of silu).
     On the bfloat16 path the activation is formed from the float32 sums inside the product's
     kernel; otherwise the [M, 2I] intermediate is float32 and a second kernel forms it."""
     rows2, K = w_gate_up.shape
@@ -821,19 +826,23 @@ def gemm_swiglu(a: torch.Tensor, w_gate_up: torch.Tensor, w_tiled: Optional[torc
         if a.shape[1] != K:
             raise KernelError(f"gemm_swiglu: a is {tuple(a.shape)} but w is {tuple(w_gate_up.shape)}")
         out = torch.empty((a.shape[0], rows2 // 2), dtype=torch.bfloat16, device=a.device)
-        _fast_gemm(a, w_gate_up, None, out, BF16, 2, rows2 // 2, w_tiled)
+        _fast_gemm(a, w_gate_up, None, out, BF16_GEGLU if gelu else BF16, 2, rows2 // 2, w_tiled)
         return out
-    return swiglu(gemm_generic(a, w_gate_up, out_dtype=torch.float32), out_dtype=a.dtype)
+    return swiglu(gemm_generic(a, w_gate_up, out_dtype=torch.float32), out_dtype=a.dtype, gelu=gelu)
 
 
 # ---- fused products for decode steps of up to 16 rows --------------------------------------------
 EPILOGUE_STORE, EPILOGUE_ACCUMULATE, EPILOGUE_SWIGLU, EPILOGUE_CONV = 0, 1, 2, 3
 
 
-def _glu(glu: Optional[tuple]):
-    """The three numbers a gated epilogue takes: (0, 1, 0) is SwiGLU; else (limit > 0, alpha, shift)."""
-    if glu is None:
-        return ctypes.c_float(0.0), ctypes.c_float(1.0), ctypes.c_float(0.0)
+GEGLU = "gelu_tanh"       # in place of a clamped unit's three numbers
+
+
+def _glu(glu):
+    """The three numbers a gated epilogue takes: (0, 1, 0) is SwiGLU, (-1, 1, 0) the same around the tanh form of gelu
+    (``GEGLU``); else (limit > 0, alpha, shift)."""
+    if glu is None or glu == GEGLU:
+        return ctypes.c_float(0.0 if glu is None else -1.0), ctypes.c_float(1.0), ctypes.c_float(0.0)
     limit, alpha, shift = glu
     if not limit > 0:
         raise KernelError("a gated unit with clamped halves needs a positive limit")
@@ -1963,18 +1972,18 @@ MAX_DECAY_DIM = 256      # key channels of a head
 
 
 def _chunks(name: str, chunks: Optional[tuple], segments: int):
-    """(chunk_seg, chunk_row0, seg_chunk0, rows from which a segment is walked in chunks) -> the arguments of a launch, their
-    number."""
+    """(chunk_seg, chunk_row0, seg_chunk0, rows beyond which a segment is walked in chunks, whether every segment of the step is
+    that long) -> a launch's arguments: the arrays, their number, the rows, the flag."""
     if chunks is None:
-        return (None, None, None), 0, 0
-    chunk_seg, chunk_row0, seg_chunk0, long_rows = chunks
+        return (None, None, None), 0, 0, 0
+    chunk_seg, chunk_row0, seg_chunk0, long_rows, all_long = chunks
     _dev(chunk_seg, chunk_row0, seg_chunk0)
     count = chunk_seg.numel()
     for which, t, n in (("chunk_seg", chunk_seg, count), ("chunk_row0", chunk_row0, count), ("seg_chunk0", seg_chunk0, segments + 1)):
         _want(t, torch.int32, which)
         if t.numel() < n:
             raise KernelError(f"{name}: {which} holds {t.numel()} entries, needs {n}")
-    return (chunk_seg, chunk_row0, seg_chunk0), count, int(long_rows)
+    return (chunk_seg, chunk_row0, seg_chunk0), count, int(long_rows), int(all_long)
 
 
 DECAY_CHUNK = 64        # rows of a chunk, as the kernels have them
@@ -1993,7 +2002,7 @@ def decay_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, powers: 
     """Per head S <- decay S + silu(k) silu(v)^T, o = S^T silu(q) over each segment's rows in order. ``q``, ``k`` float32
     [rows, heads dim] and ``v`` [rows, heads vdim] with one row stride (views of wider rows will do); ``powers``: see
     ``decay_powers``; ``state`` float32 [slots, heads, dim, vdim] is read and moved on. ``chunks`` (chunk_seg, chunk_row0, seg_chunk0,
-    long_rows): segments of more than long_rows rows are walked in these chunks side by side. Returns float32 [rows, heads vdim]."""
+    long_rows, whether every segment is longer than that): segments of more than long_rows rows are walked in these chunks side by side. Returns float32 [rows, heads vdim]."""
     _dev(powers, state)
     _segments("decay_recurrence", segments, seg_row0, seg_slot)
     rows = q.shape[0]
@@ -2010,10 +2019,10 @@ def decay_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, powers: 
         if t.shape != shape:
             raise KernelError(f"decay_recurrence: {name} is {tuple(t.shape)}, expected {shape}")
     out = torch.empty((rows, heads * vdim), dtype=torch.float32, device=q.device)
-    places, count, long_rows = _chunks("decay_recurrence", chunks, segments)
+    places, count, *how = _chunks("decay_recurrence", chunks, segments)
     workspace = torch.empty((count, heads, dim, vdim), dtype=torch.float32, device=q.device) if count else None
     _check(library().fw_decay_recurrence(_p(q), _p(k), _p(v), stride, _p(powers), _p(state), state.shape[0], _p(out), _p(seg_row0),
-                                         _p(seg_slot), rows, int(segments), heads, dim, vdim, *(_p(t) for t in places), count, long_rows,
+                                         _p(seg_slot), rows, int(segments), heads, dim, vdim, *(_p(t) for t in places), count, *how,
                                          _p(workspace), _stream()))
     return out
 
@@ -2043,11 +2052,11 @@ def selective_scan(x: torch.Tensor, z: torch.Tensor, bc: torch.Tensor, gate: tor
         if t.shape != shape:
             raise KernelError(f"selective_scan: {name} is {tuple(t.shape)}, expected {shape}")
     out = torch.empty((rows, channels), dtype=out_dtype, device=x.device)
-    places, count, long_rows = _chunks("selective_scan", chunks, segments)
+    places, count, *how = _chunks("selective_scan", chunks, segments)
     workspace = torch.empty((count, states + 1, channels), dtype=torch.float32, device=x.device) if count else None
     _check(library().fw_selective_scan(_p(x), _stride(x), _p(z), _stride(z), _p(bc), _stride(bc), _p(gate), _stride(gate), _p(A2), _p(D), _p(state),
                                        state.shape[0], _p(out), _code(out_dtype), _p(seg_row0), _p(seg_slot), rows, int(segments), channels,
-                                       states, *(_p(t) for t in places), count, long_rows, _p(workspace), _stream()))
+                                       states, *(_p(t) for t in places), count, *how, _p(workspace), _stream()))
     return out
 
 

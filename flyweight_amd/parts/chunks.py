@@ -39,4 +39,5 @@ class RecurrenceChunks:
         own = ctx.step_arrays(self) if not ctx.all_decode else {}
         if not own or own["chunk_seg"].numel() == 0:
             return {}
-        return {"chunks": (own["chunk_seg"], own["chunk_row0"], own["seg_chunk0"], self.LONG_ROWS)}
+        lengths = np.diff(ctx.host_seg_row0)
+        return {"chunks": (own["chunk_seg"], own["chunk_row0"], own["seg_chunk0"], self.LONG_ROWS, bool(lengths.min() > self.LONG_ROWS))}

@@ -139,14 +139,13 @@ class Linear:
     def swiglu(self, a: Input, gelu: bool = False) -> torch.Tensor:
         """The weight holds gate rows then up rows: silu(a . gate^T) * (a . up^T); ``gelu``: the tanh form of gelu in
         place of silu."""
-        if gelu:
-            return ops.swiglu(self.forward(a, out_dtype=torch.float32), out_dtype=a.dtype, gelu=True)
+        glu = ops.GEGLU if gelu else None
         if self.bias is None and self._medium(a):
-            return ops.gemm_medium(self._rows_of(a), self.weight, ops.EPILOGUE_SWIGLU, w_tiled=self.tiled, **self._prepared_arguments(a))
+            return ops.gemm_medium(self._rows_of(a), self.weight, ops.EPILOGUE_SWIGLU, w_tiled=self.tiled, glu=glu, **self._prepared_arguments(a))
         if self.bias is None and self._fused(a, self.out_features // 2, ops.EPILOGUE_SWIGLU):
             return ops.gemm_decode(self._rows_of(a), self.weight, ops.EPILOGUE_SWIGLU, out_dtype=torch.bfloat16,
-                                   w_tiled=self.tiled, **self._norm_arguments(a))
-        return ops.gemm_swiglu(self._tensor_of(a), self.weight, w_tiled=self.tiled)
+                                   w_tiled=self.tiled, glu=glu, **self._norm_arguments(a))
+        return ops.gemm_swiglu(self._tensor_of(a), self.weight, w_tiled=self.tiled, gelu=gelu)
 
     def gelu(self, a: torch.Tensor) -> torch.Tensor:
         """gelu(a . W^T (+ bias)), the error-function form, in a's dtype."""

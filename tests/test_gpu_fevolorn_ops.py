@@ -50,7 +50,7 @@ def chunks_of(lengths, long_rows=32, size=64):
             seg.append(s)
             first.append(row0[s] + at)
         begins.append(len(seg))
-    return (ints(seg), ints(first), ints(begins), long_rows) if seg else None
+    return (ints(seg), ints(first), ints(begins), long_rows, min(lengths) > long_rows) if seg else None
 
 
 def near(found, want, limit, what=""):
@@ -169,14 +169,15 @@ def test_streams_refuse_what_does_not_fit(ops):
 
 def test_embedding_rows_in_copies(ops):
     rng = np.random.default_rng(4)
-    table = rng.normal(size=(50, 33))
     ids = [3, 49, 0, 3]
-    for dtype in DTYPES:
-        stored = dev(table, dtype)
-        found = ops.embed_rows(stored, ints(ids), scale=1.5, copies=3)
-        assert found.shape == (4, 3, 33)
-        for copy in range(3):
-            near(host(found[:, copy]), host(stored)[ids] * 1.5, 1e-6)
+    for width in (33, 2052):
+        table = rng.normal(size=(50, width))
+        for dtype in DTYPES:
+            stored = dev(table, dtype)
+            found = ops.embed_rows(stored, ints(ids), scale=1.5, copies=3)
+            assert found.shape == (4, 3, width)
+            for copy in range(3):
+                near(host(found[:, copy]), host(stored)[ids] * 1.5, 1e-6)
 
 
 # ---- the recurrence with a fixed decay ------------------------------------------------------------------------
